@@ -158,7 +158,11 @@ class NativeInferenceEngine:
             per_tok = 0  # cached numbers per token, over all layer runs
             for li in getattr(self.model, "layer_runs", range(len(self.model.layers))):
                 blk = self.model.layers[li]
-                if blk.kind == "attention":
+                if hasattr(blk, "paged"):  # blocks that name the mixer with a paged cache
+                    if blk.paged() is not None:
+                        g, d, v = blk.paged().cache_shape()
+                        per_tok += g * (d + v)
+                elif blk.kind == "attention":
                     g, d, v = blk.mix.cache_shape()
                     per_tok += g * (d + v)
                 elif blk.kind == "latent_attention":
@@ -177,8 +181,10 @@ class NativeInferenceEngine:
             num_pages = int(budget // per_page)
         else:
             num_pages = 256
-        num_pages = max(8, num_pages)
         max_running = int(cfg.max_running_requests or 256)
+        if hybrid and per_tok == 0:  # no paged cache at all: as many (empty) pages as the running requests can hold
+            num_pages = min(num_pages, max_running * ((ctx + PAGE_SIZE - 1) // PAGE_SIZE) + 1)
+        num_pages = max(8, num_pages)
         self.decode_steps = max(1, int(cfg.num_continuous_decode_steps))
         # models with recurrent layers: one state slot per request the scheduler may hold
         recurrent = hybrid and bool(getattr(mc, "has_recurrent_state", False))

@@ -871,14 +871,21 @@ class HybridModelRunner(ModelRunner):
         self.sandwich = bool(getattr(self.model, "sandwich", False))
         self.parallel = bool(getattr(self.model, "parallel", False))
         self.prepost = bool(getattr(self.model, "prepost", False))
-        self.keeps_positions = self.sandwich or self.parallel or self.prepost
+        self.post_add = bool(getattr(self.model, "post_add", False))
+        self.keeps_positions = self.sandwich or self.parallel or self.prepost or self.post_add
         # one cache / state per layer RUN: a layer that runs several times keeps every pass apart
         self.layer_runs = list(getattr(self.model, "layer_runs", range(len(self.model.layers))))
         self.kv, self.state = [], []
         tables: Dict[Any, torch.Tensor] = {}
         for li in self.layer_runs:
             blk = self.model.layers[li]
-            if blk.kind == "attention":
+            if hasattr(blk, "alloc"):  # blocks that name their own caches and states
+                if blk.paged() is not None:
+                    blk.paged().prepare(self.max_context + 1, tables, self.device)
+                kv, state = blk.alloc(self.num_pages, self.n_state_slots, self.dtype, self.device)
+                self.kv.append(kv)
+                self.state.append(state)
+            elif blk.kind == "attention":
                 G, D, V = blk.mix.cache_shape()
                 if hasattr(blk.mix, "prepare"):  # mixers that rotate by position
                     blk.mix.prepare(self.max_context + 1, tables, self.device)
@@ -916,7 +923,7 @@ class HybridModelRunner(ModelRunner):
         self._neg1 = torch.full((1,), -1, dtype=torch.int32, device=self.device)
 
     def _embed(self, ids: torch.Tensor, pos: torch.Tensor) -> torch.Tensor:
-        if self.sandwich or self.parallel or self.prepost:  # the fp32 stream starts in `_run_layers`, from the token ids
+        if self.keeps_positions:  # the fp32 stream starts in `_run_layers`, from the token ids
             return ids
         return self.model.embed_tokens(ids, pos)
 
@@ -925,8 +932,12 @@ class HybridModelRunner(ModelRunner):
         for c in self.kv:
             for t in (c if isinstance(c, tuple) else (c,)):
                 n += t.numel() * t.element_size() if t is not None else 0
-        for s in self.state:
-            if s is not None:
+        states = list(self.state)
+        while states:
+            s = states.pop()
+            if isinstance(s, (dict, tuple)):
+                states += list(s.values() if isinstance(s, dict) else s)
+            elif s is not None:
                 n += s.nbytes() if hasattr(s, "nbytes") and callable(s.nbytes) else s.numel() * s.element_size()
         return n
 
@@ -942,6 +953,8 @@ class HybridModelRunner(ModelRunner):
             return self._run_layers_parallel(xc, st)
         if self.prepost:
             return self._run_layers_prepost(xc, st)
+        if self.post_add:
+            return self._run_layers_post_add(xc, st)
         x32 = xc.float() if xc.dtype != torch.float32 else xc.clone()
         alpha, eps = float(cfg.postln_alpha), float(cfg.rms_norm_eps)
         trace = getattr(self, "layer_trace", None)
@@ -1034,6 +1047,32 @@ class HybridModelRunner(ModelRunner):
                 trace.append(x.clone())
         return x
 
+    def _run_layers_post_add(self, ids: torch.Tensor, st) -> torch.Tensor:
+        """Token ids -> fp32 residual stream after the last layer. One call closes a sublayer: the norm of its output, the
+        sum, and the convolution through which the next sublayer reads the stream."""
+        from ..ops import parallel_block as pb
+        from ..ops import sandwich as sw
+
+        model, eps = self.model, float(self.cfg.rms_norm_eps)
+        blocks = [model.layers[li] for li in self.layer_runs]
+        trace = getattr(self, "layer_trace", None)
+        rows = (st.cu_q, st.first_pos, st.state_slots)
+        x = pb.embed_scaled(ids, model.embed, float(self.cfg.embed_scale))
+        hc = sw.stream_conv(x, blocks[0].canon1, self.state[0]["canon1"], *rows, self.dtype)
+        for ri, blk in enumerate(blocks):
+            y = blk.mix_step(hc, st, self.kv[ri], self.state[ri]["mix"])
+            nxt = (blocks[ri + 1].canon1, self.state[ri + 1]["canon1"]) if ri + 1 < len(blocks) else None
+            if blk.mlp is not None:
+                x, hc = sw.norm_add_conv(x, y, blk.norm1, blk.norm1_bias, eps, (blk.canon2, self.state[ri]["canon2"]),
+                                         *rows)
+                y = blk.mlp(None, hc, None)
+                x, hc = sw.norm_add_conv(x, y, blk.norm2, blk.norm2_bias, eps, nxt, *rows)
+            else:
+                x, hc = sw.norm_add_conv(x, y, blk.norm1, blk.norm1_bias, eps, nxt, *rows)
+            if trace is not None:
+                trace.append(x.clone())
+        return x
+
     def _final_logits(self, h, residual, fp32: bool = False) -> torch.Tensor:
         from ..ops.post_norm import scaled_add_norm
 
@@ -1055,7 +1094,7 @@ class HybridModelRunner(ModelRunner):
             if want32:
                 return F.linear(x32, self.model.head_weight.float())
             return F.linear(xc, self.model.head_weight)
-        if self.sandwich:
+        if self.sandwich or self.post_add:
             from ..ops import sandwich as sw
 
             x32, xc = sw.layer_norm(h.contiguous(), self.model.norm, self.model.norm_bias,
@@ -1089,6 +1128,12 @@ class HybridModelRunner(ModelRunner):
         from ..ops import window_attention as wattn
 
         nsplit, ws = 1, None
+        if self.post_add:  # every mixer takes its own number of splits; they share one workspace
+            need = [blk.paged().workspace_floats(Bp) for blk in self.model.layers if blk.paged() is not None]
+            if need and self.device.type == "cuda":
+                ws = tuple(torch.empty(max(1, max(n[i] for n in need)), dtype=torch.float32, device=self.device)
+                           for i in range(2))
+            return nsplit, ws
         latent = [blk.mix for blk in self.model.layers if blk.kind == "latent_attention"]
         if self.prepost and self.device.type == "cuda":
             # mixers of several kinds share one workspace; each takes its own share of the step's splits

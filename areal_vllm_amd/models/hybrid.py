@@ -35,12 +35,25 @@ ff:         gated MLP, or routed gated experts chosen by sigmoid scores among th
             the scores as they are, plus a shared expert
 Embedding:  table row plus a learned vector per position
 
+The Gusolix design is the fifth member. A layer norm (weight and bias) sits on every sublayer's OUTPUT only:
+
+Layer:      x <- x + norm1(mixer(h(x)));  x <- x + norm2(ff(h(x))),  h(x) = x + conv(x) with a causal per-channel
+            convolution over time of each sublayer's own (the last inputs are state)
+Mixers:     grouped-query attention inside chunks of positions, RMS norm over all query (key) heads together, rotated
+            halves with frequencies stretched between two wavelength limits, the keys as projected as values;  selective
+            scan (Mamba) behind a short convolution;  or two mixers side by side on the same input: causal attention
+            without rotation whose softmax weights are mixed over the heads, and gated linear attention, summed with one
+            constant each
+ff:         gated MLP
+Embedding:  table row times a constant
+
 The mechanisms are separate modules with their constants as constructor arguments (``WindowAttentionMixer``,
 ``MLSTMMixer``, ``XieluMLP``, ``LatentAttentionMixer``, ``RoutedGLUExperts``, ``RotaryWindowAttentionMixer``,
 ``LightningMixer``, ``SquaredReluMLP``, ``RoutedSwiGLUExperts``, ``LogBiasWindowAttentionMixer``, ``GLAMixer``,
-``GatedMLP``); what they compute is documented with
-their kernels (``ops/window_attention.py``, ``ops/mlstm.py``, ``ops/post_norm.py``, ``ops/latent_attention.py``,
-``ops/sandwich.py``, ``ops/lightning.py``, ``ops/parallel_block.py``, ``ops/gla.py``, ``ops/depth_avg.py``). The modules hold parameters and know how to run ONE step on the tensors of a
+``GatedMLP``, ``RowNormAttentionMixer``, ``MixedAttentionMixer``, ``MambaMixer``, ``SideBySideMixer``); what they compute is
+documented with their kernels (``ops/window_attention.py``, ``ops/mlstm.py``, ``ops/post_norm.py``, ``ops/latent_attention.py``,
+``ops/sandwich.py``, ``ops/lightning.py``, ``ops/parallel_block.py``, ``ops/gla.py``, ``ops/depth_avg.py``,
+``ops/mixed_attention.py``, ``ops/mamba.py``). The modules hold parameters and know how to run ONE step on the tensors of a
 batch plan; paged caches, state slots and the loop over layers belong to the model runner
 (``inference/model_runner.py::HybridModelRunner``).
 """
@@ -57,6 +70,8 @@ from .. import ops
 from ..ops import depth_avg as davg
 from ..ops import gla as gla_ops
 from ..ops import lightning as lightning_ops
+from ..ops import mamba as mamba_ops
+from ..ops import mixed_attention as xattn
 from ..ops import mlstm as mlstm_ops
 from ..ops import parallel_block as pblock
 from ..ops import latent_attention as lattn
@@ -76,18 +91,20 @@ class HybridConfig(ModelConfig):
     design: str = "Kuzanex"
     # "post_norm": norm after every sum; "sandwich": layer norms before and after a sublayer, gated; "parallel": one
     # norm, mixer and feed-forward read it and are added together; "prepost": RMS norms before and after a sublayer,
-    # the normed output times `residual_mult` added to the stream, optionally averaged over depth
+    # the normed output times `residual_mult` added to the stream, optionally averaged over depth; "post_add": layer norm
+    # on a sublayer's output, which is added to the stream; sublayers read the stream through a short convolution
     block_style: str = "post_norm"
     residual_mult: float = 1.0  # factor on every normed sublayer output ("prepost" designs)
     depth_average: bool = False  # the stream that leaves a layer is a learned average of all streams so far
-    embed_scale: float = 1.0  # factor on the embedding rows ("parallel" designs)
+    embed_scale: float = 1.0  # factor on the embedding rows ("parallel" and "post_add" designs)
     loop: Optional[Dict[str, int]] = None  # layers start .. stop - 1 run `times` times in a row
-    canon_taps: int = 0  # taps of the causal convolution on a mixer's input (0: none)
+    canon_taps: int = 0  # taps of the causal convolution on a mixer's ("post_add": every sublayer's) input (0: none)
     bigram: Optional[Dict[str, int]] = None  # hashed-bigram embedding: buckets, mul_prev, mul_cur
 
     @property
     def has_recurrent_state(self) -> bool:
-        return (any(l["type"] in ("mlstm", "lightning", "gla") for l in self.layers) or self.canon_taps > 1
+        return (any(l["type"] in ("mlstm", "lightning", "gla", "mamba1", "parallel") for l in self.layers)
+                or self.canon_taps > 1
                 or self.bigram is not None)
 
     @property
@@ -106,6 +123,8 @@ class HybridConfig(ModelConfig):
             return self._n_params_parallel(with_embedding)
         if self.block_style == "prepost":
             return self._n_params_prepost(with_embedding)
+        if self.block_style == "post_add":
+            return self._n_params_post_add(with_embedding)
         W, n = self.hidden_size, 1
         for l in self.layers:
             m = l["mixer"]
@@ -185,7 +204,33 @@ class HybridConfig(ModelConfig):
             n += 2 * self.vocab_size * W + (self.max_position_embeddings * W if self.pos_embed == "learned" else 0)
         return n
 
+    def _n_params_post_add(self, with_embedding: bool) -> int:
+        W = self.hidden_size
+        n = 2 * W  # final norm
+        for l in self.layers:
+            m = l["mixer"]
+            if l["type"] == "attention":
+                H, G, D = m["heads"], m["kv_heads"], m["dim"]
+                n += (W + 1) * (H + G) * D + W * H * D
+            elif l["type"] == "mamba1":
+                I, R, N = m["inner"], m["dt_rank"], m["state"]
+                n += W * 2 * I + I * (m["conv"] + 1) + (R + 2 * N) * I + I * R + I + I * N + I + W * I
+            else:
+                a, b = m["left"], m["right"]
+                H, G, D, V = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+                n += (W + 1) * (H + G) * D + W * G * V + H * H + W * H * V
+                H, D, V, r = b["heads"], b["dim"], b["vdim"], b["decay_rank"]
+                n += W * (2 * H * D + 2 * H * V + r) + r * H * D + H * D + V + W * H * V
+            n += 2 * W + W * self.canon_taps
+            if l.get("mlp"):
+                n += 2 * W + W * self.canon_taps + 3 * W * l["mlp"]["ff"]
+        return n + (2 * self.vocab_size * W if with_embedding else 0)
+
     def to_hf_dict(self) -> Dict[str, Any]:
+        if self.block_style == "post_add":  # right-hand mixers carry `decay_rank` (a checkpoint's shapes give it too)
+            return {"architecture": self.design, "canon": {"taps": self.canon_taps},
+                    "embedding": {"scale": self.embed_scale}, "layers": json.loads(json.dumps(self.layers)),
+                    "norm": {"eps": self.rms_norm_eps}, "vocab": self.vocab_size, "width": self.hidden_size}
         if self.block_style == "prepost":
             layers = json.loads(json.dumps(self.layers))  # gla entries carry `decay_rank` (a checkpoint's shapes give it too)
             return {"architecture": self.design, "layers": layers, "max_positions": self.max_position_embeddings,
@@ -369,18 +414,76 @@ def zusotar_config_from_dir(path: str) -> HybridConfig:
     """config.json plus one look at the checkpoint's tensor shapes (the rank of every decay projection)."""
     with open(os.path.join(path, "config.json")) as f:
         d = json.load(f)
-    ranks: Dict[int, int] = {}
-    want = {f"l{i}.mix.a1": i for i, l in enumerate(d["layers"]) if l["type"] == "gla"}
-    if want:
-        from safetensors import safe_open
+    return zusotar_config(d, _first_sizes(path, {f"l{i}.mix.a1": i for i, l in enumerate(d["layers"]) if l["type"] == "gla"}))
 
-        for fn in sorted(os.listdir(path)):
-            if fn.endswith(".safetensors"):
-                with safe_open(os.path.join(path, fn), framework="pt") as f:
-                    for name in f.keys():
-                        if name in want:
-                            ranks[want[name]] = int(f.get_slice(name).get_shape()[0])
-    return zusotar_config(d, ranks)
+
+def _first_sizes(path: str, want: Dict[str, int]) -> Dict[int, int]:
+    """`want`: tensor name -> key. {key: size of the tensor's first axis} for those that the checkpoint in `path` holds."""
+    from safetensors import safe_open
+
+    out: Dict[int, int] = {}
+    for fn in sorted(os.listdir(path)) if want else []:
+        if fn.endswith(".safetensors"):
+            with safe_open(os.path.join(path, fn), framework="pt") as f:
+                for name in f.keys():
+                    if name in want:
+                        out[want[name]] = int(f.get_slice(name).get_shape()[0])
+    return out
+
+
+def gusolix_config(d: Dict[str, Any], decay_ranks: Optional[Dict[int, int]] = None) -> HybridConfig:
+    """config.json of a Gusolix checkpoint -> HybridConfig. Every size and constant is taken from it; the rank of a decay
+    projection is a tensor's shape (`decay_ranks`: layer index -> rank, or `decay_rank` in the right-hand mixer's entry)."""
+    layers = []
+
+    def heads_fit(i, m):
+        m.setdefault("kv_heads", m["heads"])
+        m.setdefault("vdim", m["dim"])
+        m.setdefault("scale", float(m["dim"]) ** -0.5)
+        if int(m["heads"]) % int(m["kv_heads"]):
+            raise ValueError(f"layer {i}: heads is not a multiple of kv_heads")
+
+    for i, l in enumerate(d["layers"]):
+        mlp = l.get("mlp")
+        if mlp is not None and mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+        m = json.loads(json.dumps(l["mixer"]))
+        if l["type"] == "attention":
+            heads_fit(i, m)
+            if int(m["vdim"]) != int(m["dim"]):
+                raise ValueError(f"layer {i}: keys that are values have one size")
+            rot = m.get("rot")
+            if rot and (int(rot["dims"]) % 2 or int(rot["dims"]) > int(m["dim"])):
+                raise ValueError(f"layer {i}: the rotated part is an even number of at most dim coordinates")
+        elif l["type"] == "parallel":
+            heads_fit(i, m["left"])
+            r = m["right"]
+            r.setdefault("vdim", r["dim"])
+            if decay_ranks and i in decay_ranks:
+                r["decay_rank"] = int(decay_ranks[i])
+            if "decay_rank" not in r:
+                raise ValueError(f"layer {i}: the rank of the decay projection is not known")
+        elif l["type"] != "mamba1":
+            raise ValueError(f"layer {i}: unknown mixer type {l['type']!r}")
+        layers.append({"type": l["type"], "mixer": m, "mlp": json.loads(json.dumps(mlp)) if mlp is not None else None})
+    att = next((l["mixer"].get("left", l["mixer"]) for l in layers if l["type"] != "mamba1"), None)
+    return HybridConfig(
+        family="gusolix", design="Gusolix", block_style="post_add", vocab_size=int(d["vocab"]),
+        hidden_size=int(d["width"]), n_layers=len(layers), n_q_heads=int(att["heads"]) if att else 1,
+        n_kv_heads=int(att["kv_heads"]) if att else 1, head_dim=int(att["dim"]) if att else 1,
+        intermediate_size=max([l["mlp"]["ff"] for l in layers if l["mlp"]] or [0]), rms_norm_eps=float(d["norm"]["eps"]),
+        max_position_embeddings=int(d.get("max_positions", 1 << 17)), tie_word_embeddings=False, qkv_bias=False,
+        pos_embed="none", norm_type="layer", layers=layers, canon_taps=int((d.get("canon") or {}).get("taps", 0)),
+        embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)), eos_token_id=d.get("eos_token_id"),
+        pad_token_id=d.get("pad_token_id"))
+
+
+def gusolix_config_from_dir(path: str) -> HybridConfig:
+    """config.json plus one look at the checkpoint's tensor shapes (the rank of every decay projection)."""
+    with open(os.path.join(path, "config.json")) as f:
+        d = json.load(f)
+    return gusolix_config(d, _first_sizes(path, {f"l{i}.mix.right.a1": i for i, l in enumerate(d["layers"])
+                                                 if l["type"] == "parallel"}))
 
 
 class StepTensors:
@@ -631,8 +734,7 @@ class RotaryWindowAttentionMixer(nn.Module):
         if not self.rot:
             return
         sc = self.rot.get("scaling") or None
-        key = ("rot", float(self.rot["base"]), int(self.rot["dims"]), int(n_pos),
-               tuple(float(sc[k]) for k in ("factor", "original", "fast", "slow")) if sc else None)
+        key = wattn.table_key(self.rot, n_pos)
         if key not in tables:
             tables[key] = wattn.rotation_table(float(self.rot["base"]), int(self.rot["dims"]), int(n_pos), device, sc)
         self.table = tables[key]
@@ -819,6 +921,15 @@ class LogBiasWindowAttentionMixer(nn.Module):
         return F.linear(o.view(T, self.H * self.V), self.o)
 
 
+def linear32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """x W^T in fp32: operands in the compute dtype, fp32 accumulation AND fp32 results."""
+    if x.dtype == torch.float32:
+        return F.linear(x, weight)
+    if x.is_cuda:
+        return torch.mm(x, weight.t(), out_dtype=torch.float32)
+    return F.linear(x.float(), weight.float())
+
+
 class GLAMixer(nn.Module):
     """Gated linear attention (``ops/gla.py``): q | k | v | output gate | the low-rank input of the decay logits come
     out of ONE projection; the decay logits are the low-rank product plus a bias, formed in fp32; per key channel the
@@ -826,33 +937,203 @@ class GLAMixer(nn.Module):
     gate on the read-out."""
 
     def __init__(self, width: int, heads: int, dim: int, vdim: int, tau: float, decay_rank: int, q_scale: float,
-                 eps: float, dtype, device):
+                 eps: float, dtype, device, own_proj: bool = True):
+        """`own_proj` False: the in- and out-projections belong to a module that holds this one (`run`)."""
         super().__init__()
         self.H, self.D, self.V, self.rank = heads, dim, vdim, int(decay_rank)
         self.tau, self.q_scale, self.eps = float(tau), float(q_scale), float(eps)
         self.n_main = 2 * heads * dim + 2 * heads * vdim
-        self.proj = nn.Parameter(torch.empty(self.n_main + self.rank, width, dtype=dtype, device=device))
+        self.proj = (nn.Parameter(torch.empty(self.n_main + self.rank, width, dtype=dtype, device=device))
+                     if own_proj else None)
         self.a2 = nn.Parameter(torch.empty(heads * dim, self.rank, dtype=dtype, device=device))
         self.a2_bias = nn.Parameter(torch.zeros(heads * dim, dtype=dtype, device=device))
         self.norm = nn.Parameter(torch.ones(vdim, dtype=dtype, device=device))
-        self.o = nn.Parameter(torch.empty(width, heads * vdim, dtype=dtype, device=device))
+        self.o = nn.Parameter(torch.empty(width, heads * vdim, dtype=dtype, device=device)) if own_proj else None
 
     def state_shape(self):
         return self.H, self.D, self.V
 
     def step(self, hc: torch.Tensor, st: StepTensors, state: torch.Tensor) -> torch.Tensor:
+        return F.linear(self.run(F.linear(hc, self.proj), st, state), self.o)
+
+    def run(self, proj: torch.Tensor, st: StepTensors, state: torch.Tensor, out: Optional[torch.Tensor] = None,
+            out_scale: float = 1.0) -> torch.Tensor:
+        """proj [T, n_main + rank] (a view with unit column stride) -> what the output projection reads, times
+        `out_scale`, into `out` [T, H V] when given."""
         H, D, V = self.H, self.D, self.V
-        proj = F.linear(hc, self.proj)
-        low = proj[:, self.n_main:]
-        if low.dtype == torch.float32:
-            z = F.linear(low, self.a2)
-        elif low.is_cuda:  # 16-bit operands, fp32 accumulation AND fp32 logits
-            z = torch.mm(low, self.a2.t(), out_dtype=torch.float32)
-        else:
-            z = F.linear(low.float(), self.a2.float())
+        z = linear32(proj[:, self.n_main:self.n_main + self.rank], self.a2)
         o = gla_ops.gla_scan(proj, 0, H * D, 2 * H * D, z, self.a2_bias, self.tau, self.q_scale, st.cu_q, st.first_pos,
                              st.state_slots, state, max_q=st.max_q)
-        y = gla_ops.gla_out(o, proj[:, 2 * H * D + H * V:self.n_main], self.norm, self.eps)
+        return gla_ops.gla_out(o, proj[:, 2 * H * D + H * V:self.n_main], self.norm, self.eps, out, out_scale)
+
+
+class RowNormAttentionMixer(nn.Module):
+    """Grouped-query attention whose queries (keys) are RMS-normed over all heads together, then rotated on their first
+    coordinates (i with i + dims/2, optionally stretched frequencies): a sliding window, chunks of positions, or every
+    earlier key; ordinary softmax. `key_values`: the keys as projected are the values (no value projection)."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, window: int, chunk: int,
+                 rot: Optional[Dict[str, Any]], key_values: bool, eps: float, dtype, device):
+        super().__init__()
+        assert heads % kv_heads == 0 and (vdim == dim or not key_values)
+        self.H, self.G, self.D, self.V, self.eps = heads, kv_heads, dim, vdim, float(eps)
+        self.shape = wattn.ScoreShape(scale=float(scale), window=int(window), chunk=int(chunk))
+        self.rot = dict(rot) if rot else None
+        self.v_off = heads * dim if key_values else (heads + kv_heads) * dim
+        self.proj = nn.Parameter(torch.empty(self.v_off + kv_heads * vdim, width, dtype=dtype, device=device))
+        self.q_norm = nn.Parameter(torch.ones(heads * dim, dtype=dtype, device=device))
+        self.k_norm = nn.Parameter(torch.ones(kv_heads * dim, dtype=dtype, device=device))
+        self.o = nn.Parameter(torch.empty(width, heads * vdim, dtype=dtype, device=device))
+        self.table: Optional[torch.Tensor] = None
+        self.max_context = 1 << 30
+        self.standard = False  # the cache is in the engine's standard layout (`alloc_cache`)
+
+    def cache_shape(self):
+        return self.G, self.D, self.V
+
+    def alloc_cache(self, num_pages: int, dtype, device):
+        """Paged K / V of this layer: the engine's standard layout (and its flash / paged-decode kernels) for bf16
+        heads of 128 on the GPU, otherwise token-major pages of any key and value size."""
+        from ..ops.attention import alloc_kv_cache
+
+        self.standard = wattn.standard_layout_ok(self.D, self.V, dtype, device) and self.H // self.G <= 16
+        if self.standard:
+            return alloc_kv_cache(num_pages, self.G, self.D, dtype, device)
+        return wattn.alloc_window_cache(num_pages, self.G, self.D, self.V, dtype, device)
+
+    def prepare(self, n_pos: int, tables: Dict[Any, torch.Tensor], device):
+        self.max_context = int(n_pos) - 1
+        if self.rot:
+            key = wattn.table_key(self.rot, n_pos)
+            if key not in tables:
+                tables[key] = wattn.rotation_table(float(self.rot["base"]), int(self.rot["dims"]), int(n_pos), device,
+                                                   self.rot.get("scaling") or None)
+            self.table = tables[key]
+
+    def decode_splits(self, batch: int, max_context: int) -> int:
+        s = self.shape
+        if self.standard:
+            from ..ops.attention import decode_num_splits
+
+            return decode_num_splits(batch, self.G, wattn.visible_span(s.window, max_context, s.keep_first, s.chunk))
+        return wattn.decode_splits(batch, s.window, max_context, s.keep_first, s.chunk)
+
+    def workspace_floats(self, batch: int):
+        n = self.decode_splits(batch, self.max_context)
+        return batch * n * self.H * self.V, batch * n * self.H * 2
+
+    def step(self, hc: torch.Tensor, st: StepTensors, cache) -> torch.Tensor:
+        kc, vc = cache
+        T = hc.shape[0]
+        proj = F.linear(hc, self.proj)
+        q = wattn.qk_rows_norm_cache_write(proj, self.v_off, self.q_norm, self.k_norm, st.positions, self.table, st.slots,
+                                           kc, vc, self.H, self.eps, v_transposed=self.standard)
+        nsplit = self.decode_splits(T, self.max_context) if st.max_q == 1 else 1
+        if self.standard:
+            o = wattn.window_attention_standard(q, kc, vc, st.block_tables, st.cu_q, st.cu_k, st.ctx_len, st.max_q,
+                                                self.shape, nsplit=nsplit, workspace=st.workspace)
+        else:
+            o = wattn.window_attention(q, kc, vc, st.block_tables, st.cu_q, st.ctx_len, st.max_q, self.shape, None,
+                                       nsplit=nsplit, workspace=st.workspace)
+        return F.linear(o.view(T, self.H * self.V), self.o)
+
+
+class MixedAttentionMixer(nn.Module):
+    """Causal grouped-query attention without rotation whose softmax weights are mixed over the heads (``ops/
+    mixed_attention.py``); queries and keys are RMS-normed over all heads together. q | k | v are the first columns of the
+    projection that the module holding this one hands in."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, eps: float, dtype, device):
+        super().__init__()
+        assert heads % kv_heads == 0
+        self.H, self.G, self.D, self.V = heads, kv_heads, dim, vdim
+        self.scale, self.eps = float(scale), float(eps)
+        self.q_norm = nn.Parameter(torch.ones(heads * dim, dtype=dtype, device=device))
+        self.k_norm = nn.Parameter(torch.ones(kv_heads * dim, dtype=dtype, device=device))
+        self.talk = nn.Parameter(torch.eye(heads, dtype=dtype, device=device))
+        self.max_context = 1 << 30
+
+    def in_rows(self) -> int:
+        return (self.H + self.G) * self.D + self.G * self.V
+
+    def out_cols(self) -> int:
+        return self.H * self.V
+
+    def cache_shape(self):
+        return self.G, self.D, self.V
+
+    def alloc_cache(self, num_pages: int, dtype, device):
+        return xattn.alloc_mixed_cache(num_pages, self.G, self.D, self.V, dtype, device)
+
+    def prepare(self, n_pos: int, tables, device):
+        self.max_context = int(n_pos) - 1
+
+    def workspace_floats(self, batch: int):
+        return xattn.workspace_floats(batch, xattn.decode_splits(batch, self.max_context), self.H, self.V)
+
+    def run(self, proj: torch.Tensor, st: StepTensors, cache, out: torch.Tensor, out_scale: float) -> torch.Tensor:
+        kc, vc = cache
+        q = wattn.qk_rows_norm_cache_write(proj, (self.H + self.G) * self.D, self.q_norm, self.k_norm, None, None, st.slots,
+                                           kc, vc, self.H, self.eps, v_transposed=True)
+        nsplit = xattn.decode_splits(proj.shape[0], self.max_context) if st.max_q == 1 else 1
+        return xattn.mixed_attention(q, kc, vc, st.block_tables, st.cu_q, st.ctx_len, st.max_q, self.scale, self.talk, out,
+                                     out_scale, nsplit, st.workspace)
+
+
+class SideBySideMixer(nn.Module):
+    """Two mixers on the same input, left_scale * left + right_scale * right: attention with mixed weights on the left,
+    gated linear attention on the right. ONE in-projection yields both mixers' operands; both write what their output
+    projections read (times their constant) side by side, so ONE out-projection sums them."""
+
+    def __init__(self, width: int, left: MixedAttentionMixer, right: GLAMixer, left_scale: float, right_scale: float, dtype,
+                 device):
+        super().__init__()
+        self.left, self.right = left, right
+        self.left_scale, self.right_scale = float(left_scale), float(right_scale)
+        self.n_left, self.c_left = left.in_rows(), left.out_cols()
+        self.proj = nn.Parameter(torch.empty(self.n_left + right.n_main + right.rank, width, dtype=dtype, device=device))
+        self.o = nn.Parameter(torch.empty(width, self.c_left + right.H * right.V, dtype=dtype, device=device))
+
+    def step(self, hc: torch.Tensor, st: StepTensors, cache, state: torch.Tensor) -> torch.Tensor:
+        proj = F.linear(hc, self.proj)
+        both = torch.empty(hc.shape[0], self.o.shape[1], dtype=hc.dtype, device=hc.device)
+        self.left.run(proj, st, cache, both[:, :self.c_left], self.left_scale)
+        self.right.run(proj[:, self.n_left:], st, state, both[:, self.c_left:], self.right_scale)
+        return F.linear(both, self.o)
+
+
+class MambaMixer(nn.Module):
+    """Selective scan (``ops/mamba.py``): x | z come out of one projection, x passes a short causal convolution with bias
+    and SiLU; step sizes (through a low-rank projection, softplus), read-in and read-out weights come from x; the read-out
+    is gated by SiLU(z)."""
+
+    def __init__(self, width: int, inner: int, n_state: int, dt_rank: int, taps: int, dtype, device):
+        super().__init__()
+        self.I, self.N, self.rank, self.taps = inner, n_state, dt_rank, taps
+
+        def par(*shape):
+            return nn.Parameter(torch.zeros(*shape, dtype=dtype, device=device))
+
+        self.proj = par(2 * inner, width)
+        self.conv, self.conv_bias = par(inner, taps), par(inner)
+        self.x_proj = par(dt_rank + 2 * n_state, inner)
+        self.dt, self.dt_bias = par(inner, dt_rank), par(inner)
+        self.a_log, self.d_skip = par(inner, n_state), par(inner)
+        self.o = par(width, inner)
+
+    def alloc_state(self, n_slots: int, device):
+        """(scan state, the convolution's last inputs or None), both fp32 per request slot."""
+        hist = (torch.zeros(n_slots, self.taps - 1, self.I, dtype=torch.float32, device=device) if self.taps > 1 else None)
+        return mamba_ops.alloc_state(n_slots, self.I, self.N, device), hist
+
+    def step(self, hc: torch.Tensor, st: StepTensors, state) -> torch.Tensor:
+        S, hist = state
+        xz = F.linear(hc, self.proj)
+        x = sandwich.conv_silu(xz[:, :self.I], self.conv, self.conv_bias, hist, st.cu_q, st.first_pos, st.state_slots)
+        low = F.linear(x, self.x_proj)
+        r = linear32(low[:, :self.rank], self.dt)
+        y = mamba_ops.selective_scan(x, r, self.dt_bias, self.a_log, low[:, self.rank:], self.d_skip, xz[:, self.I:],
+                                     st.cu_q, st.first_pos, st.state_slots, S, max_q=st.max_q)
         return F.linear(y, self.o)
 
 
@@ -949,6 +1230,101 @@ class PrePostBlock(nn.Module):
                 sf = e.shared_ff
                 out[q + "shared.gate"], out[q + "shared.up"] = e.shared_in.data[:sf], e.shared_in.data[sf:]
                 out[q + "shared.down"] = e.shared_down.data
+        return out
+
+
+class PostAddBlock(nn.Module):
+    """A layer with one layer norm on each sublayer's output: x <- x + norm(sublayer(x + conv(x))), for the mixer and (when
+    the layer has one) the feed-forward, the convolution being each sublayer's own."""
+
+    def __init__(self, cfg: HybridConfig, spec: Dict[str, Any], dtype, device):
+        super().__init__()
+        W, m, eps = cfg.hidden_size, spec["mixer"], cfg.rms_norm_eps
+        self.kind = spec["type"]
+        if self.kind == "attention":
+            self.mix = RowNormAttentionMixer(
+                W, int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), float(m["scale"]), 0,
+                int((m.get("mask") or {}).get("size") or 0), m.get("rot"), True, eps, dtype, device)
+        elif self.kind == "mamba1":
+            self.mix = MambaMixer(W, int(m["inner"]), int(m["state"]), int(m["dt_rank"]), int(m["conv"]), dtype, device)
+        else:
+            a, b = m["left"], m["right"]
+            left = MixedAttentionMixer(int(a["heads"]), int(a["kv_heads"]), int(a["dim"]), int(a["vdim"]),
+                                       float(a["scale"]), eps, dtype, device)
+            right = GLAMixer(W, int(b["heads"]), int(b["dim"]), int(b["vdim"]), float(b["tau"]), int(b["decay_rank"]),
+                             float(b["dim"]) ** -0.5, eps, dtype, device, own_proj=False)
+            self.mix = SideBySideMixer(W, left, right, float(m["left_scale"]), float(m["right_scale"]), dtype, device)
+
+        def vec(one=False):
+            return nn.Parameter((torch.ones if one else torch.zeros)(W, dtype=dtype, device=device))
+
+        def taps():
+            return (nn.Parameter(torch.zeros(W, cfg.canon_taps, dtype=dtype, device=device)) if cfg.canon_taps > 0
+                    else None)
+
+        self.norm1, self.norm1_bias, self.canon1 = vec(True), vec(), taps()
+        self.mlp = self.canon2 = None
+        if spec.get("mlp"):
+            self.norm2, self.norm2_bias, self.canon2 = vec(True), vec(), taps()
+            self.mlp = GatedMLP(W, int(spec["mlp"]["ff"]), "silu", dtype, device)
+
+    def paged(self):
+        """The mixer whose keys and values live in the paged cache, or None."""
+        return {"attention": self.mix, "parallel": getattr(self.mix, "left", None)}.get(self.kind)
+
+    def alloc(self, num_pages: int, n_slots: int, dtype, device):
+        """(paged cache or None, fp32 state per request slot: the mixer's and the two convolutions' last inputs)."""
+        cache = self.paged().alloc_cache(num_pages, dtype, device) if self.paged() is not None else None
+        if self.kind == "mamba1":
+            state = self.mix.alloc_state(n_slots, device)
+        elif self.kind == "parallel":
+            state = gla_ops.alloc_state(n_slots, *self.mix.right.state_shape(), device)
+        else:
+            state = None
+
+        def hist(w):
+            return (torch.zeros(n_slots, w.shape[1] - 1, w.shape[0], dtype=torch.float32, device=device)
+                    if w is not None and w.shape[1] > 1 else None)
+
+        return cache, {"mix": state, "canon1": hist(self.canon1), "canon2": hist(self.canon2)}
+
+    def mix_step(self, hc: torch.Tensor, st: StepTensors, cache, state) -> torch.Tensor:
+        if self.kind == "attention":
+            return self.mix.step(hc, st, cache)
+        if self.kind == "mamba1":
+            return self.mix.step(hc, st, state)
+        return self.mix.step(hc, st, cache, state)
+
+    def checkpoint_tensors(self, p: str) -> Dict[str, torch.Tensor]:
+        m = self.mix
+        out = {p + "norm1": self.norm1.data, p + "norm1.b": self.norm1_bias.data}
+        if self.canon1 is not None:
+            out[p + "canon1"] = self.canon1.data
+        w = m.proj.data
+        if self.kind == "attention":
+            a = m.H * m.D
+            out.update({p + "mix.q": w[:a], p + "mix.k": w[a:], p + "mix.q.norm": m.q_norm.data,
+                        p + "mix.k.norm": m.k_norm.data, p + "mix.o": m.o.data})
+        elif self.kind == "mamba1":
+            out.update({p + "mix.in": w, p + "mix.conv": m.conv.data, p + "mix.conv.b": m.conv_bias.data,
+                        p + "mix.x": m.x_proj.data, p + "mix.dt": m.dt.data, p + "mix.dt.b": m.dt_bias.data,
+                        p + "mix.A_log": m.a_log.data, p + "mix.D": m.d_skip.data, p + "mix.o": m.o.data})
+        else:
+            l, r, q = m.left, m.right, p + "mix.left."
+            a, b = l.H * l.D, (l.H + l.G) * l.D
+            out.update({q + "q": w[:a], q + "k": w[a:b], q + "v": w[b:m.n_left], q + "q.norm": l.q_norm.data,
+                        q + "k.norm": l.k_norm.data, q + "talk": l.talk.data, q + "o": m.o.data[:, :m.c_left]})
+            q, w = p + "mix.right.", w[m.n_left:]
+            a, b, c = r.H * r.D, 2 * r.H * r.D, 2 * r.H * r.D + r.H * r.V
+            out.update({q + "q": w[:a], q + "k": w[a:b], q + "v": w[b:c], q + "g": w[c:r.n_main], q + "a1": w[r.n_main:],
+                        q + "a2": r.a2.data, q + "a2.b": r.a2_bias.data, q + "norm": r.norm.data,
+                        q + "o": m.o.data[:, m.c_left:]})
+        if self.mlp is not None:
+            e, q = self.mlp, p + "mlp."
+            out.update({p + "norm2": self.norm2.data, p + "norm2.b": self.norm2_bias.data,
+                        q + "gate": e.gate_up.data[:e.ff], q + "up": e.gate_up.data[e.ff:], q + "down": e.down.data})
+            if self.canon2 is not None:
+                out[p + "canon2"] = self.canon2.data
         return out
 
 
@@ -1146,8 +1522,13 @@ class HybridDecoder(nn.Module):
         self.sandwich = cfg.block_style == "sandwich"
         self.parallel = cfg.block_style == "parallel"
         self.prepost = cfg.block_style == "prepost"
+        self.post_add = cfg.block_style == "post_add"
         self.layer_runs = cfg.layer_runs
-        if self.prepost:
+        if self.post_add:
+            self.layers = nn.ModuleList([PostAddBlock(cfg, spec, dtype, device) for spec in cfg.layers])
+            self.norm = nn.Parameter(torch.ones(cfg.hidden_size, dtype=dtype, device=device))
+            self.norm_bias = nn.Parameter(torch.zeros(cfg.hidden_size, dtype=dtype, device=device))
+        elif self.prepost:
             if cfg.loop:
                 raise NotImplementedError("depth-averaged layers run once each")
             W = cfg.hidden_size
@@ -1200,7 +1581,29 @@ class HybridDecoder(nn.Module):
         W = self.cfg.hidden_size
         for n, p in self.named_parameters():
             leaf = n.rsplit(".", 1)[-1]
-            if self.prepost:
+            if self.post_add:
+                if leaf == "talk":
+                    p.data.copy_(torch.eye(p.shape[0]) + 0.3 * torch.randn(p.shape, generator=g))
+                elif leaf == "a_log":
+                    p.data.copy_(torch.log(torch.arange(1, p.shape[1] + 1).float()).expand(p.shape)
+                                 + 0.1 * torch.randn(p.shape, generator=g))
+                elif leaf == "a2_bias":
+                    p.data.copy_(1.0 + torch.randn(p.shape, generator=g))
+                elif leaf == "dt_bias":  # step sizes of about 0.01 .. 0.3
+                    p.data.copy_(-4.5 + 3.0 * torch.rand(p.shape, generator=g))
+                elif leaf in ("canon1", "canon2"):
+                    p.data.copy_(0.3 * torch.randn(p.shape, generator=g))
+                elif leaf == "conv":
+                    p.data.copy_(torch.randn(p.shape, generator=g) / (p.shape[1] ** 0.5))
+                elif leaf.endswith("bias"):
+                    p.data.copy_(0.1 * torch.randn(p.shape, generator=g))
+                elif p.dim() == 1:  # norm weights, the scan's direct path
+                    p.data.copy_(1.0 + 0.1 * torch.randn(p.shape, generator=g))
+                elif leaf == "embed":  # rows of about unit RMS once the embedding's factor is applied
+                    p.data.copy_(torch.randn(p.shape, generator=g) / max(self.cfg.embed_scale, 1e-6))
+                else:
+                    p.data.copy_(torch.randn(p.shape, generator=g) / (p.shape[-1] ** 0.5))
+            elif self.prepost:
                 if leaf == "dwa":  # mostly the layer's own result, a little of every earlier stream
                     w = 0.3 * torch.rand(p.shape, generator=g) / p.shape[0]
                     w[-1] = 1.0 - w[:-1].sum()
@@ -1274,6 +1677,12 @@ class HybridDecoder(nn.Module):
     # ------------------------------------------------------------------------- checkpoint names
     def checkpoint_tensors(self) -> Dict[str, torch.Tensor]:
         """Checkpoint name -> the view of this model's parameters that holds it (fused projections are sliced)."""
+        if self.post_add:
+            out = {"embed": self.embed.data, "head": self.head.data, "final.norm": self.norm.data,
+                   "final.norm.b": self.norm_bias.data}
+            for i, blk in enumerate(self.layers):
+                out.update(blk.checkpoint_tensors(f"l{i}."))
+            return out
         if self.prepost:
             out = {"embed": self.embed.data, "head": self.head.data, "final.norm": self.norm.data}
             if self.pos is not None:

@@ -4,7 +4,8 @@
     x       <- x + s * LN'(y * sigmoid(r))             y: the sublayer's output, r: gate logits (a projection of h),
                                                        s: one scale per channel ("layer scale")
     conv(h)_t = sum_j w[:, j] * h_(t - taps + 1 + j)   causal per-channel convolution over time; the last taps - 1
-                                                       inputs of every sequence live in a state slot
+                                                       inputs of every sequence live in a state slot (`conv_silu`: the
+                                                       convolution with a bias and SiLU instead of the sum with h)
     x_0      = LN(E[tok] + B[(prev * a + tok * b) mod n])   token plus hashed-bigram embedding (row n of B for a
                                                        sequence's first token); the previous token lives in a slot
 
@@ -100,29 +101,74 @@ def canon_conv(h: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tens
                                          L.ptr(state_slots), L.ptr(out), L.c_int(B), L.c_int(T), L.c_int(W),
                                          L.c_int(taps), L.c_int(L.dtype_flag(weight)), L.stream_ptr()), "canon_conv")
         return out
-    out = torch.empty_like(h)
+    conv = _causal_conv_cpu(h, weight, state, cu_q, first_pos, state_slots)
+    out = h + conv
+    return out if dtype == torch.float32 else out.to(dtype)
+
+
+def stream_conv(x: torch.Tensor, weight: Optional[torch.Tensor], state: Optional[torch.Tensor], cu_q: torch.Tensor,
+                first_pos: torch.Tensor, state_slots: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+    """`canon_conv` of the stream itself; without a weight the stream in `dtype`."""
+    if weight is None:
+        return x if dtype == torch.float32 else x.to(dtype)
+    return canon_conv(x, weight, state, cu_q, first_pos, state_slots, dtype)
+
+
+def norm_add_conv(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, eps: float,
+                  conv: Optional[Tuple[Optional[torch.Tensor], Optional[torch.Tensor]]], cu_q: torch.Tensor,
+                  first_pos: torch.Tensor, state_slots: torch.Tensor) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """x + LN(y; weight, bias) on the fp32 stream x [T, W] (y [T, W] in the compute dtype; x itself may be overwritten) and,
+    with `conv` = (weight, state), `stream_conv` of the sum in y's dtype. Returns (new stream, convolved stream or None)."""
+    x, _, _ = gated_norm_add(x, y, None, weight, bias, None, eps)
+    return x, (None if conv is None else stream_conv(x, conv[0], conv[1], cu_q, first_pos, state_slots, y.dtype))
+
+
+def conv_silu(h: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
+              cu_q: torch.Tensor, first_pos: torch.Tensor, state_slots: torch.Tensor) -> torch.Tensor:
+    """silu(conv(h) + bias) of h [T, W] in the compute dtype (a view with unit column stride), contiguous; weight, state
+    and history as in `canon_conv` (the state is fp32 and holds the inputs h exactly)."""
+    T, W = h.shape
+    taps = weight.shape[1]
+    assert weight.shape[0] == W and weight.is_contiguous() and h.stride(1) == 1
+    assert taps == 1 or (state is not None and state.shape[1:] == (taps - 1, W) and state.dtype == torch.float32)
+    if L.use_hip(h):
+        assert weight.dtype == h.dtype and (bias is None or (bias.dtype == h.dtype and bias.numel() == W))
+        assert cu_q.dtype == torch.int32 and first_pos.dtype == torch.int32 and state_slots.dtype == torch.int32
+        out = torch.empty(T, W, dtype=h.dtype, device=h.device)
+        L.check(L.lib().areal_conv_silu(L.ptr(h), L.c_int64(h.stride(0)), L.ptr(weight), L.ptr(bias), L.ptr(state),
+                                        L.ptr(cu_q), L.ptr(first_pos), L.ptr(state_slots), L.ptr(out),
+                                        L.c_int(cu_q.numel() - 1), L.c_int(T), L.c_int(W), L.c_int(taps),
+                                        L.c_int(L.dtype_flag(h)), L.stream_ptr()), "conv_silu")
+        return out
+    a = _causal_conv_cpu(h.float(), weight, state, cu_q, first_pos, state_slots)
+    if bias is not None:
+        a = a + bias.float()
+    return (a * torch.sigmoid(a)).to(h.dtype)
+
+
+def _causal_conv_cpu(h, weight, state, cu_q, first_pos, state_slots):
+    """The convolution alone, fp32 (zero for padding rows); rewrites the rows' state slots."""
+    out = torch.zeros_like(h)
     w = weight.float()
-    cq, fp, ss = cu_q.tolist(), first_pos.tolist(), state_slots.tolist()
+    taps = w.shape[1]
     K = taps - 1
-    for b in range(B):
+    cq, fp, ss = cu_q.tolist(), first_pos.tolist(), state_slots.tolist()
+    for b in range(len(cq) - 1):
         lo, hi = cq[b], cq[b + 1]
         if hi <= lo or ss[b] < 0:
-            out[lo:hi] = h[lo:hi]
             continue
         if K == 0:
-            out[lo:hi] = h[lo:hi] * (1.0 + w[:, 0])
+            out[lo:hi] = h[lo:hi] * w[:, 0]
             continue
         hist = state[ss[b]].clone()  # [K, W], oldest first
         if fp[b] < K:  # before the sequence's start there is nothing
             hist[:K - fp[b]] = 0
         ext = torch.cat([hist, h[lo:hi]], 0)
         n = hi - lo
-        acc = h[lo:hi].clone()
         for j in range(taps):
-            acc += w[:, j] * ext[j:j + n]
-        out[lo:hi] = acc
+            out[lo:hi] += w[:, j] * ext[j:j + n]
         state[ss[b]] = ext[n:n + K]
-    return out if dtype == torch.float32 else out.to(dtype)
+    return out
 
 
 def embed_bigram_norm(tokens: torch.Tensor, embed: torch.Tensor, bigram: Optional[torch.Tensor], mul_prev: int,

@@ -1,8 +1,9 @@
 """Sliding-window attention over the paged cache with shaped scores: soft cap, linear distance bias, mixing of the
 heads' scores ahead of the softmax, an optional value-less sink in the denominator, optionally the first tokens of a
-sequence kept visible beyond the window. Two ways of preparing queries and keys: RMS norm with a weight
-(`qk_norm_cache_write`), or rotation by position followed by a weightless RMS norm, with the values optionally mixed
-with those of another layer (`rot_norm_cache_write`).
+sequence kept visible beyond the window, or visibility confined to chunks of positions. Three ways of preparing queries
+and keys: RMS norm with a weight (`qk_norm_cache_write`); rotation by position followed by a weightless RMS norm, with
+the values optionally mixed with those of another layer (`rot_norm_cache_write`); RMS norm over all heads together
+followed by a rotation, the values optionally the keys as projected (`qk_rows_norm_cache_write`).
 
 GPU: ``csrc/hip/window_attn.hip`` (one kernel for prompt portions and, with a split key range, for decoding).
 CPU: a PyTorch formulation used by the unit tests and CPU runs.
@@ -28,6 +29,7 @@ class ScoreShape:
     window: int = 0  # <= 0: all earlier tokens
     sink: bool = False
     keep_first: int = 0  # keys at positions below this stay visible to every later query, whatever the window
+    chunk: int = 0  # > 0: a query sees keys of its own chunk of positions only (chunks counted from position 0)
 
 
 def alloc_window_cache(num_pages: int, n_kv_heads: int, k_dim: int, v_dim: int, dtype, device
@@ -119,31 +121,107 @@ def sigmoid_gate_rows(x: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
     return x
 
 
-def rotation_table(base: float, dims: int, n_pos: int, device, scaling: Optional[dict] = None) -> torch.Tensor:
-    """fp32 [n_pos, dims]: m cos(p f_i) for i < dims/2, then m sin(p f_i), with f_i = base^(-2i/dims).
+def rotation_frequencies(base: float, dims: int, scaling: Optional[dict] = None) -> Tuple[torch.Tensor, float]:
+    """float64 [dims/2] angles per position of the rotated pairs, f_i = base^(-2i/dims), and the factor on their cosines
+    and sines. Two kinds of `scaling` for contexts beyond `original` positions:
 
-    `scaling` = {factor, original, fast, slow} stretches the slow pairs for contexts beyond `original` positions (YaRN:
-    Peng et al., "YaRN: Efficient Context Window Extension of Large Language Models"): with
-    d(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor(d(fast)), 0), hi = min(ceil(d(slow)), dims - 1) and
-    ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1) the frequency is f_i (1 - ramp_i) + f_i ramp_i / factor, and
-    m = 0.1 ln(factor) + 1 (1 without scaling). Angles are formed in float64 and rounded once."""
+    {factor, original, fast, slow} (YaRN: Peng et al., "YaRN: Efficient Context Window Extension of Large Language
+    Models"): with d(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor(d(fast)), 0),
+    hi = min(ceil(d(slow)), dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1) the frequency is
+    f_i (1 - ramp_i) + f_i ramp_i / factor, the factor 0.1 ln(factor) + 1;
+
+    {factor, original, low, high} (as in Llama 3.1): with n_i = original f_i / (2 pi) turns over the original context and
+    s_i = clamp((n_i - low) / (high - low), 0, 1) the frequency is f_i s_i + f_i (1 - s_i) / factor, the factor 1."""
     assert dims % 2 == 0 and dims > 0
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims)
-    m = 1.0
-    if scaling:
-        factor, orig = float(scaling["factor"]), float(scaling["original"])
+    if not scaling:
+        return f, 1.0
+    factor, orig = float(scaling["factor"]), float(scaling["original"])
+    if "low" in scaling:
+        low, high = float(scaling["low"]), float(scaling["high"])
+        turns = orig * f / (2.0 * math.pi)
+        if high > low:
+            s = ((turns - low) / (high - low)).clamp(0.0, 1.0)
+        else:  # no blend between the two limits
+            s = (turns >= low).double()
+        return f * s + f * (1.0 - s) / factor, 1.0
 
-        def d_of(turns: float) -> float:
-            return dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(float(base)))
+    def d_of(t: float) -> float:
+        return dims * math.log(orig / (2.0 * math.pi * t)) / (2.0 * math.log(float(base)))
 
-        lo = max(math.floor(d_of(float(scaling["fast"]))), 0)
-        hi = min(math.ceil(d_of(float(scaling["slow"]))), dims - 1)
-        ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
-        f = f / factor * ramp + f * (1.0 - ramp)
-        m = 0.1 * math.log(factor) + 1.0
+    lo = max(math.floor(d_of(float(scaling["fast"]))), 0)
+    hi = min(math.ceil(d_of(float(scaling["slow"]))), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return f / factor * ramp + f * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
+
+
+def rotation_table(base: float, dims: int, n_pos: int, device, scaling: Optional[dict] = None) -> torch.Tensor:
+    """fp32 [n_pos, dims]: m cos(p f_i) for i < dims/2, then m sin(p f_i), with f_i and m from `rotation_frequencies`.
+    Angles are formed in float64 and rounded once."""
+    f, m = rotation_frequencies(base, dims, scaling)
     a = torch.arange(n_pos, dtype=torch.float64).unsqueeze(1) * f
     return (torch.cat([a.cos(), a.sin()], 1) * m).float().to(device)
+
+
+def table_key(rot: dict, n_pos: int) -> Tuple:
+    """What tells one rotation table from another (mixers with equal constants share one)."""
+    sc = rot.get("scaling") or None
+    return ("rot", float(rot["base"]), int(rot["dims"]), int(n_pos),
+            tuple(sorted((k, float(v)) for k, v in sc.items())) if sc else None)
+
+
+def qk_rows_norm_cache_write(proj: torch.Tensor, v_off: int, q_weight: torch.Tensor, k_weight: torch.Tensor,
+                             positions: Optional[torch.Tensor], table: Optional[torch.Tensor], slots: torch.Tensor,
+                             kcache: torch.Tensor, vcache: torch.Tensor, n_heads: int, eps: float,
+                             v_transposed: bool = False) -> torch.Tensor:
+    """proj [T, *]: q heads | k heads from column 0, values (G Dv numbers) from column v_off on (v_off = H D: the keys as
+    projected are the values). RMS norm over ALL query numbers of a token and over all its key numbers (weights [H D] and
+    [G D]), then - with `table` as `rotation_table` makes it - rotation of the first table.shape[1] coordinates of every
+    head, coordinate i with i + dims/2. Keys and values of tokens with slot >= 0 go into the paged caches
+    (`v_transposed`: V pages [pages, G, Dv, 32]). Returns the queries [T, H, D]."""
+    T = proj.shape[0]
+    G, D, V = kcache.shape[1], kcache.shape[3], vcache.shape[2 if v_transposed else 3]
+    H = n_heads
+    R = 0 if table is None else table.shape[1]
+    assert proj.stride(1) == 1 and proj.shape[1] >= max((H + G) * D, v_off + G * V) and R <= D and R % 2 == 0
+    assert q_weight.numel() == H * D and k_weight.numel() == G * D
+    q = torch.empty(T, H, D, dtype=proj.dtype, device=proj.device)
+    if L.use_hip(proj):
+        assert slots.dtype == torch.int64 and kcache.dtype == proj.dtype and vcache.dtype == proj.dtype
+        assert q_weight.dtype == proj.dtype and k_weight.dtype == proj.dtype
+        assert q_weight.is_contiguous() and k_weight.is_contiguous()
+        assert table is None or (table.dtype == torch.float32 and table.is_contiguous()
+                                 and positions.dtype == torch.int32)
+        L.check(L.lib().areal_qk_rows_norm_cache_write(
+            L.ptr(proj), L.c_int64(proj.stride(0)), L.c_int(int(v_off)), L.ptr(q_weight), L.ptr(k_weight),
+            L.ptr(positions) if table is not None else None, L.ptr(table),
+            L.c_int(table.shape[0] if table is not None else 0), L.c_int(R), L.ptr(slots), L.ptr(q), L.ptr(kcache),
+            L.ptr(vcache), L.c_int(T), L.c_int(H), L.c_int(G), L.c_int(D), L.c_int(V), L.c_float(eps),
+            L.c_int(int(v_transposed)), L.c_int(L.dtype_flag(proj)), L.stream_ptr()), "qk_rows_norm_cache_write")
+        return q
+
+    def normed(x, w):
+        x = x.float()
+        return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+
+    qk = torch.cat([normed(proj[:, :H * D], q_weight), normed(proj[:, H * D:(H + G) * D], k_weight)], 1).view(T, H + G, D)
+    if R:
+        cs = table[positions.long()]
+        c, s = cs[:, :R // 2].unsqueeze(1), cs[:, R // 2:].unsqueeze(1)
+        u, w = qk[..., :R // 2], qk[..., R // 2:R]
+        qk = torch.cat([u * c - w * s, w * c + u * s, qk[..., R:]], -1)
+    q.copy_(qk[:, :H])
+    ok = slots >= 0
+    if ok.any():
+        pg, off = (slots[ok] // PAGE_SIZE).long(), (slots[ok] % PAGE_SIZE).long()
+        kcache[pg, :, off, :] = qk[:, H:][ok].to(kcache.dtype)
+        v = proj[ok, v_off:v_off + G * V].reshape(-1, G, V)
+        if v_transposed:
+            vcache[pg, :, :, off] = v
+        else:
+            vcache[pg, :, off, :] = v
+    return q
 
 
 def rot_norm_cache_write(proj: torch.Tensor, positions: torch.Tensor, table: Optional[torch.Tensor],
@@ -251,23 +329,29 @@ def window_attention_standard(q: torch.Tensor, kcache: torch.Tensor, vcache_t: t
             L.ptr(q), L.ptr(kcache), L.ptr(vcache_t), L.ptr(block_tables), L.ptr(ctx_len), L.ptr(out), L.ptr(pa),
             L.ptr(pm), L.c_int(B), L.c_int(H), L.c_int(G), L.c_int(D), L.c_int(block_tables.shape[1]),
             L.c_int(int(nsplit)), L.c_float(shape.scale), L.c_int(q.stride(0)), L.c_int(int(shape.window)),
-            L.c_int(int(shape.keep_first)), L.ptr(r1), L.ptr(r2), L.ptr(gate), L.c_int64(gstride), L.stream_ptr()),
-            "paged_decode_window")
+            L.c_int(int(shape.keep_first)), L.ptr(r1), L.ptr(r2), L.ptr(gate), L.c_int64(gstride),
+            L.c_int(int(shape.chunk)), L.stream_ptr()), "paged_decode_window")
         return out
     assert cu_q.dtype == torch.int32 and cu_k.dtype == torch.int32
     L.check(L.lib().areal_flash_fwd_paged_window(
         L.ptr(q), L.ptr(kcache), L.ptr(vcache_t), L.ptr(block_tables), L.c_int(block_tables.shape[1]), L.ptr(out),
         L.ptr(cu_q), L.ptr(cu_k), L.c_int(B), L.c_int(int(max_q)), L.c_int(T), L.c_int(H), L.c_int(G), L.c_int(D),
         L.c_int64(q.stride(0)), L.c_int64(out.stride(0)), L.c_float(shape.scale), L.c_int(int(shape.window)),
-        L.c_int(int(shape.keep_first)), L.ptr(r1), L.ptr(r2), L.ptr(gate), L.c_int64(gstride), L.stream_ptr()),
-        "flash_fwd_paged_window")
+        L.c_int(int(shape.keep_first)), L.ptr(r1), L.ptr(r2), L.ptr(gate), L.c_int64(gstride), L.c_int(int(shape.chunk)),
+        L.stream_ptr()), "flash_fwd_paged_window")
     return out
 
 
-def decode_splits(batch: int, window: int, max_context: int, keep_first: int = 0) -> int:
+def visible_span(window: int, max_context: int, keep_first: int = 0, chunk: int = 0) -> int:
+    """The most keys (whole pages at both ends counted) that a decoded token's pages hold."""
+    span = max_context if window <= 0 else min(window + PAGE_SIZE + max(0, keep_first), max_context)
+    return span if chunk <= 0 else min(span, chunk + PAGE_SIZE + max(0, keep_first))
+
+
+def decode_splits(batch: int, window: int, max_context: int, keep_first: int = 0, chunk: int = 0) -> int:
     """Key-range splits of a decode launch: about two workgroups per compute unit, down to one page each (a
     workgroup walks its pages one after the other, so short ranges are what makes a decode step short)."""
-    span = max_context if window <= 0 else min(window + PAGE_SIZE + max(0, keep_first), max_context)
+    span = visible_span(window, max_context, keep_first, chunk)
     pages = max(1, (span + PAGE_SIZE - 1) // PAGE_SIZE)
     return int(max(1, min(512 // max(1, batch), pages, 32)))
 
@@ -321,7 +405,7 @@ def window_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
             L.ptr(pa), L.ptr(pm), L.c_int(B), L.c_int(int(max_q)), L.c_int(T),
             L.c_int(H), L.c_int(G), L.c_int(D), L.c_int(V), L.c_int(bq), L.c_float(shape.scale),
             L.c_float(shape.softcap), L.c_float(shape.slope_exp), L.c_int(int(shape.window)),
-            L.c_int(int(shape.keep_first)), L.c_int(int(shape.sink)),
+            L.c_int(int(shape.keep_first)), L.c_int(int(shape.chunk)), L.c_int(int(shape.sink)),
             L.c_int(int(nsplit)), L.c_int(L.dtype_flag(q)), L.c_int(int(matrix_cores)), L.stream_ptr()), "window_attn")
         return out
     out = torch.zeros(T, H, V, dtype=torch.float32, device=q.device)
@@ -334,6 +418,8 @@ def window_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
         if n == 0:
             continue
         lo = 0 if (shape.window <= 0 or shape.keep_first > 0) else max(0, ctx - n - shape.window + 1)
+        if shape.chunk > 0 and shape.keep_first <= 0:
+            lo = max(lo, (ctx - n) // shape.chunk * shape.chunk)
         pages = block_tables[b, :(ctx + PAGE_SIZE - 1) // PAGE_SIZE].long()
         kk = kcache[pages].permute(1, 0, 2, 3).reshape(G, -1, D)[:, lo:ctx].float().repeat_interleave(rep, 0)
         vv = vcache[pages].permute(1, 0, 2, 3).reshape(G, -1, V)[:, lo:ctx].float().repeat_interleave(rep, 0)
@@ -348,7 +434,12 @@ def window_attention(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor
                                                                       * (i - j).clamp(min=0).float())
         if mix is not None:
             s = torch.einsum("hg,gij->hij", mix.float(), s)
-        ok = (i - j >= 0) & (((i - j < shape.window) | (j < shape.keep_first)) if shape.window > 0 else True)
+        near = torch.ones_like(i - j, dtype=torch.bool)
+        if shape.window > 0:
+            near = near & (i - j < shape.window)
+        if shape.chunk > 0:
+            near = near & (i // shape.chunk == j // shape.chunk)
+        ok = (i - j >= 0) & (near | (j < shape.keep_first))
         s = s.masked_fill(~ok, float("-inf"))
         m = s.max(-1, keepdim=True).values
         if shape.sink:

@@ -18,7 +18,8 @@
 // WIN = true adds a sliding window that keeps the first tokens (a query at position p sees key j <= p when
 // p - j < window or j < keep): key tiles that no query of the workgroup can see are skipped (the tiles that hold kept
 // tokens, then the tiles from the window's start on), and the softmax weights enter O^T += V^T.P^T as the pair
-// (bf16(p), bf16(p - bf16(p))), two products, so that they carry 16 bits of mantissa instead of 8.
+// (bf16(p), bf16(p - bf16(p))), two products, so that they carry 16 bits of mantissa instead of 8. chunk > 0 confines a
+// query to the keys of its own chunk of positions (counted from the sequence's start).
 //
 // Role in the reference: prefill against the radix cache inside its serving engine, and
 // flash_attn_with_kvcache at realhf/impl/model/modules/attn.py:272.
@@ -33,7 +34,7 @@ __global__ __launch_bounds__(256, 2) void flash_fwd_paged_kernel(
     const int* __restrict__ cu_q, const int* __restrict__ cu_k, int64_t q_stride, int64_t o_stride, int Hq, int Hkv,
     int nbatch, int total_q, float scale_log2, int causal, int window = 0, int keep = 0,
     const bf16_t* __restrict__ r1 = nullptr, const bf16_t* __restrict__ r2 = nullptr,
-    const bf16_t* __restrict__ gate = nullptr, int64_t gate_stride = 0) {
+    const bf16_t* __restrict__ gate = nullptr, int64_t gate_stride = 0, int chunk = 0) {
   constexpr int D = 128;
   __shared__ __attribute__((aligned(16))) char smem[2 * 64 * 256];
   char* ks = smem;             // K tile  [64 keys][256 B], 16-byte chunks swizzled (flash_tiles.hpp)
@@ -87,9 +88,19 @@ __global__ __launch_bounds__(256, 2) void flash_fwd_paged_kernel(
   const int ntile_k = k_hi > 0 ? (k_hi + 63) / 64 : 0;
   // WIN: tiles [0, n_keep) and [t_lo, ntile_k) are walked, `tile_of` maps the step to its tile
   int t_lo = 0, n_keep = 0;
-  if (WIN && window > 0) {
-    t_lo = min(max(0, qt * 128 + shift - window + 1) / 64, ntile_k);
+  const bool windowed = WIN && (window > 0 || chunk > 0);
+  // the first key a query at position p sees besides the kept ones; never decreases as p grows
+  auto first_key = [&](int p) {
+    int lo = window > 0 ? max(0, p - window + 1) : 0;
+    if (chunk > 0) lo = max(lo, p / chunk * chunk);
+    return lo;
+  };
+  int my_lo = 0, wave_lo = 0;
+  if (windowed) {
+    t_lo = min(first_key(qt * 128 + shift) / 64, ntile_k);
     n_keep = min((max(keep, 0) + 63) / 64, t_lo);
+    my_lo = first_key(my_q + shift);
+    wave_lo = first_key(q0 + 31 + shift);
   }
   const int n_iter = n_keep + ntile_k - t_lo;
   auto tile_of = [&](int it) { return it < n_keep ? it : t_lo + it - n_keep; };
@@ -160,9 +171,8 @@ __global__ __launch_bounds__(256, 2) void flash_fwd_paged_kernel(
       }
     }
     const int kbase = t * 64;
-    const bool windowed = WIN && window > 0;
     const bool need_mask = (kbase + 64 > k_len) || (causal && (kbase + 63 > q0 + shift)) ||
-                           (windowed && kbase < q0 + 31 + shift - window + 1);
+                           (windowed && kbase < wave_lo);
     float mx = -INFINITY;
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb)
@@ -176,7 +186,7 @@ __global__ __launch_bounds__(256, 2) void flash_fwd_paged_kernel(
         if (need_mask) {
           const int key = kbase + 32 * kb + (j & 3) + 8 * (j >> 2) + 4 * hf;
           if (key >= k_len || (causal && key > my_q + shift)) sv = -INFINITY;
-          if (windowed && my_q + shift - key >= window && key >= keep) sv = -INFINITY;
+          if (windowed && key < my_lo && key >= keep) sv = -INFINITY;
         }
         sacc[kb][j] = sv;
         mx = fmaxf(mx, sv);
@@ -278,13 +288,13 @@ extern "C" int areal_flash_fwd_paged(const void* q, const void* kcache, const vo
 // The same over a sliding window that keeps the first `keep` tokens (window <= 0: every earlier key), bf16 caches,
 // softmax weights at 16 bits of mantissa; always causal. r1 / r2 (one number per query head each, or null): a learned
 // logarithmic distance penalty r1_h ln(1 + r2_h (i - j)) on the scaled scores. gate (rows of Hq 128 numbers, gate_stride
-// apart, or null): the output is multiplied by sigmoid(gate) element by element.
+// apart, or null): the output is multiplied by sigmoid(gate) element by element. chunk > 0: keys of the query's own chunk.
 extern "C" int areal_flash_fwd_paged_window(const void* q, const void* kcache, const void* vcache,
                                             const int* block_tables, int max_pages, void* o, const int* cu_q,
                                             const int* cu_k, int B, int max_q, int total_q, int Hq, int Hkv, int D,
                                             int64_t q_stride, int64_t o_stride, float softmax_scale, int window, int keep,
                                             const void* r1, const void* r2, const void* gate, int64_t gate_stride,
-                                            hipStream_t st) {
+                                            int chunk, hipStream_t st) {
   if (B == 0 || max_q == 0) return 0;
   if (D != 128) return -1;
   if (Hq % Hkv != 0) return -2;
@@ -297,6 +307,6 @@ extern "C" int areal_flash_fwd_paged_window(const void* q, const void* kcache, c
   hipLaunchKernelGGL((flash_fwd_paged_kernel<false, true>), grid, block, 0, st, (const bf16_t*)q, kcache, vcache,
                      block_tables, max_pages, (bf16_t*)o, (float*)nullptr, cu_q, cu_k, q_stride, o_stride, Hq, Hkv, B,
                      total_q, scale_log2, 1, window, keep, (const bf16_t*)r1, (const bf16_t*)r2, (const bf16_t*)gate,
-                     gate_stride);
+                     gate_stride, chunk);
   return (int)hipGetLastError();
 }

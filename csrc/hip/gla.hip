@@ -319,7 +319,8 @@ __global__ void __launch_bounds__(256) gla_chunk_kernel(
 template <typename T>
 __global__ void __launch_bounds__(256) gla_out_kernel(const float* __restrict__ obuf, const T* __restrict__ gate,
                                                       int64_t gate_stride, const T* __restrict__ w, T* __restrict__ out,
-                                                      int64_t n_rows, int NH, int V, float eps) {
+                                                      int64_t out_stride, float out_scale, int64_t n_rows, int NH, int V,
+                                                      float eps) {
   const int lane = threadIdx.x & 63;
   const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= n_rows) return;
@@ -331,7 +332,7 @@ __global__ void __launch_bounds__(256) gla_out_kernel(const float* __restrict__ 
   const float r = 1.f / sqrtf(wave_sum(ss) / (float)V + eps);
   for (int i = lane; i < V; i += 64) {
     const float g = ldf<T>(gate, t * gate_stride + hd * V + i);
-    stf<T>(out, row * V + i, o[i] * r * ldf<T>(w, i) * (g / (1.f + expf(-g))));
+    stf<T>(out, t * out_stride + hd * V + i, o[i] * r * ldf<T>(w, i) * (g / (1.f + expf(-g))) * out_scale);
   }
 }
 
@@ -398,17 +399,18 @@ extern "C" int areal_gla_scan(const void* proj, int64_t row_stride, int q_off, i
   return (int)hipGetLastError();
 }
 
-// obuf [T, NH, V] fp32, gate rows of NH V with gate_stride, w [V]; out [T, NH V] contiguous
-extern "C" int areal_gla_out(const float* obuf, const void* gate, int64_t gate_stride, const void* w, void* out, int T,
-                             int NH, int V, float eps, int dt, hipStream_t st) {
+// obuf [T, NH, V] fp32, gate rows of NH V with gate_stride, w [V]; out rows of NH V numbers, out_stride apart, times out_scale
+extern "C" int areal_gla_out(const float* obuf, const void* gate, int64_t gate_stride, const void* w, void* out,
+                             int64_t out_stride, float out_scale, int T, int NH, int V, float eps, int dt,
+                             hipStream_t st) {
   if (T == 0) return 0;
   const int64_t n = (int64_t)T * NH;
   const dim3 grid((unsigned)((n + 3) / 4));
   if (dt == 0)
     hipLaunchKernelGGL(gla_out_kernel<bf16_t>, grid, dim3(256), 0, st, obuf, (const bf16_t*)gate, gate_stride,
-                       (const bf16_t*)w, (bf16_t*)out, n, NH, V, eps);
+                       (const bf16_t*)w, (bf16_t*)out, out_stride, out_scale, n, NH, V, eps);
   else
     hipLaunchKernelGGL(gla_out_kernel<float>, grid, dim3(256), 0, st, obuf, (const float*)gate, gate_stride,
-                       (const float*)w, (float*)out, n, NH, V, eps);
+                       (const float*)w, (float*)out, out_stride, out_scale, n, NH, V, eps);
   return (int)hipGetLastError();
 }

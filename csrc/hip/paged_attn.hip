@@ -30,7 +30,7 @@ DEVINL f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) {
 // FP8: the caches hold e4m3 bytes (same layouts); a lane fetches 8 bytes per fragment and widens them to bf16 in
 // registers - half the HBM traffic of the kernel, which is what bounds it at long contexts.
 // WIN = true: the query (the context's last token) sees key j when ctx - 1 - j < window or j < keep (window <= 0:
-// every key); pages without a visible key are skipped, and the softmax weights enter the P.V product as the pair
+// every key; chunk > 0: and floor(j / chunk) = floor((ctx - 1) / chunk)); pages without a visible key are skipped, and the softmax weights enter the P.V product as the pair
 // (bf16(p), bf16(p - bf16(p))) so that they carry 16 bits of mantissa.
 template <int D, bool FP8, bool WIN = false>
 __global__ __launch_bounds__(256, (D > 128 ? 1 : 2)) void paged_decode_kernel(
@@ -39,7 +39,7 @@ __global__ __launch_bounds__(256, (D > 128 ? 1 : 2)) void paged_decode_kernel(
     const int* __restrict__ context_lens, bf16_t* __restrict__ out, float* __restrict__ part_o,
     float* __restrict__ part_ml, int Hq, int Hkv, int max_pages, float scale_log2, int q_stride, int window = 0,
     int keep = 0, const bf16_t* __restrict__ r1 = nullptr, const bf16_t* __restrict__ r2 = nullptr,
-    const bf16_t* __restrict__ gate = nullptr, int64_t gate_stride = 0) {
+    const bf16_t* __restrict__ gate = nullptr, int64_t gate_stride = 0, int chunk = 0) {
   constexpr int KS = D / 32;  // k-steps of the QK product
   constexpr int DB = D / 16;  // 16-wide d blocks of the PV product
   extern __shared__ __attribute__((aligned(16))) float smem[];
@@ -50,8 +50,10 @@ __global__ __launch_bounds__(256, (D > 128 ? 1 : 2)) void paged_decode_kernel(
   const int ctx = context_lens[b];
   const int npages = (ctx + PAGE - 1) / PAGE;
   // WIN: pages [0, n_keep) and [p_lo, npages) are walked; step i of the walk is page i (i < n_keep) or p_lo + i - n_keep
-  const bool windowed = WIN && window > 0;
-  const int p_lo = windowed ? max(0, ctx - window) / PAGE : 0;
+  const bool windowed = WIN && (window > 0 || chunk > 0);
+  int first = windowed && window > 0 ? max(0, ctx - window) : 0;  // first key seen besides the kept ones
+  if (windowed && chunk > 0) first = max(first, (ctx - 1) / chunk * chunk);
+  const int p_lo = first / PAGE;
   const int n_keep = windowed ? min((max(keep, 0) + PAGE - 1) / PAGE, p_lo) : 0;
   const int nwalk = n_keep + npages - p_lo;
   const int per = (nwalk + nsplit - 1) / nsplit;
@@ -107,7 +109,7 @@ __global__ __launch_bounds__(256, (D > 128 ? 1 : 2)) void paged_decode_kernel(
     for (int r = 0; r < 8; ++r) {
       float v = (r < 4 ? sa[r] : sb[r - 4]) * scale_log2;
       if (WIN && r1 != nullptr) v -= b1 * __log2f(1.f + b2 * (float)max(ctx - 1 - (key0 + r), 0));
-      s[r] = (key0 + r < ctx && (!windowed || ctx - 1 - (key0 + r) < window || key0 + r < keep)) ? v : -INFINITY;
+      s[r] = (key0 + r < ctx && (!windowed || key0 + r >= first || key0 + r < keep)) ? v : -INFINITY;
       mx = fmaxf(mx, s[r]);
     }
     mx = max_xor16(mx);
@@ -287,7 +289,7 @@ extern "C" int areal_paged_decode_window(const void* q, const void* kcache, cons
                                          const int* context_lens, void* out, float* part_o, float* part_ml, int B,
                                          int Hq, int Hkv, int D, int max_pages, int nsplit, float softmax_scale,
                                          int q_stride, int window, int keep, const void* r1, const void* r2,
-                                         const void* gate, int64_t gate_stride, hipStream_t st) {
+                                         const void* gate, int64_t gate_stride, int chunk, hipStream_t st) {
   if (B == 0) return 0;
   if (Hq % Hkv != 0 || Hq / Hkv > 16) return -1;
   if (D != 128 && D != 64) return -2;
@@ -298,12 +300,12 @@ extern "C" int areal_paged_decode_window(const void* q, const void* kcache, cons
     hipLaunchKernelGGL((paged_decode_kernel<128, false, true>), dim3(B, Hkv, nsplit), dim3(256), lds, st,
                        (const bf16_t*)q, kcache, vcache, block_tables, context_lens, (bf16_t*)out, part_o, part_ml, Hq,
                        Hkv, max_pages, scale_log2, q_stride, window, keep, (const bf16_t*)r1, (const bf16_t*)r2,
-                       (const bf16_t*)gate, gate_stride);
+                       (const bf16_t*)gate, gate_stride, chunk);
   else
     hipLaunchKernelGGL((paged_decode_kernel<64, false, true>), dim3(B, Hkv, nsplit), dim3(256), lds, st,
                        (const bf16_t*)q, kcache, vcache, block_tables, context_lens, (bf16_t*)out, part_o, part_ml, Hq,
                        Hkv, max_pages, scale_log2, q_stride, window, keep, (const bf16_t*)r1, (const bf16_t*)r2,
-                       (const bf16_t*)gate, gate_stride);
+                       (const bf16_t*)gate, gate_stride, chunk);
   if (nsplit > 1)
     hipLaunchKernelGGL(paged_decode_reduce_kernel, dim3(B * Hq), dim3(D), 0, st, part_o, part_ml, (bf16_t*)out, nsplit, D,
                        (const bf16_t*)gate, gate_stride, Hq);

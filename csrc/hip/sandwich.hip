@@ -6,6 +6,7 @@
 //   gated_norm_add    x <- x + s * LN(y * sigmoid(r); w, b)   [+ the next sublayer's norm of the new x]
 //   canon_conv        out_t = h_t + sum_j w[:, j] h_(t - taps + 1 + j); history before a row's first token comes
 //                     from the row's state slot (zeros before position 0); the slot then takes the row's last inputs
+//   conv_silu         out_t = silu(sum_j w[:, j] h_(t - taps + 1 + j) + bias), the same history
 //   embed_bigram_norm x = LN(E[tok] + B[(prev * a + tok * b) mod n])   (row n of B at position 0)
 //
 // T is the storage type (bf16 / fp32) of weights and of the sublayers' outputs; the stream x is fp32.
@@ -167,26 +168,38 @@ __global__ void __launch_bounds__(1024) gated_norm_add_kernel(
 
 // One workgroup per token. The workgroup of a row's FIRST token also serves the row's next taps - 2 tokens (all those
 // whose history reaches into the state slot) and then rewrites the slot, so nobody else reads or writes that slot.
-template <typename T>
-__global__ void __launch_bounds__(256) canon_conv_kernel(const float* __restrict__ h, const T* __restrict__ w,
-                                                         float* __restrict__ state, const int* __restrict__ cu_q,
-                                                         const int* __restrict__ first_pos,
-                                                         const int* __restrict__ state_slots, T* __restrict__ out,
-                                                         int B, int W, int taps) {
+// TI: type of the inputs (rows h_stride apart). ACT = false: out = h + conv(h); true: out = silu(conv(h) + bias).
+template <typename TI, typename T, bool ACT>
+__global__ void __launch_bounds__(256) causal_conv_kernel(const TI* __restrict__ h, int64_t h_stride,
+                                                          const T* __restrict__ w, const T* __restrict__ bias,
+                                                          float* __restrict__ state, const int* __restrict__ cu_q,
+                                                          const int* __restrict__ first_pos,
+                                                          const int* __restrict__ state_slots, T* __restrict__ out,
+                                                          int B, int W, int taps) {
   const int t = blockIdx.x, K = taps - 1, c = blockIdx.y * 256 + threadIdx.x;  // one channel per thread
   const int b = row_of(cu_q, B, t);
   const int q0 = cu_q[b], n = cu_q[b + 1] - q0, off = t - q0;
   if (off >= n) return;  // a token no row owns
   const int slot = state_slots[b];
+  auto put = [&](int tok, float self, float conv) {
+    float a;
+    if (ACT) {
+      a = conv + (bias ? ldf<T>(bias, c) : 0.f);
+      a /= 1.f + expf(-a);
+    } else {
+      a = self + conv;
+    }
+    stf<T>(out, (size_t)tok * W + c, a);
+  };
   if (slot < 0) {  // padding row: its values go nowhere, they only have to be finite
-    if (c < W) stf<T>(out, (size_t)t * W + c, h[(size_t)t * W + c]);
+    if (c < W) put(t, ldf<TI>(h, (size_t)t * h_stride + c), 0.f);
     return;
   }
   if (off >= K) {  // the whole history is inside the row
     if (c < W) {
-      float a = h[(size_t)t * W + c];
-      for (int j = 0; j < taps; ++j) a += ldf<T>(w, (size_t)c * taps + j) * h[(size_t)(t - K + j) * W + c];
-      stf<T>(out, (size_t)t * W + c, a);
+      float a = 0.f;
+      for (int j = 0; j < taps; ++j) a += ldf<T>(w, (size_t)c * taps + j) * ldf<TI>(h, (size_t)(t - K + j) * h_stride + c);
+      put(t, ldf<TI>(h, (size_t)t * h_stride + c), a);
     }
     return;
   }
@@ -195,15 +208,15 @@ __global__ void __launch_bounds__(256) canon_conv_kernel(const float* __restrict
   float* sl = state + (size_t)slot * K * W;
   // input at index p relative to the row's first token (p < 0: the state slot, or zero before the sequence's start)
   auto val = [&](int p, int c) -> float {
-    if (p >= 0) return h[(size_t)(q0 + p) * W + c];
+    if (p >= 0) return ldf<TI>(h, (size_t)(q0 + p) * h_stride + c);
     return p0 + p >= 0 ? sl[(size_t)(K + p) * W + c] : 0.f;
   };
   const int m = min(K, n);
   if (c < W) {
     for (int i = 0; i < m; ++i) {
-      float a = val(i, c);
+      float a = 0.f;
       for (int j = 0; j < taps; ++j) a += ldf<T>(w, (size_t)c * taps + j) * val(i - K + j, c);
-      stf<T>(out, (size_t)(q0 + i) * W + c, a);
+      put(q0 + i, val(i, c), a);
     }
     // the slot's entry k becomes the input K - k tokens before the NEXT token; reads run ahead of the writes
     for (int k = 0; k < K; ++k) sl[(size_t)k * W + c] = val(n - K + k, c);
@@ -321,12 +334,29 @@ extern "C" int areal_canon_conv(const float* h, const void* w, float* state, con
                                 hipStream_t st) {
   if (T == 0 || B == 0) return 0;
   if (taps < 1 || (taps > 1 && !state) || (W + 255) / 256 > 65535) return -1;
+  const dim3 grid(T, (W + 255) / 256);
   if (dt == 0)
-    hipLaunchKernelGGL(canon_conv_kernel<bf16_t>, dim3(T, (W + 255) / 256), dim3(256), 0, st, h, (const bf16_t*)w, state, cu_q,
-                       first_pos, state_slots, (bf16_t*)out, B, W, taps);
+    hipLaunchKernelGGL((causal_conv_kernel<float, bf16_t, false>), grid, dim3(256), 0, st, h, (int64_t)W, (const bf16_t*)w,
+                       (const bf16_t*)nullptr, state, cu_q, first_pos, state_slots, (bf16_t*)out, B, W, taps);
   else
-    hipLaunchKernelGGL(canon_conv_kernel<float>, dim3(T, (W + 255) / 256), dim3(256), 0, st, h, (const float*)w, state, cu_q,
-                       first_pos, state_slots, (float*)out, B, W, taps);
+    hipLaunchKernelGGL((causal_conv_kernel<float, float, false>), grid, dim3(256), 0, st, h, (int64_t)W, (const float*)w,
+                       (const float*)nullptr, state, cu_q, first_pos, state_slots, (float*)out, B, W, taps);
+  return (int)hipGetLastError();
+}
+
+// out [T, W] = silu(conv(h) + bias), h rows in the storage type, h_stride apart; bias [W] or null
+extern "C" int areal_conv_silu(const void* h, int64_t h_stride, const void* w, const void* bias, float* state,
+                               const int* cu_q, const int* first_pos, const int* state_slots, void* out, int B, int T,
+                               int W, int taps, int dt, hipStream_t st) {
+  if (T == 0 || B == 0) return 0;
+  if (taps < 1 || (taps > 1 && !state) || (W + 255) / 256 > 65535) return -1;
+  const dim3 grid(T, (W + 255) / 256);
+  if (dt == 0)
+    hipLaunchKernelGGL((causal_conv_kernel<bf16_t, bf16_t, true>), grid, dim3(256), 0, st, (const bf16_t*)h, h_stride,
+                       (const bf16_t*)w, (const bf16_t*)bias, state, cu_q, first_pos, state_slots, (bf16_t*)out, B, W, taps);
+  else
+    hipLaunchKernelGGL((causal_conv_kernel<float, float, true>), grid, dim3(256), 0, st, (const float*)h, h_stride,
+                       (const float*)w, (const float*)bias, state, cu_q, first_pos, state_slots, (float*)out, B, W, taps);
   return (int)hipGetLastError();
 }
 

@@ -6,7 +6,8 @@
 //   s_g       <- s_g - r1_g * ln(1 + r2_g * (i - j))              (r1 / r2 given: a learned logarithmic distance penalty)
 //   t_h        = sum_g M[h, g] s_g                                 head mixing (M = null: t_h = s_h)
 //   visible:     0 <= i - j < window, or j <= i and j < keep_first    (window <= 0: every earlier key; the first
-//                keep_first tokens of a sequence stay visible to every later query, at their true positions)
+//                keep_first tokens of a sequence stay visible to every later query, at their true positions);
+//                chunk > 0: additionally floor(j / chunk) = floor(i / chunk), positions counted from the sequence's start
 //   p_h(j)     = exp(t_h(j)) / (sink + sum_j' exp(t_h(j')))        sink = 1: a key of score 0 that has no value
 //   o_h(i)     = sum_j p_h(j) v_c(h)(j)  [* sigmoid(gate_h(i)) when a gate is given: one number per head and token, or
 //                one per head, token and value channel (`gate_elem`)]
@@ -27,6 +28,13 @@
 namespace {
 
 constexpr int PAGE = 32;
+
+// First key (besides kept first ones) that a query at position `pos` sees; never decreases as pos grows.
+DEVINL int first_key(int pos, int window, int chunk) {
+  int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  if (chunk > 0) lo = max(lo, (pos / chunk) * chunk);
+  return lo;
+}
 
 template <typename T> DEVINL float ldf(const T* p, size_t i);
 template <> DEVINL float ldf<bf16_t>(const bf16_t* p, size_t i) { return bf2f(p[i]); }
@@ -261,6 +269,139 @@ __global__ void __launch_bounds__(256) qkv_vnorm_cache_write_kernel(
   }
 }
 
+// Sum of two values over a workgroup of 256 threads; every thread gets both. `red` holds 8 floats.
+DEVINL void block_sum2(float& a, float& b, float* red) {
+  a = wave_sum(a);
+  b = wave_sum(b);
+  if ((threadIdx.x & 63) == 0) {
+    red[threadIdx.x >> 6] = a;
+    red[4 + (threadIdx.x >> 6)] = b;
+  }
+  __syncthreads();
+  a = red[0] + red[1] + red[2] + red[3];
+  b = red[4] + red[5] + red[6] + red[7];
+}
+
+// Per token: the H D query numbers are RMS-normed together, and so are the G D key numbers (weights of those sizes);
+// then the first R coordinates of every head are rotated by the token's position, coordinate i with i + R / 2 (table rows
+// as above). Queries go to q_out, keys into the K cache. The values are the G V columns from v_off on, as they are
+// (v_off = H D: the keys as projected).
+template <typename T>
+__global__ void __launch_bounds__(256) qk_rows_norm_cache_write_kernel(
+    const T* __restrict__ proj, int64_t row_stride, int v_off, const T* __restrict__ qw, const T* __restrict__ kw,
+    const int* __restrict__ positions, const float* __restrict__ table, int n_pos, int R,
+    const int64_t* __restrict__ slots, T* __restrict__ q_out, T* __restrict__ kcache, T* __restrict__ vcache, int H, int G,
+    int D, int V, float eps, int v_transposed) {
+  __shared__ float red[8];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const T* row = proj + (size_t)t * row_stride;
+  const int64_t slot = slots[t];
+  const size_t page = slot >= 0 ? (size_t)(slot / PAGE) : 0;
+  const int off = slot >= 0 ? (int)(slot % PAGE) : 0;
+  const int nq = H * D, nk = G * D, half = R / 2;
+  float sq = 0.f, sk = 0.f;
+  for (int i = tid; i < nq; i += 256) sq += ldf<T>(row, i) * ldf<T>(row, i);
+  for (int i = tid; i < nk; i += 256) sk += ldf<T>(row, nq + i) * ldf<T>(row, nq + i);
+  block_sum2(sq, sk, red);
+  const float rq = 1.f / sqrtf(sq / (float)nq + eps), rk = 1.f / sqrtf(sk / (float)nk + eps);
+  const int pos = R > 0 ? min(max(positions[t], 0), n_pos - 1) : 0;
+  const float* cs = table + (size_t)pos * R;
+  const int units = half + (D - R);  // per head: pairs, then single coordinates
+  for (int i = tid; i < (H + G) * units; i += 256) {
+    const int u = i / units, e = i % units;
+    if (u >= H && slot < 0) continue;
+    const T* src = row + (size_t)u * D;
+    const T* w = u < H ? qw + (size_t)u * D : kw + (size_t)(u - H) * D;
+    const float r = u < H ? rq : rk;
+    T* dst = u < H ? q_out + ((size_t)t * H + u) * D : kcache + ((page * G + (u - H)) * PAGE + off) * D;
+    if (e < half) {
+      const float a = ldf<T>(src, e) * r * ldf<T>(w, e), b = ldf<T>(src, e + half) * r * ldf<T>(w, e + half);
+      const float c = cs[e], s = cs[half + e];
+      stf<T>(dst, e, a * c - b * s);
+      stf<T>(dst, e + half, b * c + a * s);
+    } else {
+      stf<T>(dst, half + e, ldf<T>(src, half + e) * r * ldf<T>(w, half + e));
+    }
+  }
+  if (slot >= 0) {
+    const T* vsrc = row + v_off;
+    for (int i = tid; i < G * V; i += 256) {
+      const int c = i / V, v = i % V;
+      vcache[v_transposed ? ((page * G + c) * V + v) * PAGE + off : ((page * G + c) * PAGE + off) * V + v] = vsrc[i];
+    }
+  }
+}
+
+// The same for bf16 rows whose sizes, halves, strides and addresses are multiples of 8 elements: 16-byte moves.
+__global__ void __launch_bounds__(256) qk_rows_norm_cache_write_vec_kernel(
+    const bf16_t* __restrict__ proj, int64_t row_stride, int v_off, const bf16_t* __restrict__ qw,
+    const bf16_t* __restrict__ kw, const int* __restrict__ positions, const float* __restrict__ table, int n_pos, int R,
+    const int64_t* __restrict__ slots, bf16_t* __restrict__ q_out, bf16_t* __restrict__ kcache,
+    bf16_t* __restrict__ vcache, int H, int G, int D, int V, float eps, int v_transposed) {
+  __shared__ float red[8];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const bf16_t* row = proj + (size_t)t * row_stride;
+  const int64_t slot = slots[t];
+  const size_t page = slot >= 0 ? (size_t)(slot / PAGE) : 0;
+  const int off = slot >= 0 ? (int)(slot % PAGE) : 0;
+  const int nq = H * D, nk = G * D, half = R / 2;
+  float sq = 0.f, sk = 0.f;
+  for (int i = 8 * tid; i < nq + nk; i += 8 * 256) {
+    const bf16x8 x = ld8(row + i);
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s += bf2f(x[e]) * bf2f(x[e]);
+    if (i < nq) sq += s;
+    else sk += s;
+  }
+  block_sum2(sq, sk, red);
+  const float rq = 1.f / sqrtf(sq / (float)nq + eps), rk = 1.f / sqrtf(sk / (float)nk + eps);
+  const int pos = R > 0 ? min(max(positions[t], 0), n_pos - 1) : 0;
+  const float* cs = table + (size_t)pos * R;
+  const int h8 = half / 8, units = h8 + (D - R) / 8;
+  for (int i = tid; i < (H + G) * units; i += 256) {
+    const int u = i / units, e = i % units;
+    if (u >= H && slot < 0) continue;
+    const bf16_t* src = row + (size_t)u * D;
+    const bf16_t* w = u < H ? qw + (size_t)u * D : kw + (size_t)(u - H) * D;
+    const float r = u < H ? rq : rk;
+    bf16_t* dst = u < H ? q_out + ((size_t)t * H + u) * D : kcache + ((page * G + (u - H)) * PAGE + off) * D;
+    if (e < h8) {
+      const bf16x8 a8 = ld8(src + 8 * e), b8 = ld8(src + half + 8 * e), wa = ld8(w + 8 * e), wb = ld8(w + half + 8 * e);
+      bf16x8 x8, y8;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        const float a = bf2f(a8[k]) * r * bf2f(wa[k]), b = bf2f(b8[k]) * r * bf2f(wb[k]);
+        const float c = cs[8 * e + k], s = cs[half + 8 * e + k];
+        x8[k] = f2bf(a * c - b * s);
+        y8[k] = f2bf(b * c + a * s);
+      }
+      st8(dst + 8 * e, x8);
+      st8(dst + half + 8 * e, y8);
+    } else {
+      const int d = half + 8 * e;  // = R + 8 (e - h8)
+      const bf16x8 a8 = ld8(src + d), wa = ld8(w + d);
+      bf16x8 x8;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) x8[k] = f2bf(bf2f(a8[k]) * r * bf2f(wa[k]));
+      st8(dst + d, x8);
+    }
+  }
+  if (slot >= 0) {
+    const bf16_t* vsrc = row + v_off;
+    for (int i = 8 * tid; i < G * V; i += 8 * 256) {
+      const int c = i / V, v = i % V;
+      const bf16x8 raw = ld8(vsrc + i);
+      if (v_transposed) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) vcache[((page * G + c) * V + v + e) * PAGE + off] = raw[e];
+      } else {
+        st8(vcache + ((page * G + c) * PAGE + off) * V + v, raw);
+      }
+    }
+  }
+}
+
 // x[t, i] *= sigmoid(gate[t, i]) over rows of n elements (x contiguous, gate rows gate_stride apart)
 template <typename T>
 __global__ void __launch_bounds__(256) sigmoid_gate_rows_kernel(T* __restrict__ x, const T* __restrict__ gate,
@@ -289,8 +430,8 @@ __global__ void __launch_bounds__(256) window_attn_kernel(
     const int* __restrict__ block_tables, int max_pages, const int* __restrict__ cu_q,
     const int* __restrict__ ctx_len, const T* __restrict__ mix, const T* __restrict__ gate, int64_t gate_stride,
     int gate_elem, const T* __restrict__ r1, const T* __restrict__ r2,
-    T* __restrict__ out, float* __restrict__ part_acc, float* __restrict__ part_ml, AttnShape sh, float scale, float softcap, float slope_exp, int window, int keep, int sink,
-    int nsplit) {
+    T* __restrict__ out, float* __restrict__ part_acc, float* __restrict__ part_ml, AttnShape sh, float scale, float softcap, float slope_exp, int window, int keep, int chunk,
+    int sink, int nsplit) {
   extern __shared__ float lds[];
   const int H = sh.H, G = sh.G, D = sh.D, V = sh.V, BQ = sh.BQ;
   const int b = blockIdx.y, split = blockIdx.z, tid = threadIdx.x;
@@ -328,7 +469,7 @@ __global__ void __launch_bounds__(256) window_attn_kernel(
   // visible keys of the tile: [j_lo, j_hi) and the kept first ones; pages [0, p_keep) and [p_lo, p_hi), this split's
   // share of them
   const int j_hi = pos0 + nq;
-  const int j_lo = window > 0 ? max(0, pos0 - window + 1) : 0;
+  const int j_lo = first_key(pos0, window, chunk);
   const int p_lo = j_lo / PAGE, p_hi = (j_hi + PAGE - 1) / PAGE;
   const int p_keep = min((max(keep, 0) + PAGE - 1) / PAGE, p_lo);
   const int n_pages = p_keep + p_hi - p_lo;
@@ -379,7 +520,7 @@ __global__ void __launch_bounds__(256) window_attn_kernel(
         s = S1[e];
       }
       const int dist = pos0 + qi - (jb + kj);
-      const bool ok = qi < nq && dist >= 0 && (window <= 0 || dist < window || jb + kj < keep);
+      const bool ok = qi < nq && dist >= 0 && (jb + kj >= first_key(pos0 + qi, window, chunk) || jb + kj < keep);
       S2[e] = ok ? s : -INFINITY;
     }
     __syncthreads();
@@ -466,7 +607,7 @@ __global__ void __launch_bounds__(MAXT) window_attn_mfma_kernel(
     const int* __restrict__ ctx_len, const bf16_t* __restrict__ mix, const bf16_t* __restrict__ gate,
     int64_t gate_stride, int gate_elem, const bf16_t* __restrict__ r1, const bf16_t* __restrict__ r2,
     bf16_t* __restrict__ out, int Hall, int Gall, int H, float scale, float softcap,
-    float slope_exp, int window, int keep, int sink) {
+    float slope_exp, int window, int keep, int chunk, int sink) {
   constexpr int D = DK * 32, V = VT_ * 16, KS = D + 8, VS = PAGE + 8, SS = PAGE + 4;
   // this workgroup's heads: hbase .. hbase + H - 1 of Hall (several groups only without head mixing), and their G
   // key/value heads from c0 on
@@ -513,7 +654,7 @@ __global__ void __launch_bounds__(MAXT) window_attn_mfma_kernel(
     for (int vt = 0; vt < VT_; ++vt) acc[hh][vt] = (f32x4){0.f, 0.f, 0.f, 0.f};
   }
   const int j_hi = pos0 + nq;
-  const int j_lo = window > 0 ? max(0, pos0 - window + 1) : 0;
+  const int j_lo = first_key(pos0, window, chunk);
   const int p_lo = j_lo / PAGE, p_hi = (j_hi + PAGE - 1) / PAGE;
   const int p_keep = min((max(keep, 0) + PAGE - 1) / PAGE, p_lo);  // pages of kept first tokens below the window's
   const float inv_cap = softcap > 0.f ? 1.f / softcap : 0.f;
@@ -576,8 +717,9 @@ __global__ void __launch_bounds__(MAXT) window_attn_mfma_kernel(
         m1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a, b1, m1, 0, 0, 0);
       }
       const int d0 = pos0 + qi - (jb + r16), d1 = d0 - 16;
-      const bool ok0 = qi < nq && d0 >= 0 && (window <= 0 || d0 < window || jb + r16 < keep);
-      const bool ok1 = qi < nq && d1 >= 0 && (window <= 0 || d1 < window || jb + 16 + r16 < keep);
+      const int lo = first_key(pos0 + qi, window, chunk);
+      const bool ok0 = qi < nq && d0 >= 0 && (jb + r16 >= lo || jb + r16 < keep);
+      const bool ok1 = qi < nq && d1 >= 0 && (jb + 16 + r16 >= lo || jb + 16 + r16 < keep);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int h = 4 * quad + i;
@@ -677,7 +819,7 @@ int launch_mfma(dim3 grid, int nthr, size_t lds, hipStream_t st, const bf16_t* q
                 const int* bt, int max_pages, const int* cu_q, const int* ctx_len, const bf16_t* mix,
                 const bf16_t* gate, int64_t gate_stride, int gate_elem, const bf16_t* r1, const bf16_t* r2, bf16_t* out,
                 int Hall, int Gall, int H, int D, int V, float scale, float softcap, float slope_exp, int window,
-                int keep, int sink) {
+                int keep, int chunk, int sink) {
 #define MFMA_CASE(DKV, VTV)                                                                                        \
   do {                                                                                                             \
     static bool raised = false; /* once per kernel: no attribute call inside a stream capture later */            \
@@ -688,7 +830,7 @@ int launch_mfma(dim3 grid, int nthr, size_t lds, hipStream_t st, const bf16_t* q
     }                                                                                                              \
     hipLaunchKernelGGL((window_attn_mfma_kernel<HPW, DKV, VTV, MAXT>), grid, dim3(nthr), lds, st, q, kc, vc, bt,   \
                        max_pages, cu_q, ctx_len, mix, gate, gate_stride, gate_elem, r1, r2, out, Hall, Gall, H,    \
-                       scale, softcap, slope_exp, window, keep, sink);                                             \
+                       scale, softcap, slope_exp, window, keep, chunk, sink);                                      \
   } while (0)
   if (D == 64 && V == 32) MFMA_CASE(2, 2);
   else if (D == 64 && V == 64) MFMA_CASE(2, 4);
@@ -791,6 +933,31 @@ extern "C" int areal_qkv_vnorm_cache_write(const void* proj, int64_t row_stride,
   return (int)hipGetLastError();
 }
 
+// proj rows: q heads | k heads from the pointer on, values at column v_off. qw [H D], kw [G D]. table fp32 [n_pos, R] (R = 0:
+// no rotation).
+extern "C" int areal_qk_rows_norm_cache_write(const void* proj, int64_t row_stride, int v_off, const void* qw,
+                                              const void* kw, const int* positions, const float* table, int n_pos, int R,
+                                              const int64_t* slots, void* q_out, void* kcache, void* vcache, int T, int H,
+                                              int G, int D, int V, float eps, int v_transposed, int dt, hipStream_t st) {
+  if (T == 0) return 0;
+  if (R < 0 || R > D || R % 2 != 0 || (R > 0 && (n_pos < 1 || !table || !positions)) || !qw || !kw) return -1;
+  if (dt == 0 && D % 8 == 0 && V % 8 == 0 && R % 16 == 0 && v_off % 8 == 0 && row_stride % 8 == 0 &&
+      (((uintptr_t)proj | (uintptr_t)qw | (uintptr_t)kw) % 16) == 0) {
+    hipLaunchKernelGGL(qk_rows_norm_cache_write_vec_kernel, dim3(T), dim3(256), 0, st, (const bf16_t*)proj, row_stride,
+                       v_off, (const bf16_t*)qw, (const bf16_t*)kw, positions, table, n_pos, R, slots, (bf16_t*)q_out,
+                       (bf16_t*)kcache, (bf16_t*)vcache, H, G, D, V, eps, v_transposed);
+    return (int)hipGetLastError();
+  }
+#define ROWS(TT)                                                                                                     \
+  hipLaunchKernelGGL(qk_rows_norm_cache_write_kernel<TT>, dim3(T), dim3(256), 0, st, (const TT*)proj, row_stride, v_off, \
+                     (const TT*)qw, (const TT*)kw, positions, table, n_pos, R, slots, (TT*)q_out, (TT*)kcache,        \
+                     (TT*)vcache, H, G, D, V, eps, v_transposed)
+  if (dt == 0) ROWS(bf16_t);
+  else ROWS(float);
+#undef ROWS
+  return (int)hipGetLastError();
+}
+
 // x [rows, n] contiguous <- x * sigmoid(gate), gate rows gate_stride apart
 extern "C" int areal_sigmoid_gate_rows(void* x, const void* gate, int64_t gate_stride, int64_t rows, int n, int dt,
                                        hipStream_t st) {
@@ -821,8 +988,8 @@ extern "C" int areal_window_attn(const void* q, const void* kcache, const void* 
                                  int max_pages, const int* cu_q, const int* ctx_len, const void* mix, const void* gate,
                                  int64_t gate_stride, int gate_elem, const void* r1, const void* r2, void* out,
                                  float* part_acc, float* part_ml, int B, int max_q, int T, int H, int G, int D, int V,
-                                 int bq, float scale, float softcap, float slope_exp, int window, int keep, int sink,
-                                 int nsplit, int dt, int matrix_cores, hipStream_t st) {
+                                 int bq, float scale, float softcap, float slope_exp, int window, int keep, int chunk,
+                                 int sink, int nsplit, int dt, int matrix_cores, hipStream_t st) {
   if (B == 0 || T == 0) return 0;
   if (G <= 0 || H % G != 0 || bq <= 0 || nsplit < 1 || (r1 == nullptr) != (r2 == nullptr)) return -1;
   if (matrix_cores && dt == 0 && nsplit == 1 && max_q > 1 && mfma_usable(H, G, D, V, mix != nullptr)) {
@@ -833,7 +1000,7 @@ extern "C" int areal_window_attn(const void* q, const void* kcache, const void* 
 #define MFMA_ARGS                                                                                                  \
   mgrid, nthr, mlds, st, (const bf16_t*)q, (const bf16_t*)kcache, (const bf16_t*)vcache, block_tables, max_pages,   \
       cu_q, ctx_len, (const bf16_t*)mix, (const bf16_t*)gate, gate_stride, gate_elem, (const bf16_t*)r1,            \
-      (const bf16_t*)r2, (bf16_t*)out, H, G, hb, D, V, scale, softcap, slope_exp, window, keep, sink
+      (const bf16_t*)r2, (bf16_t*)out, H, G, hb, D, V, scale, softcap, slope_exp, window, keep, chunk, sink
     if (hpw == 4) return launch_mfma<4, 256>(MFMA_ARGS);
     if (hpw == 2) return launch_mfma<2, 512>(MFMA_ARGS);
     return launch_mfma<1, 512>(MFMA_ARGS);
@@ -855,7 +1022,7 @@ extern "C" int areal_window_attn(const void* q, const void* kcache, const void* 
     hipLaunchKernelGGL(window_attn_kernel<TT>, grid, dim3(256), lds, st, (const TT*)q, (const TT*)kcache,            \
                        (const TT*)vcache, block_tables, max_pages, cu_q, ctx_len, (const TT*)mix, (const TT*)gate,   \
                        gate_stride, gate_elem, (const TT*)r1, (const TT*)r2, (TT*)out, part_acc, part_ml, sh, scale, \
-                       softcap, slope_exp, window, keep, sink, nsplit);                                             \
+                       softcap, slope_exp, window, keep, chunk, sink, nsplit);                                      \
     if (nsplit > 1)                                                                                                  \
       hipLaunchKernelGGL(window_attn_combine_kernel<TT>, dim3(T, H), dim3(128), 0, st, part_acc, part_ml,           \
                          (const TT*)gate, gate_stride, gate_elem, (TT*)out, H, V, nsplit);                          \
