@@ -36,7 +36,8 @@ def workspace_floats(rows: int, nsplit: int, heads: int, vdim: int) -> Tuple[int
 def mixed_attention(q: torch.Tensor, kcache: torch.Tensor, vcache_t: torch.Tensor, block_tables: torch.Tensor,
                     cu_q: torch.Tensor, ctx_len: torch.Tensor, max_q: int, scale: float, mix: torch.Tensor,
                     out: Optional[torch.Tensor] = None, out_scale: float = 1.0, nsplit: int = 1,
-                    workspace: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> torch.Tensor:
+                    workspace: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
+                    matrix_cores: bool = True) -> torch.Tensor:
     """q [T, H, D] (row b owns tokens cu_q[b]:cu_q[b+1], the LAST positions of its context of ctx_len[b] tokens, whose
     keys / values are in the cache already), mix [H, H]. Writes out_scale * o into `out` ([T, H Dv], a view with unit
     stride along the columns; None: a new tensor) and returns it. nsplit > 1 (single-query rows): the keys of a row are
