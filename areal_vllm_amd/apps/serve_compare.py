@@ -17,6 +17,10 @@ compared with the same kind of twin.
 The Zusotar design (sublayers between two RMS norms, a learned average over depth; window attention with a logarithmic
 distance penalty, latent attention with a sink and gated linear attention in turn; group-routed + shared gated
 experts, the first layer a gated MLP) is compared with the same kind of twin.
+
+The Gusolix design (layer norm on sublayer outputs, short convolutions ahead of every sublayer; attention inside chunks of
+positions with keys as values, attention with mixed weights beside gated linear attention, and selective scan in turn;
+gated MLP) is compared with the dense Qwen3-style twin.
 """
 import json
 import sys
@@ -52,6 +56,13 @@ ZUSOTAR_SIZES = {
     "w1024": (1024, 4, 8, 2, 128, 512, 64, 32, 64, 256, 4, 128, 256, 16, 16, 2, 4, 2, 512, 512),
     "w2048": (2048, 4, 16, 4, 128, 1024, 128, 64, 128, 512, 8, 128, 256, 16, 32, 4, 4, 2, 768, 768),
     "w4096": (4096, 3, 32, 8, 128, 1024, 128, 64, 128, 512, 16, 128, 256, 32, 64, 4, 8, 4, 1024, 1024),
+}
+# Gusolix: width, layers, heads, kv heads, head size (keys = values) of both attention kinds, chunk, gla heads / key size /
+# value size / decay rank, inner size / state / step rank / taps of the selective scan, feed-forward
+GUSOLIX_SIZES = {
+    "w1024": (1024, 6, 8, 2, 128, 512, 4, 128, 256, 16, 2048, 16, 64, 4, 4096),
+    "w2048": (2048, 6, 16, 4, 128, 1024, 8, 128, 256, 16, 4096, 16, 128, 4, 8192),
+    "w4096": (4096, 3, 32, 8, 128, 1024, 16, 128, 256, 32, 8192, 16, 256, 4, 14336),
 }
 VOCAB = 32768
 
@@ -118,6 +129,24 @@ def zusotar_dict(width, layers, heads, kv, dim, window, ldim, rot, lvdim, rank, 
         ls.append({"type": kind, "mixer": json.loads(json.dumps(mixer)), "mlp": mlp})
     return {"architecture": "Zusotar", "layers": ls, "max_positions": positions, "norm": {"eps": 1e-5},
             "residual_mult": 0.5, "vocab": VOCAB, "width": width}
+
+
+def gusolix_dict(width, layers, heads, kv, dim, chunk, gheads, gdim, gvdim, grank, inner, state, srank, taps, ff) -> Dict[str, Any]:
+    mixers = [
+        ("attention", {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": chunk},
+                       "rot": {"base": 500000.0, "dims": dim,
+                               "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}),
+        ("parallel", {"left": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5},
+                      "right": {"heads": gheads, "dim": gdim, "vdim": gvdim, "tau": 12.0, "decay_rank": grank},
+                      "left_scale": 0.75, "right_scale": 0.6}),
+        ("mamba1", {"inner": inner, "state": state, "dt_rank": srank, "conv": taps}),
+    ]
+    ls = []
+    for i in range(layers):
+        kind, mixer = mixers[i % 3]
+        ls.append({"type": kind, "mixer": json.loads(json.dumps(mixer)), "mlp": {"kind": "dense", "ff": ff}})
+    return {"architecture": "Gusolix", "canon": {"taps": 4}, "embedding": {"scale": float(width) ** 0.5}, "layers": ls,
+            "norm": {"eps": 1e-5}, "vocab": VOCAB, "width": width}
 
 
 def moe_twin_config(lcfg, width, layers, heads, experts, top):
@@ -222,6 +251,27 @@ def run_zusotar(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: i
     return 0
 
 
+def run_gusolix(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: int, dev) -> int:
+    from ..models.config import ModelConfig
+
+    for name in sizes:
+        z = GUSOLIX_SIZES[name]
+        width, layers, heads, kv, dim = z[:5]
+        gcfg = ModelConfig.from_hf_dict(gusolix_dict(*z))
+        tcfg = twin_config(gcfg, width, layers, heads, kv, dim)
+        row = {"design": "gusolix", "size": name, "width": width, "layers": layers, "heads": heads, "kv_heads": kv,
+               "head_dim": dim, "chunk": z[5], "gla_heads": z[6], "gla_dim": z[7], "gla_vdim": z[8], "inner": z[10],
+               "state": z[11], "ff": z[14], "twin_ff": tcfg.intermediate_size, "prompts": n_prompts,
+               "prompt_len": prompt_len, "new_tokens": new_tokens, "dtype": "bf16", "data": "synthetic"}
+        for label, cfg in (("gusolix", gcfg), ("qwen3_twin", tcfg)):
+            m = measure(cfg, n_prompts, prompt_len, new_tokens, dev)
+            row[label] = {"params_no_embedding": cfg.n_params(with_embedding=False), **{k: round(v, 1) for k, v in m.items()}}
+        row["prefill_ratio"] = round(row["gusolix"]["prefill_tok_s"] / row["qwen3_twin"]["prefill_tok_s"], 3)
+        row["decode_ratio"] = round(row["gusolix"]["decode_tok_s"] / row["qwen3_twin"]["decode_tok_s"], 3)
+        print(json.dumps(row), flush=True)
+    return 0
+
+
 def run_lufivik(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: int, dev) -> int:
     from ..models.config import ModelConfig
 
@@ -252,6 +302,8 @@ def run(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: int, devi
         return run_pobelorn(sizes, n_prompts, prompt_len, new_tokens, dev)
     if design == "zusotar":
         return run_zusotar(sizes, n_prompts, prompt_len, new_tokens, dev)
+    if design == "gusolix":
+        return run_gusolix(sizes, n_prompts, prompt_len, new_tokens, dev)
     for name in sizes:
         width, layers, heads, kv, dim, ff, window = SIZES[name]
         kcfg = ModelConfig.from_hf_dict(kuzanex_dict(width, layers, heads, kv, dim, ff, window))

@@ -1052,6 +1052,7 @@ class MixedAttentionMixer(nn.Module):
         self.k_norm = nn.Parameter(torch.ones(kv_heads * dim, dtype=dtype, device=device))
         self.talk = nn.Parameter(torch.eye(heads, dtype=dtype, device=device))
         self.max_context = 1 << 30
+        self.decode_mc = False  # decoding runs the matrix-core kernels (`alloc_cache`)
 
     def in_rows(self) -> int:
         return (self.H + self.G) * self.D + self.G * self.V
@@ -1063,19 +1064,24 @@ class MixedAttentionMixer(nn.Module):
         return self.G, self.D, self.V
 
     def alloc_cache(self, num_pages: int, dtype, device):
+        self.decode_mc = xattn.matrix_cores_serve(self.H, self.G, self.D, self.V, dtype, device)[1]
         return xattn.alloc_mixed_cache(num_pages, self.G, self.D, self.V, dtype, device)
 
     def prepare(self, n_pos: int, tables, device):
         self.max_context = int(n_pos) - 1
 
+    def decode_splits(self, batch: int) -> int:
+        return xattn.decode_splits(batch, self.max_context, self.G, self.decode_mc)
+
     def workspace_floats(self, batch: int):
-        return xattn.workspace_floats(batch, xattn.decode_splits(batch, self.max_context), self.H, self.V)
+        keys = (self.max_context // xattn.PAGE_SIZE + 2) * xattn.PAGE_SIZE if self.decode_mc else 0
+        return xattn.workspace_floats(batch, self.decode_splits(batch), self.H, self.V, keys)
 
     def run(self, proj: torch.Tensor, st: StepTensors, cache, out: torch.Tensor, out_scale: float) -> torch.Tensor:
         kc, vc = cache
         q = wattn.qk_rows_norm_cache_write(proj, (self.H + self.G) * self.D, self.q_norm, self.k_norm, None, None, st.slots,
                                            kc, vc, self.H, self.eps, v_transposed=True)
-        nsplit = xattn.decode_splits(proj.shape[0], self.max_context) if st.max_q == 1 else 1
+        nsplit = self.decode_splits(proj.shape[0]) if st.max_q == 1 else 1
         return xattn.mixed_attention(q, kc, vc, st.block_tables, st.cu_q, st.ctx_len, st.max_q, self.scale, self.talk, out,
                                      out_scale, nsplit, st.workspace)
 

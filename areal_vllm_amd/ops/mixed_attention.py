@@ -13,7 +13,7 @@ from typing import Optional, Tuple
 import torch
 
 from . import _lib as L
-from .attention import PAGE_SIZE
+from .attention import PAGE_SIZE, decode_num_splits
 
 
 def alloc_mixed_cache(num_pages: int, n_kv_heads: int, k_dim: int, v_dim: int, dtype, device
@@ -22,15 +22,28 @@ def alloc_mixed_cache(num_pages: int, n_kv_heads: int, k_dim: int, v_dim: int, d
             torch.zeros(num_pages, n_kv_heads, v_dim, PAGE_SIZE, dtype=dtype, device=device))
 
 
-def decode_splits(batch: int, max_context: int) -> int:
-    """Key-range splits of a decode launch: about two workgroups per compute unit, down to one page each."""
+def matrix_cores_serve(heads: int, kv_heads: int, k_dim: int, v_dim: int, dtype, device) -> Tuple[bool, bool]:
+    """Whether (prompt portions, decoding) of these sizes run the matrix-core kernels: bf16, key and value sizes 64 / 128;
+    4, 8, 16 or 32 heads for prompts; at most 64 heads and 16 per key/value head for decoding."""
+    if dtype != torch.bfloat16 or torch.device(device).type != "cuda":
+        return False, False
+    m = int(L.lib().areal_mixed_attn_matrix_cores(L.c_int(heads), L.c_int(kv_heads), L.c_int(k_dim), L.c_int(v_dim)))
+    return bool(m & 1), bool(m & 2)
+
+
+def decode_splits(batch: int, max_context: int, kv_heads: int = 1, matrix_cores: bool = False) -> int:
+    """Key-range splits of a decode launch: about two workgroups per compute unit, down to one page each; the matrix-core
+    kernels have a workgroup per key/value head and share a split's pages among four waves."""
+    if matrix_cores:
+        return decode_num_splits(batch, kv_heads, max_context)
     pages = max(1, (max_context + PAGE_SIZE - 1) // PAGE_SIZE)
     return int(max(1, min(512 // max(1, batch), pages, 32)))
 
 
-def workspace_floats(rows: int, nsplit: int, heads: int, vdim: int) -> Tuple[int, int]:
-    """Floats of the two workspace buffers (partial sums, partial softmax statistics) of a launch over `rows` tokens."""
-    return (rows * nsplit * heads * vdim if nsplit > 1 else 0), rows * nsplit * heads * 2
+def workspace_floats(rows: int, nsplit: int, heads: int, vdim: int, score_keys: int = 0) -> Tuple[int, int]:
+    """Floats of the two workspace buffers of a launch over `rows` tokens: partial sums and (`score_keys` per row and head)
+    scores, partial softmax statistics."""
+    return (rows * nsplit * heads * vdim if nsplit > 1 else 0) + rows * heads * score_keys, rows * nsplit * heads * 2
 
 
 def mixed_attention(q: torch.Tensor, kcache: torch.Tensor, vcache_t: torch.Tensor, block_tables: torch.Tensor,
@@ -41,7 +54,7 @@ def mixed_attention(q: torch.Tensor, kcache: torch.Tensor, vcache_t: torch.Tenso
     """q [T, H, D] (row b owns tokens cu_q[b]:cu_q[b+1], the LAST positions of its context of ctx_len[b] tokens, whose
     keys / values are in the cache already), mix [H, H]. Writes out_scale * o into `out` ([T, H Dv], a view with unit
     stride along the columns; None: a new tensor) and returns it. nsplit > 1 (single-query rows): the keys of a row are
-    shared out over that many workgroups."""
+    shared out over that many workgroups. `matrix_cores` False: always the any-size kernel."""
     T, H, D = q.shape
     G, V = kcache.shape[1], vcache_t.shape[2]
     B = cu_q.numel() - 1
@@ -52,10 +65,32 @@ def mixed_attention(q: torch.Tensor, kcache: torch.Tensor, vcache_t: torch.Tenso
         assert q.is_contiguous() and kcache.dtype == q.dtype and vcache_t.dtype == q.dtype and mix.dtype == q.dtype
         assert block_tables.dtype == torch.int32 and block_tables.is_contiguous() and mix.is_contiguous()
         assert cu_q.dtype == torch.int32 and ctx_len.dtype == torch.int32 and (nsplit == 1 or max_q == 1)
-        na, nm = workspace_floats(T, nsplit, H, V)
+        prompt_mc, decode_mc = matrix_cores_serve(H, G, D, V, q.dtype, q.device) if matrix_cores else (False, False)
+        aligned = out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0
+        decode_mc = decode_mc and max_q == 1
+        prompt_mc = prompt_mc and max_q > 1 and nsplit == 1 and aligned
+        max_pages = block_tables.shape[1]
+        na, nm = workspace_floats(T, nsplit, H, V, max_pages * PAGE_SIZE if decode_mc else 0)
         if workspace is None or workspace[0].numel() < na or workspace[1].numel() < nm:
             workspace = (torch.empty(na, dtype=torch.float32, device=q.device),
                          torch.empty(nm, dtype=torch.float32, device=q.device))
+        acc, stats = workspace
+        if decode_mc:
+            assert T == B
+            ns = T * H * max_pages * PAGE_SIZE  # scores first, then the partial sums
+            L.check(L.lib().areal_mixed_attn_decode(
+                L.ptr(q), L.ptr(kcache), L.ptr(vcache_t), L.ptr(block_tables), L.c_int(max_pages), L.ptr(ctx_len), L.ptr(mix),
+                L.ptr(acc), L.ptr(stats), L.ptr(out), L.c_int64(out.stride(0)), L.ptr(acc[ns:]) if nsplit > 1 else None,
+                L.c_int(B), L.c_int(H), L.c_int(G), L.c_int(D), L.c_int(V), L.c_float(scale), L.c_float(out_scale),
+                L.c_int(int(nsplit)), L.stream_ptr()), "mixed_attn_decode")
+            return out
+        if prompt_mc:
+            L.check(L.lib().areal_mixed_attn_prompt(
+                L.ptr(q), L.ptr(kcache), L.ptr(vcache_t), L.ptr(block_tables), L.c_int(max_pages), L.ptr(cu_q),
+                L.ptr(ctx_len), L.ptr(mix), L.ptr(stats), L.ptr(out), L.c_int64(out.stride(0)), L.c_int(B),
+                L.c_int(int(max_q)), L.c_int(T), L.c_int(H), L.c_int(G), L.c_int(D), L.c_int(V), L.c_float(scale),
+                L.c_float(out_scale), L.stream_ptr()), "mixed_attn_prompt")
+            return out
         want = 1 if max_q == 1 else 16
         while want > 1 and want // 2 >= max_q:
             want //= 2
@@ -63,9 +98,9 @@ def mixed_attention(q: torch.Tensor, kcache: torch.Tensor, vcache_t: torch.Tenso
         if bq <= 0:
             raise RuntimeError(f"mixed attention: {H} heads of size {D} / {V} do not fit the kernel's tile memory")
         L.check(L.lib().areal_mixed_attn(
-            L.ptr(q), L.ptr(kcache), L.ptr(vcache_t), L.ptr(block_tables), L.c_int(block_tables.shape[1]), L.ptr(cu_q),
-            L.ptr(ctx_len), L.ptr(mix), L.ptr(workspace[1]), L.ptr(out), L.c_int64(out.stride(0)),
-            L.ptr(workspace[0]) if nsplit > 1 else None, L.c_int(B), L.c_int(int(max_q)), L.c_int(T), L.c_int(H),
+            L.ptr(q), L.ptr(kcache), L.ptr(vcache_t), L.ptr(block_tables), L.c_int(max_pages), L.ptr(cu_q),
+            L.ptr(ctx_len), L.ptr(mix), L.ptr(stats), L.ptr(out), L.c_int64(out.stride(0)),
+            L.ptr(acc) if nsplit > 1 else None, L.c_int(B), L.c_int(int(max_q)), L.c_int(T), L.c_int(H),
             L.c_int(G), L.c_int(D), L.c_int(V), L.c_int(bq), L.c_float(scale), L.c_float(out_scale), L.c_int(int(nsplit)),
             L.c_int(L.dtype_flag(q)), L.stream_ptr()), "mixed_attn")
         return out

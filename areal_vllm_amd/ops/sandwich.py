@@ -118,7 +118,25 @@ def norm_add_conv(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, bias: 
                   conv: Optional[Tuple[Optional[torch.Tensor], Optional[torch.Tensor]]], cu_q: torch.Tensor,
                   first_pos: torch.Tensor, state_slots: torch.Tensor) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
     """x + LN(y; weight, bias) on the fp32 stream x [T, W] (y [T, W] in the compute dtype; x itself may be overwritten) and,
-    with `conv` = (weight, state), `stream_conv` of the sum in y's dtype. Returns (new stream, convolved stream or None)."""
+    with `conv` = (weight, state), `stream_conv` of the sum in y's dtype: one launch for up to four taps and 8192 channels.
+    Returns (new stream, convolved stream or None)."""
+    if (conv is not None and conv[0] is not None and L.use_hip(x)
+            and L.lib().areal_norm_add_conv_serves(L.c_int(x.shape[1]), L.c_int(conv[0].shape[1]))):
+        T, W = x.shape
+        cw, state = conv
+        taps = cw.shape[1]
+        assert x.is_contiguous() and y.is_contiguous() and y.shape == x.shape and cw.is_contiguous() and cw.shape[0] == W
+        assert weight.dtype == y.dtype and bias.dtype == y.dtype and cw.dtype == y.dtype
+        assert weight.numel() == W and bias.numel() == W
+        assert taps == 1 or (state.shape[1:] == (taps - 1, W) and state.dtype == torch.float32 and state.is_contiguous())
+        assert cu_q.dtype == torch.int32 and first_pos.dtype == torch.int32 and state_slots.dtype == torch.int32
+        if all(t.data_ptr() % 16 == 0 for t in (x, y, weight, bias)):
+            xo, hc = torch.empty_like(x), torch.empty_like(y)
+            L.check(L.lib().areal_norm_add_conv(
+                L.ptr(x), L.ptr(y), L.ptr(weight), L.ptr(bias), L.ptr(cw), L.ptr(state), L.ptr(cu_q), L.ptr(first_pos),
+                L.ptr(state_slots), L.ptr(xo), L.ptr(hc), L.c_int(cu_q.numel() - 1), L.c_int(T), L.c_int(W), L.c_int(taps),
+                L.c_float(eps), L.c_int(L.dtype_flag(y)), L.stream_ptr()), "norm_add_conv")
+            return xo, hc
     x, _, _ = gated_norm_add(x, y, None, weight, bias, None, eps)
     return x, (None if conv is None else stream_conv(x, conv[0], conv[1], cu_q, first_pos, state_slots, y.dtype))
 

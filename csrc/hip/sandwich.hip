@@ -7,6 +7,7 @@
 //   canon_conv        out_t = h_t + sum_j w[:, j] h_(t - taps + 1 + j); history before a row's first token comes
 //                     from the row's state slot (zeros before position 0); the slot then takes the row's last inputs
 //   conv_silu         out_t = silu(sum_j w[:, j] h_(t - taps + 1 + j) + bias), the same history
+//   norm_add_conv     xo = x + LN(y; w, b) and xo + conv(xo) in one launch
 //   embed_bigram_norm x = LN(E[tok] + B[(prev * a + tok * b) mod n])   (row n of B at position 0)
 //
 // T is the storage type (bf16 / fp32) of weights and of the sublayers' outputs; the stream x is fp32.
@@ -223,6 +224,258 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(const TI* __restrict__
   }
 }
 
+// Eight consecutive elements (16-byte aligned) as floats, and back.
+template <typename T> DEVINL void ld8f(const T* p, float (&v)[8]);
+template <> DEVINL void ld8f<bf16_t>(const bf16_t* p, float (&v)[8]) {
+  const bf16x8 x = ld8(p);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = bf2f(x[e]);
+}
+template <> DEVINL void ld8f<float>(const float* p, float (&v)[8]) {
+  const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    v[e] = a[e];
+    v[4 + e] = b[e];
+  }
+}
+template <typename T> DEVINL void st8f(T* p, const float (&v)[8]);
+template <> DEVINL void st8f<bf16_t>(bf16_t* p, const float (&v)[8]) {
+  bf16x8 x;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) x[e] = f2bf(v[e]);
+  st8(p, x);
+}
+template <> DEVINL void st8f<float>(float* p, const float (&v)[8]) {
+  *reinterpret_cast<f32x4*>(p) = (f32x4){v[0], v[1], v[2], v[3]};
+  *reinterpret_cast<f32x4*>(p + 4) = (f32x4){v[4], v[5], v[6], v[7]};
+}
+
+// The tokens [lo, hi) that the workgroup of tile [t0, t0 + R) of the packed batch serves when a convolution with K tokens of
+// history runs along the rows: those of the tile, but a row's first K tokens - whose history reaches into the row's state
+// slot - all belong to the tile of the row's first token, so that the slot has one reader. That workgroup rewrites the slot.
+DEVINL void conv_span(const int* __restrict__ cu_q, int B, int T, int t0, int R, int K, int& lo, int& hi, int& row) {
+  row = row_of(cu_q, B, t0);
+  lo = t0;
+  hi = min(t0 + R, min(T, cu_q[B]));
+  const int q0 = cu_q[row];
+  if (t0 > q0 && t0 - q0 < K) lo = min(q0 + K, cu_q[row + 1]);  // those are another tile's
+  if (hi > lo) {
+    const int last = row_of(cu_q, B, hi - 1), s0 = cu_q[last];
+    if (s0 >= t0 && hi - s0 < K) hi = min(s0 + K, cu_q[last + 1]);
+  }
+}
+
+// silu(conv(h) + bias) of rows in the storage type: eight channels a thread, R tokens a workgroup, the history in registers.
+// (Rows of a multiple of 8 channels, 16-byte aligned; the fallback is causal_conv_kernel.)
+template <typename T, int K>
+__global__ void __launch_bounds__(256) conv_silu_vec_kernel(const T* __restrict__ h, int64_t h_stride,
+                                                            const T* __restrict__ w, const T* __restrict__ bias,
+                                                            float* __restrict__ state, const int* __restrict__ cu_q,
+                                                            const int* __restrict__ first_pos,
+                                                            const int* __restrict__ state_slots, T* __restrict__ out,
+                                                            int B, int Tn, int W, int R) {
+  const int c = 8 * (blockIdx.y * 256 + threadIdx.x);
+  int lo, hi, b;
+  conv_span(cu_q, B, Tn, blockIdx.x * R, R, K, lo, hi, b);
+  if (lo >= hi || c >= W) return;
+  float cw[K + 1][8], bb[8], ring[K + 1][8];
+#pragma unroll
+  for (int j = 0; j <= K; ++j)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) cw[j][e] = ldf<T>(w, (size_t)(c + e) * (K + 1) + j);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) bb[e] = bias ? ldf<T>(bias, c + e) : 0.f;
+  bool fresh_row = true;  // the ring has to be filled for the token at hand
+  for (int t = lo; t < hi; ++t) {
+    while (t >= cu_q[b + 1]) {
+      ++b;
+      fresh_row = true;
+    }
+    const int q0 = cu_q[b], q1 = cu_q[b + 1], slot = state_slots[b];
+    float* sl = state + (size_t)max(slot, 0) * K * W + c;
+    if (fresh_row) {
+      fresh_row = false;
+#pragma unroll
+      for (int j = 0; j < K; ++j) {
+        const int p = t - K + j;  // t is the row's first token, or at least K tokens into it
+        if (p >= q0) ld8f<T>(h + (size_t)p * h_stride + c, ring[j]);
+        else if (slot >= 0 && first_pos[b] + p - q0 >= 0) ld8f<float>(sl + (size_t)(K + p - q0) * W, ring[j]);
+        else
+#pragma unroll
+          for (int e = 0; e < 8; ++e) ring[j][e] = 0.f;
+      }
+    }
+    ld8f<T>(h + (size_t)t * h_stride + c, ring[K]);
+    float o[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float a = bb[e];
+#pragma unroll
+      for (int j = 0; j <= K; ++j) a += cw[j][e] * ring[j][e];
+      o[e] = a / (1.f + expf(-a));
+    }
+    st8f<T>(out + (size_t)t * W + c, o);
+    if (K > 0 && t == max(lo, q0) && q0 >= lo && slot >= 0) {
+      // the slot's entry k becomes the input K - k tokens before the next step's first one; entries behind it are read first
+      const int n = q1 - q0;
+#pragma unroll
+      for (int k = 0; k < K; ++k) {
+        const int p = n - K + k;
+        float v[8];
+        if (p >= 0) {
+          ld8f<T>(h + (size_t)(q0 + p) * h_stride + c, v);
+        } else {
+#pragma unroll
+          for (int j = 0; j < K; ++j)
+            if (j == K + p) {
+#pragma unroll
+              for (int e = 0; e < 8; ++e) v[e] = ring[j][e];
+            }
+        }
+        st8f<float>(sl + (size_t)k * W, v);
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < K; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ring[j][e] = ring[j + 1][e];
+  }
+}
+
+// Closes a sublayer of a stream that the next sublayer reads through a convolution:
+//   xo = x + LN(y; w, b);   hc = xo + conv(xo)
+// One workgroup serves R consecutive tokens one after the other, eight channels a thread, the last K sums in registers; a
+// tile that starts inside a row forms the K sums ahead of it once more. x and xo are different buffers.
+template <typename T, int K, int MAXT>
+__global__ void __launch_bounds__(MAXT) norm_add_conv_kernel(
+    const float* __restrict__ x, const T* __restrict__ y, const T* __restrict__ w, const T* __restrict__ bias,
+    const T* __restrict__ cw_, float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ first_pos,
+    const int* __restrict__ state_slots, float* __restrict__ xo, T* __restrict__ hc, int B, int Tn, int W, int R,
+    float eps) {
+  __shared__ float red[2][16][2];
+  const int tid = threadIdx.x, wid = tid >> 6, nw = blockDim.x >> 6, c = 8 * tid;
+  const bool has = c < W;
+  int lo, hi, b;
+  conv_span(cu_q, B, Tn, blockIdx.x * R, R, K, lo, hi, b);
+  if (lo >= hi) return;
+  float lw[8], lb[8], cw[K + 1][8], ring[K + 1][8], cx[8], cy[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) lw[e] = lb[e] = cx[e] = cy[e] = 0.f;
+#pragma unroll
+  for (int j = 0; j <= K; ++j)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      cw[j][e] = has ? ldf<T>(cw_, (size_t)(c + e) * (K + 1) + j) : 0.f;
+      ring[j][e] = 0.f;
+    }
+  if (has) {
+    ld8f<T>(w + c, lw);
+    ld8f<T>(bias + c, lb);
+  }
+  // numbers in wave i of a row: 512 but for the last wave that has any
+  auto count = [&](int i) { return (float)max(0, min(512, W - 512 * i)); };
+  const float mine = count(wid);
+  auto fetch = [&](int t) {
+    if (has) {
+      ld8f<float>(x + (size_t)t * W + c, cx);
+      ld8f<T>(y + (size_t)t * W + c, cy);
+    }
+  };
+  int parity = 0;
+  // ring[K] <- the sum of the token last fetched; `next` (>= 0) is fetched meanwhile
+  auto close = [&](int next) {
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s += cy[e];
+    const float mw = mine > 0.f ? wave_sum(s) / mine : 0.f;
+    float m2 = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) m2 += has ? (cy[e] - mw) * (cy[e] - mw) : 0.f;
+    m2 = wave_sum(m2);
+    if ((tid & 63) == 0) {
+      red[parity][wid][0] = mw;
+      red[parity][wid][1] = m2;
+    }
+    float px[8], py[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      px[e] = cx[e];
+      py[e] = cy[e];
+    }
+    if (next >= 0) fetch(next);
+    __syncthreads();
+    float mean = 0.f, var = 0.f;
+    for (int i = 0; i < nw; ++i) mean += red[parity][i][0] * count(i);
+    mean /= (float)W;
+    for (int i = 0; i < nw; ++i) {
+      const float d = red[parity][i][0] - mean;
+      var += red[parity][i][1] + count(i) * d * d;
+    }
+    parity ^= 1;
+    const float rstd = 1.f / sqrtf(var / (float)W + eps);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ring[K][e] = px[e] + ((py[e] - mean) * rstd * lw[e] + lb[e]);
+  };
+  auto shift = [&]() {
+#pragma unroll
+    for (int j = 0; j < K; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ring[j][e] = ring[j + 1][e];
+  };
+  if (lo > cu_q[b] && lo < cu_q[b + 1]) {  // inside a row (at least K tokens): the sums ahead of the tile
+    if (K > 0) fetch(lo - K);
+    for (int k = 0; k < K; ++k) {
+      close(lo - K + k + 1);
+      shift();
+    }
+    if (K == 0) fetch(lo);
+  } else {
+    fetch(lo);
+  }
+  for (int t = lo; t < hi; ++t) {
+    while (t >= cu_q[b + 1]) ++b;
+    const int q0 = cu_q[b], q1 = cu_q[b + 1], slot = state_slots[b];
+    float* sl = state + (size_t)max(slot, 0) * K * W + c;
+    if (t == q0) {
+#pragma unroll
+      for (int j = 0; j < K; ++j) {
+        if (has && slot >= 0 && first_pos[b] + j - K >= 0) ld8f<float>(sl + (size_t)j * W, ring[j]);
+        else
+#pragma unroll
+          for (int e = 0; e < 8; ++e) ring[j][e] = 0.f;
+      }
+    }
+    close(t + 1 < hi ? t + 1 : -1);
+    float o[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float a = 0.f;
+#pragma unroll
+      for (int j = 0; j <= K; ++j) a += cw[j][e] * ring[j][e];
+      o[e] = slot >= 0 ? ring[K][e] + a : ring[K][e];
+    }
+    if (has) {
+      st8f<float>(xo + (size_t)t * W + c, ring[K]);
+      st8f<T>(hc + (size_t)t * W + c, o);
+    }
+    shift();
+    if (K > 0 && q0 >= lo && slot >= 0) {  // this workgroup served the row's first token: it leaves the row's last K sums
+      if (t == hi - 1 && q1 > hi) {
+        for (int u = max(hi, q1 - K); u < q1; ++u) {
+          fetch(u);
+          close(-1);
+          shift();
+        }
+      }
+      if ((t == q1 - 1 || t == hi - 1) && has) {
+#pragma unroll
+        for (int j = 0; j < K; ++j) st8f<float>(sl + (size_t)j * W, ring[j]);
+      }
+    }
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(1024) embed_bigram_norm_kernel(
     const int64_t* __restrict__ tokens, const T* __restrict__ embed, const T* __restrict__ bigram, int buckets,
@@ -350,6 +603,25 @@ extern "C" int areal_conv_silu(const void* h, int64_t h_stride, const void* w, c
                                int W, int taps, int dt, hipStream_t st) {
   if (T == 0 || B == 0) return 0;
   if (taps < 1 || (taps > 1 && !state) || (W + 255) / 256 > 65535) return -1;
+  const int R = T <= 512 ? 1 : 16;
+  if (taps <= 4 && W % 8 == 0 && h_stride % 8 == 0 && aligned16(h) && aligned16(out) && aligned16(state)) {
+    const dim3 vgrid((T + R - 1) / R, (W / 8 + 255) / 256);
+#define CONV(TT, KV)                                                                                                \
+  hipLaunchKernelGGL((conv_silu_vec_kernel<TT, KV>), vgrid, dim3(256), 0, st, (const TT*)h, h_stride, (const TT*)w, \
+                     (const TT*)bias, state, cu_q, first_pos, state_slots, (TT*)out, B, T, W, R)
+#define CONV_K(TT)                  \
+  do {                              \
+    if (taps == 1) CONV(TT, 0);     \
+    else if (taps == 2) CONV(TT, 1); \
+    else if (taps == 3) CONV(TT, 2); \
+    else CONV(TT, 3);               \
+  } while (0)
+    if (dt == 0) CONV_K(bf16_t);
+    else CONV_K(float);
+#undef CONV_K
+#undef CONV
+    return (int)hipGetLastError();
+  }
   const dim3 grid(T, (W + 255) / 256);
   if (dt == 0)
     hipLaunchKernelGGL((causal_conv_kernel<bf16_t, bf16_t, true>), grid, dim3(256), 0, st, (const bf16_t*)h, h_stride,
@@ -357,6 +629,44 @@ extern "C" int areal_conv_silu(const void* h, int64_t h_stride, const void* w, c
   else
     hipLaunchKernelGGL((causal_conv_kernel<float, float, true>), grid, dim3(256), 0, st, (const float*)h, h_stride,
                        (const float*)w, (const float*)bias, state, cu_q, first_pos, state_slots, (float*)out, B, W, taps);
+  return (int)hipGetLastError();
+}
+
+// Whether areal_norm_add_conv serves rows of W channels and this many taps.
+extern "C" int areal_norm_add_conv_serves(int W, int taps) { return taps >= 1 && taps <= 4 && W > 0 && W % 8 == 0 && W <= 8192; }
+
+// xo = x + LN(y; w, b) and hc = xo + conv(xo) (conv weights cw [W, taps], state as in areal_canon_conv); x, xo fp32 in
+// different buffers; every pointer 16-byte aligned.
+extern "C" int areal_norm_add_conv(const float* x, const void* y, const void* w, const void* b, const void* cw,
+                                   float* state, const int* cu_q, const int* first_pos, const int* state_slots, float* xo,
+                                   void* hc, int B, int T, int W, int taps, float eps, int dt, hipStream_t st) {
+  if (T == 0 || B == 0) return 0;
+  if (!areal_norm_add_conv_serves(W, taps) || (taps > 1 && !state) || x == xo) return -1;
+  if (!aligned16(x) || !aligned16(y) || !aligned16(w) || !aligned16(b) || !aligned16(state) || !aligned16(xo) ||
+      !aligned16(hc))
+    return -2;
+  const int R = T <= 512 ? 1 : 16, nthr = ((W / 8 + 63) / 64) * 64;
+#define CLOSE_T(TT, KV, MT)                                                                                           \
+  hipLaunchKernelGGL((norm_add_conv_kernel<TT, KV, MT>), dim3((T + R - 1) / R), dim3(nthr), 0, st, x, (const TT*)y,    \
+                     (const TT*)w, (const TT*)b, (const TT*)cw, state, cu_q, first_pos, state_slots, xo, (TT*)hc, B, T, \
+                     W, R, eps)
+#define CLOSE(TT, KV)                        \
+  do {                                       \
+    if (nthr <= 512) CLOSE_T(TT, KV, 512);   \
+    else CLOSE_T(TT, KV, 1024);              \
+  } while (0)
+#define CLOSE_K(TT)                   \
+  do {                                \
+    if (taps == 1) CLOSE(TT, 0);      \
+    else if (taps == 2) CLOSE(TT, 1); \
+    else if (taps == 3) CLOSE(TT, 2); \
+    else CLOSE(TT, 3);                \
+  } while (0)
+  if (dt == 0) CLOSE_K(bf16_t);
+  else CLOSE_K(float);
+#undef CLOSE_K
+#undef CLOSE
+#undef CLOSE_T
   return (int)hipGetLastError();
 }
 
