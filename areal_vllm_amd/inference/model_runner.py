@@ -489,13 +489,18 @@ class ModelRunner:
                                                 layers[i % len(layers)].mlp.act)}
         if has_plan:
             arms["balanced"] = lambda i: dg.dgemm_swiglu_balanced(x, layers[i % len(layers)].mlp.gate_up, act=act)
+        mode = self._fastest(arms, max(8, len(layers)), f"decode batch bucket {Bp}: gate|up GEMM ")
+        self._gate_up_choice[Bp] = mode
+        return mode
+
+    def _fastest(self, arms: Dict[str, Any], n: int, what: str) -> str:
+        """Name of the arm (name -> function of the repetition's index) with the shortest time over n repetitions."""
         times = {}
         for name, fn in arms.items():
             for i in range(2):
                 fn(i)
             torch.cuda.current_stream().synchronize()
             best = float("inf")
-            n = max(8, len(layers))
             for _ in range(3):  # the smallest of three: other work on the device (a colocated trainer) only adds time
                 e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
                 e0.record()
@@ -506,9 +511,7 @@ class ModelRunner:
                 best = min(best, e0.elapsed_time(e1) / n)
             times[name] = best
         mode = min(times, key=times.get)
-        self._gate_up_choice[Bp] = mode
-        logger.info(f"decode batch bucket {Bp}: gate|up GEMM " + ", ".join(f"{k} {v * 1e3:.1f} us" for k, v in times.items())
-                    + f" -> {mode}")
+        logger.info(what + ", ".join(f"{k} {v * 1e3:.1f} us" for k, v in times.items()) + f" -> {mode}")
         return mode
 
     def _decode_layers_fused(self, st: Dict[str, torch.Tensor], h: torch.Tensor, rope_pos: torch.Tensor):
@@ -1056,7 +1059,7 @@ class HybridModelRunner(ModelRunner):
         model, eps = self.model, float(self.cfg.rms_norm_eps)
         blocks = [model.layers[li] for li in self.layer_runs]
         trace = getattr(self, "layer_trace", None)
-        rows = (st.cu_q, st.first_pos, st.state_slots)
+        rows, mq = (st.cu_q, st.first_pos, st.state_slots), st.max_q
         x = pb.embed_scaled(ids, model.embed, float(self.cfg.embed_scale))
         hc = sw.stream_conv(x, blocks[0].canon1, self.state[0]["canon1"], *rows, self.dtype)
         for ri, blk in enumerate(blocks):
@@ -1064,11 +1067,11 @@ class HybridModelRunner(ModelRunner):
             nxt = (blocks[ri + 1].canon1, self.state[ri + 1]["canon1"]) if ri + 1 < len(blocks) else None
             if blk.mlp is not None:
                 x, hc = sw.norm_add_conv(x, y, blk.norm1, blk.norm1_bias, eps, (blk.canon2, self.state[ri]["canon2"]),
-                                         *rows)
-                y = blk.mlp(None, hc, None)
-                x, hc = sw.norm_add_conv(x, y, blk.norm2, blk.norm2_bias, eps, nxt, *rows)
+                                         *rows, mq)
+                y = blk.mlp.step(hc, st)
+                x, hc = sw.norm_add_conv(x, y, blk.norm2, blk.norm2_bias, eps, nxt, *rows, mq)
             else:
-                x, hc = sw.norm_add_conv(x, y, blk.norm1, blk.norm1_bias, eps, nxt, *rows)
+                x, hc = sw.norm_add_conv(x, y, blk.norm1, blk.norm1_bias, eps, nxt, *rows, mq)
             if trace is not None:
                 trace.append(x.clone())
         return x
@@ -1124,6 +1127,39 @@ class HybridModelRunner(ModelRunner):
         return self._run_layers(h, st), None
 
     # ------------------------------------------------------------------------------ decode
+    def tune_decode_paths(self):
+        if self.post_add and self.device.type == "cuda":
+            for b in self.buckets:
+                self._decode_gemms(b)
+
+    def _decode_gemms(self, Bp: int):
+        """Decode GEMMs of models whose closing kernel takes a split GEMM's slabs: {shape of a gate | up weight: kernel}, the
+        kernels timed once per batch bucket on the model's own weights. None: library products (other dtypes, large
+        batches, CPU)."""
+        from ..ops import decode_gemm as dg
+
+        if self.dtype != torch.bfloat16 or self.device.type != "cuda" or Bp > dg.MAX_ROWS:
+            return None
+        if Bp not in self._gate_up_choice:
+            by_shape: Dict[Any, List[Any]] = {}
+            for blk in self.model.layers:
+                if blk.mlp is not None:
+                    by_shape.setdefault(tuple(blk.mlp.gate_up.shape), []).append(blk.mlp)
+            choice = {}
+            for shape, mlps in by_shape.items():
+                x = torch.randn(Bp, shape[1], device=self.device, dtype=self.dtype)
+                names = ["library"]
+                if shape[1] % 64 == 0:
+                    names += ["balanced"] * (dg.swiglu_plan(Bp, shape[0] // 2) is not None)
+                    names += ["tiled"] * (shape[0] % 64 == 0)
+                if len(names) == 1 or torch.cuda.is_current_stream_capturing():
+                    choice[shape] = names[0]
+                    continue
+                arms = {k: (lambda i, k=k: mlps[i % len(mlps)].gated(x, k)) for k in names}
+                choice[shape] = self._fastest(arms, max(8, len(mlps)), f"decode batch bucket {Bp}: gate|up {shape} ")
+            self._gate_up_choice[Bp] = choice
+        return self._gate_up_choice[Bp]
+
     def _decode_workspace(self, Bp: int):
         from ..ops import window_attention as wattn
 
@@ -1173,4 +1209,6 @@ class HybridModelRunner(ModelRunner):
         eff = torch.where(st["slots"] < 0, self._neg1, st["state_slots"])
         step = StepTensors(st["cu_rows"], st["context_lens"], 1, st["slots"], st["block_tables"], st["positions"], eff,
                            nsplit=st["nsplit"], workspace=st["ws"], positions=st["positions"])
+        if self.post_add:
+            step.decode_gemms = self._decode_gemms(Bp)
         return self._final_logits(self._run_layers(h, step), None)

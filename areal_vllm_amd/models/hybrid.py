@@ -67,6 +67,7 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from .. import ops
+from ..ops import decode_gemm
 from ..ops import depth_avg as davg
 from ..ops import gla as gla_ops
 from ..ops import lightning as lightning_ops
@@ -497,6 +498,9 @@ class StepTensors:
         self.block_tables, self.first_pos, self.state_slots = block_tables, first_pos, state_slots
         self.nsplit, self.workspace = int(nsplit), workspace
         self.positions = positions  # position of every token (int32), for mixers that rotate by position
+        # decode steps whose closing kernel sums the partial products of a split GEMM: {(rows, inputs) of a gate | up weight:
+        # kernel for it}; None: library products
+        self.decode_gemms = None
         self._cu_k = None
         self.v_first = None  # this step's values of the first value-sharing attention layer [T, G Dv] (set by it)
 
@@ -930,6 +934,14 @@ def linear32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
     return F.linear(x.float(), weight.float())
 
 
+def closing_linear(x: torch.Tensor, weight: torch.Tensor, st: StepTensors) -> torch.Tensor:
+    """x W^T for a kernel that adds up what it reads: in decode steps fp32 slabs [S, T, N] of the split decode GEMM where it
+    serves the shape, else [T, N] in the compute dtype."""
+    if st.decode_gemms is not None and decode_gemm.serves(x, weight):
+        return decode_gemm.dgemm(x, weight, epilogue=decode_gemm.EPI_SLAB)
+    return F.linear(x, weight)
+
+
 class GLAMixer(nn.Module):
     """Gated linear attention (``ops/gla.py``): q | k | v | output gate | the low-rank input of the decay logits come
     out of ONE projection; the decay logits are the low-rank product plus a bias, formed in fp32; per key channel the
@@ -1035,7 +1047,7 @@ class RowNormAttentionMixer(nn.Module):
         else:
             o = wattn.window_attention(q, kc, vc, st.block_tables, st.cu_q, st.ctx_len, st.max_q, self.shape, None,
                                        nsplit=nsplit, workspace=st.workspace)
-        return F.linear(o.view(T, self.H * self.V), self.o)
+        return closing_linear(o.view(T, self.H * self.V), self.o, st)
 
 
 class MixedAttentionMixer(nn.Module):
@@ -1105,7 +1117,7 @@ class SideBySideMixer(nn.Module):
         both = torch.empty(hc.shape[0], self.o.shape[1], dtype=hc.dtype, device=hc.device)
         self.left.run(proj, st, cache, both[:, :self.c_left], self.left_scale)
         self.right.run(proj[:, self.n_left:], st, state, both[:, self.c_left:], self.right_scale)
-        return F.linear(both, self.o)
+        return closing_linear(both, self.o, st)
 
 
 class MambaMixer(nn.Module):
@@ -1135,12 +1147,13 @@ class MambaMixer(nn.Module):
     def step(self, hc: torch.Tensor, st: StepTensors, state) -> torch.Tensor:
         S, hist = state
         xz = F.linear(hc, self.proj)
-        x = sandwich.conv_silu(xz[:, :self.I], self.conv, self.conv_bias, hist, st.cu_q, st.first_pos, st.state_slots)
+        x = sandwich.conv_silu(xz[:, :self.I], self.conv, self.conv_bias, hist, st.cu_q, st.first_pos, st.state_slots,
+                               st.max_q)
         low = F.linear(x, self.x_proj)
         r = linear32(low[:, :self.rank], self.dt)
         y = mamba_ops.selective_scan(x, r, self.dt_bias, self.a_log, low[:, self.rank:], self.d_skip, xz[:, self.I:],
                                      st.cu_q, st.first_pos, st.state_slots, S, max_q=st.max_q)
-        return F.linear(y, self.o)
+        return closing_linear(y, self.o, st)
 
 
 class GatedMLP(nn.Module):
@@ -1154,6 +1167,19 @@ class GatedMLP(nn.Module):
 
     def forward(self, cols, hc: torch.Tensor, h32: Optional[torch.Tensor]) -> torch.Tensor:
         return F.linear(pblock.glu_rows(F.linear(hc, self.gate_up), self.act), self.down)
+
+    def step(self, hc: torch.Tensor, st: StepTensors) -> torch.Tensor:
+        """As `forward`, for a closing kernel that takes slabs (`closing_linear`)."""
+        mode = st.decode_gemms.get(tuple(self.gate_up.shape)) if st.decode_gemms is not None else None
+        return closing_linear(self.gated(hc, mode), self.down, st)
+
+    def gated(self, hc: torch.Tensor, mode: Optional[str]) -> torch.Tensor:
+        """act(gate h) * (up h) by the kernel `mode` names (None: library product, then the activation)."""
+        if mode == "balanced":
+            return decode_gemm.dgemm_swiglu_balanced(hc, self.gate_up, act=self.act)
+        if mode == "tiled":
+            return decode_gemm.dgemm(hc, self.gate_up, epilogue=decode_gemm.gated_epilogue(self.act))
+        return pblock.glu_rows(F.linear(hc, self.gate_up), self.act)
 
 
 class PrePostBlock(nn.Module):

@@ -101,6 +101,16 @@ def pick_config(M: int, N: int, K: int, epilogue: int) -> Tuple[int, int, int, i
 _OVERRIDES = {}
 
 
+MAX_ROWS = 512  # rows of a decode batch the kernels are laid out for
+
+
+def serves(x: torch.Tensor, w: torch.Tensor) -> bool:
+    """Whether `dgemm` takes these operands (bf16 on the GPU, K a multiple of 64, N of 32, aligned rows)."""
+    return (x.is_cuda and x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and x.shape[0] <= MAX_ROWS
+            and w.shape[1] % 64 == 0 and w.shape[0] % 32 == 0 and x.stride(1) == 1 and x.stride(0) % 8 == 0
+            and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and w.is_contiguous())
+
+
 def dgemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None, *, epilogue: int = EPI_BF16,
           cfg: Optional[int] = None, stages: Optional[int] = None, ksplit: Optional[int] = None,
           out: Optional[torch.Tensor] = None, loader_waves: Optional[int] = None,

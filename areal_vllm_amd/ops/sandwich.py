@@ -116,33 +116,43 @@ def stream_conv(x: torch.Tensor, weight: Optional[torch.Tensor], state: Optional
 
 def norm_add_conv(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, eps: float,
                   conv: Optional[Tuple[Optional[torch.Tensor], Optional[torch.Tensor]]], cu_q: torch.Tensor,
-                  first_pos: torch.Tensor, state_slots: torch.Tensor) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
-    """x + LN(y; weight, bias) on the fp32 stream x [T, W] (y [T, W] in the compute dtype; x itself may be overwritten) and,
-    with `conv` = (weight, state), `stream_conv` of the sum in y's dtype: one launch for up to four taps and 8192 channels.
+                  first_pos: torch.Tensor, state_slots: torch.Tensor, max_q: int = 0
+                  ) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """x + LN(y; weight, bias) on the fp32 stream x [T, W] (x itself may be overwritten) and, with `conv` = (weight, state),
+    `stream_conv` of the sum in the weights' dtype: one launch for up to four taps and 8192 channels. y [T, W] in the compute
+    dtype, or fp32 [S, T, W]: the sum of S slabs (a split GEMM's partial products). `max_q`: longest row when it is known.
     Returns (new stream, convolved stream or None)."""
-    if (conv is not None and conv[0] is not None and L.use_hip(x)
-            and L.lib().areal_norm_add_conv_serves(L.c_int(x.shape[1]), L.c_int(conv[0].shape[1]))):
-        T, W = x.shape
-        cw, state = conv
-        taps = cw.shape[1]
-        assert x.is_contiguous() and y.is_contiguous() and y.shape == x.shape and cw.is_contiguous() and cw.shape[0] == W
-        assert weight.dtype == y.dtype and bias.dtype == y.dtype and cw.dtype == y.dtype
+    T, W = x.shape
+    dtype = weight.dtype
+    slabs = y.shape[0] if y.dim() == 3 else 0
+    assert y.shape[-2:] == x.shape and y.dtype == (torch.float32 if slabs else dtype)
+    cw, state = conv if conv is not None else (None, None)
+    taps = cw.shape[1] if cw is not None else 0
+    if L.use_hip(x) and L.lib().areal_norm_add_conv_serves(L.c_int(W), L.c_int(taps)):
+        assert x.is_contiguous() and y.is_contiguous() and bias.dtype == dtype
         assert weight.numel() == W and bias.numel() == W
-        assert taps == 1 or (state.shape[1:] == (taps - 1, W) and state.dtype == torch.float32 and state.is_contiguous())
+        assert taps == 0 or (cw.is_contiguous() and cw.shape[0] == W and cw.dtype == dtype)
+        assert taps <= 1 or (state.shape[1:] == (taps - 1, W) and state.dtype == torch.float32 and state.is_contiguous())
         assert cu_q.dtype == torch.int32 and first_pos.dtype == torch.int32 and state_slots.dtype == torch.int32
-        if all(t.data_ptr() % 16 == 0 for t in (x, y, weight, bias)):
-            xo, hc = torch.empty_like(x), torch.empty_like(y)
+        if all(t.data_ptr() % 16 == 0 for t in (x, y, weight, bias, *([cw] if taps else []))):
+            xo = torch.empty_like(x)
+            hc = torch.empty(T, W, dtype=dtype, device=x.device) if taps else None
             L.check(L.lib().areal_norm_add_conv(
-                L.ptr(x), L.ptr(y), L.ptr(weight), L.ptr(bias), L.ptr(cw), L.ptr(state), L.ptr(cu_q), L.ptr(first_pos),
-                L.ptr(state_slots), L.ptr(xo), L.ptr(hc), L.c_int(cu_q.numel() - 1), L.c_int(T), L.c_int(W), L.c_int(taps),
-                L.c_float(eps), L.c_int(L.dtype_flag(y)), L.stream_ptr()), "norm_add_conv")
+                L.ptr(x), L.ptr(y), L.c_int(slabs), L.ptr(weight), L.ptr(bias), L.ptr(cw), L.ptr(state), L.ptr(cu_q),
+                L.ptr(first_pos), L.ptr(state_slots), L.ptr(xo), L.ptr(hc), L.c_int(cu_q.numel() - 1), L.c_int(T),
+                L.c_int(W), L.c_int(taps), L.c_int(int(max_q)), L.c_float(eps), L.c_int(L.dtype_flag(weight)),
+                L.stream_ptr()), "norm_add_conv")
+            if conv is not None and cw is None:
+                hc = stream_conv(xo, None, None, cu_q, first_pos, state_slots, dtype)
             return xo, hc
+    if slabs:
+        y = y.sum(0).to(dtype)
     x, _, _ = gated_norm_add(x, y, None, weight, bias, None, eps)
-    return x, (None if conv is None else stream_conv(x, conv[0], conv[1], cu_q, first_pos, state_slots, y.dtype))
+    return x, (None if conv is None else stream_conv(x, cw, state, cu_q, first_pos, state_slots, dtype))
 
 
 def conv_silu(h: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
-              cu_q: torch.Tensor, first_pos: torch.Tensor, state_slots: torch.Tensor) -> torch.Tensor:
+              cu_q: torch.Tensor, first_pos: torch.Tensor, state_slots: torch.Tensor, max_q: int = 0) -> torch.Tensor:
     """silu(conv(h) + bias) of h [T, W] in the compute dtype (a view with unit column stride), contiguous; weight, state
     and history as in `canon_conv` (the state is fp32 and holds the inputs h exactly)."""
     T, W = h.shape
@@ -156,7 +166,7 @@ def conv_silu(h: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor
         L.check(L.lib().areal_conv_silu(L.ptr(h), L.c_int64(h.stride(0)), L.ptr(weight), L.ptr(bias), L.ptr(state),
                                         L.ptr(cu_q), L.ptr(first_pos), L.ptr(state_slots), L.ptr(out),
                                         L.c_int(cu_q.numel() - 1), L.c_int(T), L.c_int(W), L.c_int(taps),
-                                        L.c_int(L.dtype_flag(h)), L.stream_ptr()), "conv_silu")
+                                        L.c_int(int(max_q)), L.c_int(L.dtype_flag(h)), L.stream_ptr()), "conv_silu")
         return out
     a = _causal_conv_cpu(h.float(), weight, state, cu_q, first_pos, state_slots)
     if bias is not None:

@@ -254,7 +254,14 @@ template <> DEVINL void st8f<float>(float* p, const float (&v)[8]) {
 // The tokens [lo, hi) that the workgroup of tile [t0, t0 + R) of the packed batch serves when a convolution with K tokens of
 // history runs along the rows: those of the tile, but a row's first K tokens - whose history reaches into the row's state
 // slot - all belong to the tile of the row's first token, so that the slot has one reader. That workgroup rewrites the slot.
-DEVINL void conv_span(const int* __restrict__ cu_q, int B, int T, int t0, int R, int K, int& lo, int& hi, int& row) {
+// single: every row has exactly one token (nothing to search for).
+DEVINL void conv_span(const int* __restrict__ cu_q, int B, int T, int t0, int R, int K, bool single, int& lo, int& hi,
+                      int& row) {
+  if (single) {
+    row = lo = t0;
+    hi = min(t0 + R, T);
+    return;
+  }
   row = row_of(cu_q, B, t0);
   lo = t0;
   hi = min(t0 + R, min(T, cu_q[B]));
@@ -266,6 +273,18 @@ DEVINL void conv_span(const int* __restrict__ cu_q, int B, int T, int t0, int R,
   }
 }
 
+// w[c + e][j] of eight channels and all taps: 8 (K + 1) consecutive numbers, 16-byte aligned
+template <typename T, int K>
+DEVINL void load_taps(const T* w, int c, float (&cw)[K + 1][8]) {
+#pragma unroll
+  for (int i = 0; i <= K; ++i) {
+    float v[8];
+    ld8f<T>(w + (size_t)c * (K + 1) + 8 * i, v);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) cw[(8 * i + e) % (K + 1)][(8 * i + e) / (K + 1)] = v[e];
+  }
+}
+
 // silu(conv(h) + bias) of rows in the storage type: eight channels a thread, R tokens a workgroup, the history in registers.
 // (Rows of a multiple of 8 channels, 16-byte aligned; the fallback is causal_conv_kernel.)
 template <typename T, int K>
@@ -274,16 +293,13 @@ __global__ void __launch_bounds__(256) conv_silu_vec_kernel(const T* __restrict_
                                                             float* __restrict__ state, const int* __restrict__ cu_q,
                                                             const int* __restrict__ first_pos,
                                                             const int* __restrict__ state_slots, T* __restrict__ out,
-                                                            int B, int Tn, int W, int R) {
+                                                            int B, int Tn, int W, int R, int single) {
   const int c = 8 * (blockIdx.y * 256 + threadIdx.x);
   int lo, hi, b;
-  conv_span(cu_q, B, Tn, blockIdx.x * R, R, K, lo, hi, b);
+  conv_span(cu_q, B, Tn, blockIdx.x * R, R, K, single, lo, hi, b);
   if (lo >= hi || c >= W) return;
   float cw[K + 1][8], bb[8], ring[K + 1][8];
-#pragma unroll
-  for (int j = 0; j <= K; ++j)
-#pragma unroll
-    for (int e = 0; e < 8; ++e) cw[j][e] = ldf<T>(w, (size_t)(c + e) * (K + 1) + j);
+  load_taps<T, K>(w, c, cw);
 #pragma unroll
   for (int e = 0; e < 8; ++e) bb[e] = bias ? ldf<T>(bias, c + e) : 0.f;
   bool fresh_row = true;  // the ring has to be filled for the token at hand
@@ -346,18 +362,19 @@ __global__ void __launch_bounds__(256) conv_silu_vec_kernel(const T* __restrict_
 // Closes a sublayer of a stream that the next sublayer reads through a convolution:
 //   xo = x + LN(y; w, b);   hc = xo + conv(xo)
 // One workgroup serves R consecutive tokens one after the other, eight channels a thread, the last K sums in registers; a
-// tile that starts inside a row forms the K sums ahead of it once more. x and xo are different buffers.
-template <typename T, int K, int MAXT>
+// tile that starts inside a row forms the K sums ahead of it once more. x and xo are different buffers. SLAB: y is the sum of
+// n_slab fp32 slabs [Tn, W] (partial products of a split GEMM). hc null: only xo (K = 0, cw null).
+template <typename T, int K, int MAXT, bool SLAB>
 __global__ void __launch_bounds__(MAXT) norm_add_conv_kernel(
-    const float* __restrict__ x, const T* __restrict__ y, const T* __restrict__ w, const T* __restrict__ bias,
+    const float* __restrict__ x, const void* __restrict__ y_, int n_slab, const T* __restrict__ w, const T* __restrict__ bias,
     const T* __restrict__ cw_, float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ first_pos,
     const int* __restrict__ state_slots, float* __restrict__ xo, T* __restrict__ hc, int B, int Tn, int W, int R,
-    float eps) {
+    int single, float eps) {
   __shared__ float red[2][16][2];
   const int tid = threadIdx.x, wid = tid >> 6, nw = blockDim.x >> 6, c = 8 * tid;
   const bool has = c < W;
   int lo, hi, b;
-  conv_span(cu_q, B, Tn, blockIdx.x * R, R, K, lo, hi, b);
+  conv_span(cu_q, B, Tn, blockIdx.x * R, R, K, single, lo, hi, b);
   if (lo >= hi) return;
   float lw[8], lb[8], cw[K + 1][8], ring[K + 1][8], cx[8], cy[8];
 #pragma unroll
@@ -365,11 +382,9 @@ __global__ void __launch_bounds__(MAXT) norm_add_conv_kernel(
 #pragma unroll
   for (int j = 0; j <= K; ++j)
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      cw[j][e] = has ? ldf<T>(cw_, (size_t)(c + e) * (K + 1) + j) : 0.f;
-      ring[j][e] = 0.f;
-    }
+    for (int e = 0; e < 8; ++e) cw[j][e] = ring[j][e] = 0.f;
   if (has) {
+    if (cw_) load_taps<T, K>(cw_, c, cw);
     ld8f<T>(w + c, lw);
     ld8f<T>(bias + c, lb);
   }
@@ -379,7 +394,19 @@ __global__ void __launch_bounds__(MAXT) norm_add_conv_kernel(
   auto fetch = [&](int t) {
     if (has) {
       ld8f<float>(x + (size_t)t * W + c, cx);
-      ld8f<T>(y + (size_t)t * W + c, cy);
+      if (SLAB) {
+        const float* y = reinterpret_cast<const float*>(y_) + (size_t)t * W + c;
+        ld8f<float>(y, cy);
+#pragma unroll 4
+        for (int s = 1; s < n_slab; ++s) {
+          float v[8];
+          ld8f<float>(y + (size_t)s * Tn * W, v);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) cy[e] += v[e];
+        }
+      } else {
+        ld8f<T>(reinterpret_cast<const T*>(y_) + (size_t)t * W + c, cy);
+      }
     }
   };
   int parity = 0;
@@ -457,7 +484,7 @@ __global__ void __launch_bounds__(MAXT) norm_add_conv_kernel(
     }
     if (has) {
       st8f<float>(xo + (size_t)t * W + c, ring[K]);
-      st8f<T>(hc + (size_t)t * W + c, o);
+      if (hc) st8f<T>(hc + (size_t)t * W + c, o);
     }
     shift();
     if (K > 0 && q0 >= lo && slot >= 0) {  // this workgroup served the row's first token: it leaves the row's last K sums
@@ -600,15 +627,17 @@ extern "C" int areal_canon_conv(const float* h, const void* w, float* state, con
 // out [T, W] = silu(conv(h) + bias), h rows in the storage type, h_stride apart; bias [W] or null
 extern "C" int areal_conv_silu(const void* h, int64_t h_stride, const void* w, const void* bias, float* state,
                                const int* cu_q, const int* first_pos, const int* state_slots, void* out, int B, int T,
-                               int W, int taps, int dt, hipStream_t st) {
+                               int W, int taps, int max_q, int dt, hipStream_t st) {
   if (T == 0 || B == 0) return 0;
   if (taps < 1 || (taps > 1 && !state) || (W + 255) / 256 > 65535) return -1;
+  const int single = max_q == 1 && T == B;
   const int R = T <= 512 ? 1 : 16;
-  if (taps <= 4 && W % 8 == 0 && h_stride % 8 == 0 && aligned16(h) && aligned16(out) && aligned16(state)) {
+  if (taps <= 4 && W % 8 == 0 && h_stride % 8 == 0 && aligned16(h) && aligned16(w) && aligned16(out) &&
+      aligned16(state)) {
     const dim3 vgrid((T + R - 1) / R, (W / 8 + 255) / 256);
 #define CONV(TT, KV)                                                                                                \
   hipLaunchKernelGGL((conv_silu_vec_kernel<TT, KV>), vgrid, dim3(256), 0, st, (const TT*)h, h_stride, (const TT*)w, \
-                     (const TT*)bias, state, cu_q, first_pos, state_slots, (TT*)out, B, T, W, R)
+                     (const TT*)bias, state, cu_q, first_pos, state_slots, (TT*)out, B, T, W, R, single)
 #define CONV_K(TT)                  \
   do {                              \
     if (taps == 1) CONV(TT, 0);     \
@@ -632,32 +661,38 @@ extern "C" int areal_conv_silu(const void* h, int64_t h_stride, const void* w, c
   return (int)hipGetLastError();
 }
 
-// Whether areal_norm_add_conv serves rows of W channels and this many taps.
-extern "C" int areal_norm_add_conv_serves(int W, int taps) { return taps >= 1 && taps <= 4 && W > 0 && W % 8 == 0 && W <= 8192; }
+// Whether areal_norm_add_conv serves rows of W channels and this many taps (0: no convolution).
+extern "C" int areal_norm_add_conv_serves(int W, int taps) { return taps >= 0 && taps <= 4 && W > 0 && W % 8 == 0 && W <= 8192; }
 
-// xo = x + LN(y; w, b) and hc = xo + conv(xo) (conv weights cw [W, taps], state as in areal_canon_conv); x, xo fp32 in
-// different buffers; every pointer 16-byte aligned.
-extern "C" int areal_norm_add_conv(const float* x, const void* y, const void* w, const void* b, const void* cw,
+// xo = x + LN(y; w, b) and, with taps > 0, hc = xo + conv(xo) (conv weights cw [W, taps], state as in areal_canon_conv); x, xo
+// fp32 in different buffers; every pointer 16-byte aligned. n_slab > 0: y is the sum of n_slab fp32 slabs [T, W] that follow
+// each other; 0: one row per token in the storage type. max_q: longest row.
+extern "C" int areal_norm_add_conv(const float* x, const void* y, int n_slab, const void* w, const void* b, const void* cw,
                                    float* state, const int* cu_q, const int* first_pos, const int* state_slots, float* xo,
-                                   void* hc, int B, int T, int W, int taps, float eps, int dt, hipStream_t st) {
+                                   void* hc, int B, int T, int W, int taps, int max_q, float eps, int dt, hipStream_t st) {
   if (T == 0 || B == 0) return 0;
-  if (!areal_norm_add_conv_serves(W, taps) || (taps > 1 && !state) || x == xo) return -1;
-  if (!aligned16(x) || !aligned16(y) || !aligned16(w) || !aligned16(b) || !aligned16(state) || !aligned16(xo) ||
-      !aligned16(hc))
+  if (!areal_norm_add_conv_serves(W, taps) || (taps > 1 && !state) || x == xo || (taps > 0) != (hc != nullptr)) return -1;
+  if (!aligned16(x) || !aligned16(y) || !aligned16(w) || !aligned16(b) || !aligned16(cw) || !aligned16(state) ||
+      !aligned16(xo) || !aligned16(hc))
     return -2;
-  const int R = T <= 512 ? 1 : 16, nthr = ((W / 8 + 63) / 64) * 64;
-#define CLOSE_T(TT, KV, MT)                                                                                           \
-  hipLaunchKernelGGL((norm_add_conv_kernel<TT, KV, MT>), dim3((T + R - 1) / R), dim3(nthr), 0, st, x, (const TT*)y,    \
-                     (const TT*)w, (const TT*)b, (const TT*)cw, state, cu_q, first_pos, state_slots, xo, (TT*)hc, B, T, \
-                     W, R, eps)
-#define CLOSE(TT, KV)                        \
-  do {                                       \
-    if (nthr <= 512) CLOSE_T(TT, KV, 512);   \
-    else CLOSE_T(TT, KV, 1024);              \
+  const int R = T <= 512 ? 1 : 16, nthr = ((W / 8 + 63) / 64) * 64, single = max_q == 1 && T == B;
+#define CLOSE_S(TT, KV, MT, SL)                                                                                     \
+  hipLaunchKernelGGL((norm_add_conv_kernel<TT, KV, MT, SL>), dim3((T + R - 1) / R), dim3(nthr), 0, st, x, y, n_slab,  \
+                     (const TT*)w, (const TT*)b, (const TT*)cw, state, cu_q, first_pos, state_slots, xo, (TT*)hc, B,  \
+                     T, W, R, single, eps)
+#define CLOSE(TT, KV)                                      \
+  do {                                                     \
+    if (nthr <= 512) {                                     \
+      if (n_slab > 0) CLOSE_S(TT, KV, 512, true);          \
+      else CLOSE_S(TT, KV, 512, false);                    \
+    } else {                                               \
+      if (n_slab > 0) CLOSE_S(TT, KV, 1024, true);         \
+      else CLOSE_S(TT, KV, 1024, false);                   \
+    }                                                      \
   } while (0)
 #define CLOSE_K(TT)                   \
   do {                                \
-    if (taps == 1) CLOSE(TT, 0);      \
+    if (taps <= 1) CLOSE(TT, 0);      \
     else if (taps == 2) CLOSE(TT, 1); \
     else if (taps == 3) CLOSE(TT, 2); \
     else CLOSE(TT, 3);                \
@@ -666,7 +701,7 @@ extern "C" int areal_norm_add_conv(const float* x, const void* y, const void* w,
   else CLOSE_K(float);
 #undef CLOSE_K
 #undef CLOSE
-#undef CLOSE_T
+#undef CLOSE_S
   return (int)hipGetLastError();
 }
 

@@ -87,12 +87,30 @@ def test_closing_norm_sum_and_convolved_stream_in_portions(device, dtype, W, tap
         for i in range(3):
             assert rel_err(torch.cat(got_x[i]), want_x[i]) < 2e-6
             assert rel_err(torch.cat(got_h[i]), want_h[i]) < (3e-6 if is32(dtype) else 1e-2)
+    # a decode step: one token a row, the sublayer's output as three fp32 slabs (partial products of a split GEMM)
+    if state is not None:
+        state[:3] = torch.randn(3, taps - 1, W, generator=g).to(device)
+    hist = state[:3].cpu().to(F64) if state is not None else torch.zeros(3, 0, W, dtype=F64)
+    x3, sl = torch.randn(3, W, generator=g), torch.randn(3, 3, W, generator=g)
+    want3 = x3.to(F64) + O.layer_norm(sl.to(F64).sum(0), w.to(F64), b.to(F64), eps)
+    nx, hc = sw.norm_add_conv(x3.clone().to(device), sl.to(device), w.to(device), b.to(device), eps, (cw.to(device) if taps else None, state),
+                              i32([0, 1, 2, 3], device), i32([9, 5, 20], device), i32([2, 0, 1], device), 1)
+    assert rel_err(nx.cpu(), want3) < (2e-6 if is32(dtype) else 1e-2)
+    for j, s in enumerate((2, 0, 1)):
+        seq = torch.cat([hist[s], want3[j:j + 1]])
+        want = O.with_history(seq, cw.to(F64))[-1:] if taps else want3[j:j + 1]
+        assert rel_err(hc[j:j + 1].float().cpu(), want) < (3e-6 if is32(dtype) else 2e-2)
+        if taps > 1:
+            assert rel_err(state[s].cpu(), seq[1:]) < (3e-6 if is32(dtype) else 2e-2)
+    nx, hc = sw.norm_add_conv(x3.clone().to(device), sl.to(device), w.to(device), b.to(device), eps, None, i32([0, 1, 2, 3], device),
+                              i32([9, 5, 20], device), i32([2, 0, 1], device), 1)
+    assert hc is None and rel_err(nx.cpu(), want3) < (2e-6 if is32(dtype) else 1e-2)
     # without a following sublayer only the sum is formed
     nx, hc = sw.norm_add_conv(xs[0].to(device), ys[0].to(device), w.to(device), b.to(device), eps, None,
                               i32([0, 41], device), i32([0], device), i32([1], device))
     assert hc is None and rel_err(nx.cpu(), want_x[0]) < 2e-6
     if taps > 1:
-        assert float(state[1].min()) == 37.0 and float(state[3].max()) == 37.0  # slots of nobody stay as they were
+        assert float(state[3].min()) == 37.0 and float(state[3].max()) == 37.0  # nobody's slot stays as it was
 
 
 ROTS = [None, {"base": 10000.0, "dims": 8}, {"base": 500.0, "dims": 16},
