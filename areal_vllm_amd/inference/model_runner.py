@@ -1104,7 +1104,7 @@ class HybridModelRunner(ModelRunner):
                                     float(self.cfg.rms_norm_eps), self.dtype)
             if fp32 or self.keep_logits:
                 return F.linear(x32, self.model.head_weight.float())
-            return F.linear(xc, self.model.head_weight)
+            return self._lm_head(xc)
         x32, xc = scaled_add_norm(h.contiguous(), None, self.model.norm, 1.0, float(self.cfg.rms_norm_eps),
                                   self.dtype, inplace=False)
         if fp32 or self.keep_logits:

@@ -67,7 +67,7 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from .. import ops
-from ..ops import decode_gemm
+from ..ops import decode_gemm, train_gemm
 from ..ops import depth_avg as davg
 from ..ops import gla as gla_ops
 from ..ops import lightning as lightning_ops
@@ -1166,7 +1166,7 @@ class GatedMLP(nn.Module):
         self.down = nn.Parameter(torch.empty(width, ff, dtype=dtype, device=device))
 
     def forward(self, cols, hc: torch.Tensor, h32: Optional[torch.Tensor]) -> torch.Tensor:
-        return F.linear(pblock.glu_rows(F.linear(hc, self.gate_up), self.act), self.down)
+        return F.linear(self.gated(hc, None), self.down)
 
     def step(self, hc: torch.Tensor, st: StepTensors) -> torch.Tensor:
         """As `forward`, for a closing kernel that takes slabs (`closing_linear`)."""
@@ -1179,7 +1179,8 @@ class GatedMLP(nn.Module):
             return decode_gemm.dgemm_swiglu_balanced(hc, self.gate_up, act=self.act)
         if mode == "tiled":
             return decode_gemm.dgemm(hc, self.gate_up, epilogue=decode_gemm.gated_epilogue(self.act))
-        return pblock.glu_rows(F.linear(hc, self.gate_up), self.act)
+        a = train_gemm.gate_up_act(hc, self.gate_up, self.act)  # prompt portions of many rows: one kernel
+        return a if a is not None else pblock.glu_rows(F.linear(hc, self.gate_up), self.act)
 
 
 class PrePostBlock(nn.Module):

@@ -47,7 +47,10 @@ def gla_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, z: torch.Te
         obuf = torch.empty(T, NH, V, dtype=torch.float32, device=proj.device)
         scratch = None
         if max_q >= CHUNK and D <= 128:  # the chunked form's state-independent operands
-            scratch = torch.empty(T * (3 * NH * D + CHUNK * NH), dtype=torch.float32, device=proj.device)
+            fn = L.lib().areal_gla_scratch
+            fn.restype = L.c_int64
+            scratch = torch.empty(int(fn(L.c_int(T), L.c_int(B), L.c_int(NH), L.c_int(D))), dtype=torch.float32,
+                                  device=proj.device)
         L.check(L.lib().areal_gla_scan(
             L.ptr(proj), L.c_int64(proj.stride(0)), L.c_int(q_off), L.c_int(k_off), L.c_int(v_off), L.ptr(z),
             L.c_int64(z.stride(0)), L.ptr(z_bias), L.c_float(tau), L.c_float(q_scale), L.ptr(cu_q), L.ptr(first_pos),

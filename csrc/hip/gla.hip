@@ -30,8 +30,15 @@ template <typename T> DEVINL void stf(T* p, size_t i, float v);
 template <> DEVINL void stf<bf16_t>(bf16_t* p, size_t i, float v) { p[i] = f2bf(v); }
 template <> DEVINL void stf<float>(float* p, size_t i, float v) { p[i] = v; }
 
-// ln sigmoid(z) / tau
-DEVINL float log_decay(float z, float inv_tau) { return -(fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z)))) * inv_tau; }
+// ln sigmoid(z) / tau; bf16 storage: hardware exponential and logarithm (a short series where 1 + e would lose e's digits)
+template <typename T> DEVINL float log_decay(float z, float inv_tau) {
+  if (sizeof(T) == 2) {
+    const float e = __expf(-fabsf(z));
+    const float l = e < 0.0156f ? e * (1.f - e * (0.5f - 0.33333333f * e)) : __logf(1.f + e);
+    return -(fmaxf(-z, 0.f) + l) * inv_tau;
+  }
+  return -(fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z)))) * inv_tau;
+}
 
 constexpr int TC = 8;  // tokens staged per step of the loop
 constexpr int RW = 4;  // waves of a workgroup
@@ -73,7 +80,7 @@ __global__ void __launch_bounds__(64 * RW) gla_scan_kernel(
       const T* row = proj + tok * row_stride;
       kqa[tt][0][d] = live ? ldf<T>(row, k_off + hd * D + d) : 0.f;
       kqa[tt][1][d] = live ? ldf<T>(row, q_off + hd * D + d) * q_scale : 0.f;
-      kqa[tt][2][d] = live ? expf(log_decay(z[tok * z_stride + hd * D + d] + (z_bias ? ldf<T>(z_bias, hd * D + d) : 0.f),
+      kqa[tt][2][d] = live ? expf(log_decay<T>(z[tok * z_stride + hd * D + d] + (z_bias ? ldf<T>(z_bias, hd * D + d) : 0.f),
                                             inv_tau))
                            : 1.f;
     }
@@ -115,12 +122,18 @@ __global__ void __launch_bounds__(64 * RW) gla_scan_kernel(
 // Prompt portions: chunks of CT tokens, in two launches. Whatever does not depend on the state is formed for all
 // chunks at once by `gla_prep_kernel` (one workgroup per (chunk, row, head), thousands of them): the per-channel log
 // decays summed along the chunk's tokens (b_t), q_t * exp(b_t), k_s * exp(b_L - b_s), exp(b_L), and the lower triangle
-// A[t, s] = sum_d q_t[d] k_s[d] exp(b_t[d] - b_s[d]), pair by pair so that every exponent is <= 0. `gla_chunk_kernel`
-// then walks a row's chunks in order with nothing but matrix products on the fp32 matrix cores (MFMA 16x16x4): the
-// read-out q~ S_prev + A V (wave w owns 16 of the workgroup's 64 value columns) and the state's move to the chunk's end
-// diag(exp(b_L)) S_prev + k~^T V (every fourth block of 16 state rows a wave). The next chunk's operands are fetched
-// into registers under the matrix work.
+// A[t, s] = sum_d q_t[d] k_s[d] exp(b_t[d] - b_s[d]), pair by pair so that every exponent is <= 0. It leaves them in the
+// order in which `gla_chunk_kernel` reads them as matrix-core operands, padded with zeros to CT tokens and DP channels:
+// per (chunk slot, head) q~ [CT][DP], k~^T [DP][CT], exp(b_L) [DP], A [CT][CT]. `gla_chunk_kernel` then walks a row's chunks
+// with nothing but products on the fp32 matrix cores (MFMA 16x16x4): a wave owns 16 value columns and keeps its slice of the
+// state in registers, which are at once the B operand of the read-out q~ S_prev + A V and the accumulator of the move to
+// the chunk's end diag(exp(b_L)) S_prev + k~^T V (lane: column, channels 16 i + 4 quad .. + 3). Waves share nothing: no LDS,
+// no barriers; the operands of the next two chunks are fetched under the matrix work.
 constexpr int CT = 16;
+
+// Slot of the chunk that starts at token tb of row b (first token t_lo) in the scratch buffers; T / CT + B + 1 slots.
+DEVINL size_t chunk_slot(int t_lo, int tb, int b) { return (size_t)(t_lo / CT + b + (tb - t_lo) / CT); }
+template <int DP> constexpr size_t chunk_floats() { return 2 * CT * DP + DP + CT * CT; }
 
 // bf16 storage: v_exp_f32 (relative error ~1e-6, far below the storage's); fp32 storage: the library's exp
 template <typename T> DEVINL float exp_le0(float x) { return sizeof(T) == 2 ? __expf(x) : expf(x); }
@@ -129,8 +142,7 @@ template <typename T, int DP>
 __global__ void __launch_bounds__(256) gla_prep_kernel(
     const T* __restrict__ proj, int64_t row_stride, int q_off, int k_off, const float* __restrict__ z, int64_t z_stride,
     const T* __restrict__ z_bias, float inv_tau, float q_scale, const int* __restrict__ cu_q,
-    const int* __restrict__ state_slots, float* __restrict__ qd, float* __restrict__ kd, float* __restrict__ el,
-    float* __restrict__ abuf, int NH, int D) {
+    const int* __restrict__ state_slots, float* __restrict__ scratch, int NH, int D) {
   constexpr int QS = DP + 1;  // odd stride: the pair loop's 16 key rows fall on different banks
   __shared__ float Qr[CT * QS], Kr[CT * QS], Bs[CT * QS];
   const int b = blockIdx.y, hd = blockIdx.z, tid = threadIdx.x;
@@ -146,7 +158,7 @@ __global__ void __launch_bounds__(256) gla_prep_kernel(
     Kr[tt * QS + d] = live ? ldf<T>(row, k_off + hd * D + dc) : 0.f;
     Qr[tt * QS + d] = live ? ldf<T>(row, q_off + hd * D + dc) * q_scale : 0.f;
     // rows past the chunk's end and padding channels do not decay
-    Bs[tt * QS + d] = live ? log_decay(z[tok * z_stride + hd * D + dc] + (z_bias ? ldf<T>(z_bias, hd * D + dc) : 0.f), inv_tau)
+    Bs[tt * QS + d] = live ? log_decay<T>(z[tok * z_stride + hd * D + dc] + (z_bias ? ldf<T>(z_bias, hd * D + dc) : 0.f), inv_tau)
                            : 0.f;
   }
   __syncthreads();
@@ -159,16 +171,15 @@ __global__ void __launch_bounds__(256) gla_prep_kernel(
     }
   }
   __syncthreads();
-  const size_t N = (size_t)NH * D;
+  float* qd = scratch + (chunk_slot(t_lo, tb, b) * NH + hd) * chunk_floats<DP>();
+  float *kd = qd + CT * DP, *el = kd + CT * DP, *abuf = el + DP;
   for (int i = tid; i < CT * DP; i += 256) {
     const int d = i % DP, tt = i / DP;
-    if (tt < nt && d < D) {
-      const float bt = Bs[tt * QS + d], bl = Bs[(nt - 1) * QS + d];
-      qd[(size_t)(tb + tt) * N + hd * D + d] = Qr[tt * QS + d] * exp_le0<T>(bt);
-      kd[(size_t)(tb + tt) * N + hd * D + d] = Kr[tt * QS + d] * exp_le0<T>(bl - bt);
-      if (tt == 0) el[(size_t)tb * N + hd * D + d] = exp_le0<T>(bl);
-    }
+    qd[i] = Qr[tt * QS + d] * exp_le0<T>(Bs[tt * QS + d]);
+    const int kt = i % CT, kc = i / CT;
+    kd[i] = Kr[kt * QS + kc] * exp_le0<T>(Bs[(CT - 1) * QS + kc] - Bs[kt * QS + kc]);
   }
+  for (int i = tid; i < DP; i += 256) el[i] = exp_le0<T>(Bs[(CT - 1) * QS + i]);
   {  // the chunk's own pairs: thread (t, s), s <= t
     const int t = tid / CT, sx = tid % CT;
     float a0 = 0.f, a1 = 0.f;
@@ -180,139 +191,105 @@ __global__ void __launch_bounds__(256) gla_prep_kernel(
         a1 += qt[d + 1] * ks[d + 1] * exp_le0<T>(bt[d + 1] - bs[d + 1]);
       }
     }
-    if (t < nt) abuf[((size_t)(tb + t) * NH + hd) * CT + sx] = a0 + a1;
+    abuf[tid] = a0 + a1;
   }
 }
 
-template <int DP>
+template <typename T, int DP>
 __global__ void __launch_bounds__(256) gla_chunk_kernel(
-    const float* __restrict__ qd, const float* __restrict__ kd, const float* __restrict__ el,
-    const float* __restrict__ abuf, const void* __restrict__ proj, int64_t row_stride, int v_off, int bf16_storage,
+    const float* __restrict__ scratch, const T* __restrict__ proj, int64_t row_stride, int v_off,
     const int* __restrict__ cu_q, const int* __restrict__ first_pos, const int* __restrict__ state_slots,
     float* __restrict__ S, float* __restrict__ obuf, int NH, int D, int V) {
-  constexpr int QS = DP + 4, CS = 64 + 4, AS = CT + 1;
-  constexpr int NE = CT * DP / 256, NV = CT * 64 / 256;  // elements per thread of q~ / k~, and of v
-  extern __shared__ float cl[];
-  float* Sst = cl;               // [DP][CS] state slice
-  float* Qd = Sst + DP * CS;     // [CT][QS] q * q_scale * exp(b_t)
-  float* Kd = Qd + CT * QS;      // [CT][QS] k * exp(b_L - b_t)
-  float* Vs = Kd + CT * QS;      // [CT][CS]
-  float* As = Vs + CT * CS;      // [CT][AS]
-  float* Es = As + CT * AS;      // [DP] exp(b_L)
-  const int b = blockIdx.x, hd = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
-  const int r16 = lane & 15, quad = lane >> 4, col0 = blockIdx.z * 64;
+  constexpr int NB = DP / 16;  // blocks of 16 state rows
+  const int b = blockIdx.x, hd = blockIdx.y, lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int r16 = lane & 15, quad = lane >> 4, c = blockIdx.z * 64 + 16 * w + r16;
+  const bool has = c < V;
   const int slot = state_slots[b];
   const int t_lo = cu_q[b], t_hi = cu_q[b + 1];
   if (slot < 0) {
-    for (int i = tid; i < (t_hi - t_lo) * 64; i += 256) {
-      const int t = t_lo + i / 64, c = col0 + i % 64;
-      if (c < V) obuf[((size_t)t * NH + hd) * V + c] = 0.f;
-    }
+    for (int t = t_lo + quad; t < t_hi; t += 4)
+      if (has) obuf[((size_t)t * NH + hd) * V + c] = 0.f;
     return;
   }
-  if (t_hi <= t_lo) return;
+  if (t_hi <= t_lo || blockIdx.z * 64 + 16 * w >= V) return;
   const bool fresh = first_pos[b] == 0;
-  const size_t sbase = ((size_t)slot * NH + hd) * D, N = (size_t)NH * D;
-  for (int i = tid; i < DP * 64; i += 256) {
-    const int d = i / 64, c = i % 64;
-    Sst[d * CS + c] = (!fresh && d < D && col0 + c < V) ? S[(sbase + d) * V + col0 + c] : 0.f;
-  }
-  float rq[NE], rk[NE], rv[NV], ra, re = 1.f;
-  auto fetch = [&](int tb) {
-    const int nt = min(CT, t_hi - tb);
+  float* Sp = S + ((size_t)slot * NH + hd) * D * V + min(c, V - 1);
+  f32x4 s[NB];
 #pragma unroll
-    for (int j = 0; j < NE; ++j) {
-      const int i = tid + 256 * j, d = i % DP, tt = i / DP;
-      const bool live = tt < nt && d < D;
-      const size_t at = (size_t)(tb + min(tt, nt - 1)) * N + hd * D + min(d, D - 1);
-      rq[j] = live ? qd[at] : 0.f;
-      rk[j] = live ? kd[at] : 0.f;
-    }
+  for (int rb = 0; rb < NB; ++rb)
 #pragma unroll
-    for (int j = 0; j < NV; ++j) {
-      const int i = tid + 256 * j, c = i % 64, tt = i / 64;
-      const size_t at = (size_t)(tb + min(tt, nt - 1)) * row_stride + v_off + hd * V + min(col0 + c, V - 1);
-      const float x = bf16_storage ? bf2f(reinterpret_cast<const bf16_t*>(proj)[at]) : reinterpret_cast<const float*>(proj)[at];
-      rv[j] = (tt < nt && col0 + c < V) ? x : 0.f;
+    for (int i = 0; i < 4; ++i) {
+      const int d = 16 * rb + 4 * quad + i;
+      s[rb][i] = (!fresh && has && d < D) ? Sp[(size_t)d * V] : 0.f;
     }
-    {
-      const int t = tid / CT, sx = tid % CT;
-      ra = (t < nt && sx <= t) ? abuf[((size_t)(tb + t) * NH + hd) * CT + sx] : 0.f;
-    }
-    if (tid < DP) re = tid < D ? el[(size_t)tb * N + hd * D + tid] : 1.f;
+  struct Operands {
+    f32x4 q[NB], k[NB], e[NB], a;
+    T v[4];  // as loaded: nothing waits for a load before its chunk's turn
   };
-  fetch(t_lo);
-  for (int tb = t_lo; tb < t_hi; tb += CT) {
-    const int nt = min(CT, t_hi - tb);
-    __syncthreads();  // the chunk before is done with the staged operands
+  const T* vp = proj + v_off + hd * V + min(c, V - 1);
+  auto fetch = [&](Operands& o, int tb) {
+    const float* base = scratch + (chunk_slot(t_lo, tb, b) * NH + hd) * chunk_floats<DP>();
 #pragma unroll
-    for (int j = 0; j < NE; ++j) {
-      const int i = tid + 256 * j, d = i % DP, tt = i / DP;
-      Qd[tt * QS + d] = rq[j];
-      Kd[tt * QS + d] = rk[j];
+    for (int i = 0; i < NB; ++i) {
+      o.q[i] = *reinterpret_cast<const f32x4*>(base + r16 * DP + 16 * i + 4 * quad);
+      o.k[i] = *reinterpret_cast<const f32x4*>(base + CT * DP + (16 * i + r16) * CT + 4 * quad);
+      o.e[i] = *reinterpret_cast<const f32x4*>(base + 2 * CT * DP + 16 * i + 4 * quad);
     }
+    o.a = *reinterpret_cast<const f32x4*>(base + 2 * CT * DP + DP + r16 * CT + 4 * quad);
 #pragma unroll
-    for (int j = 0; j < NV; ++j) {
-      const int i = tid + 256 * j;
-      Vs[(i / 64) * CS + i % 64] = rv[j];
+    for (int i = 0; i < 4; ++i)  // rows past the chunk's end meet zeros in A and k~: any finite value will do
+      o.v[i] = vp[(size_t)min(tb + 4 * quad + i, t_hi - 1) * row_stride];
+  };
+  auto chunk = [&](const Operands& o, int tb) {
+    f32x4 v;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = (float)o.v[i];
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i][0], s[i][0], acc, 0, 0, 0);
+      acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i][1], s[i][1], acc2, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i][2], s[i][2], acc, 0, 0, 0);
+      acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i][3], s[i][3], acc2, 0, 0, 0);
     }
-    As[(tid / CT) * AS + tid % CT] = ra;
-    if (tid < DP) Es[tid] = re;
-    if (tb + CT < t_hi) fetch(tb + CT);
-    __syncthreads();
-    {  // read-out: rows = the chunk's tokens, columns 16 w .. 16 w + 15 of the slice; two accumulation chains
-      f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
-      for (int kk = 0; kk < DP / 4; kk += 2) {
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(Qd[r16 * QS + 4 * kk + quad], Sst[(4 * kk + quad) * CS + 16 * w + r16],
-                                                   acc, 0, 0, 0);
-        acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(Qd[r16 * QS + 4 * kk + 4 + quad],
-                                                    Sst[(4 * kk + 4 + quad) * CS + 16 * w + r16], acc2, 0, 0, 0);
-      }
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(o.a[0], v[0], acc, 0, 0, 0);
+    acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.a[1], v[1], acc2, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(o.a[2], v[2], acc, 0, 0, 0);
+    acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.a[3], v[3], acc2, 0, 0, 0);
 #pragma unroll
-      for (int kk = 0; kk < CT / 4; kk += 2) {
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(As[r16 * AS + 4 * kk + quad], Vs[(4 * kk + quad) * CS + 16 * w + r16],
-                                                   acc, 0, 0, 0);
-        acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(As[r16 * AS + 4 * kk + 4 + quad],
-                                                    Vs[(4 * kk + 4 + quad) * CS + 16 * w + r16], acc2, 0, 0, 0);
-      }
-      acc += acc2;
-      const int c = col0 + 16 * w + r16;
+    for (int rb = 0; rb < NB; ++rb) s[rb] *= o.e[rb];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = 4 * quad + i;
-        if (t < nt && c < V) obuf[((size_t)(tb + t) * NH + hd) * V + c] = acc[i];
-      }
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int rb = 0; rb < NB; ++rb) s[rb] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.k[rb][i], v[i], s[rb], 0, 0, 0);
+    acc += acc2;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = tb + 4 * quad + i;
+      if (t < t_hi && has) obuf[((size_t)t * NH + hd) * V + c] = acc[i];
     }
-    __syncthreads();  // every read of the old state is done
-    for (int rb = w; rb < DP / 16; rb += 4) {  // state to the end of the chunk's nt tokens
-      f32x4 acc[4];
-#pragma unroll
-      for (int cb = 0; cb < 4; ++cb) acc[cb] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int kk = 0; kk < CT / 4; ++kk) {
-        const float a = Kd[(4 * kk + quad) * QS + 16 * rb + r16];
-#pragma unroll
-        for (int cb = 0; cb < 4; ++cb)
-          acc[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, Vs[(4 * kk + quad) * CS + 16 * cb + r16], acc[cb], 0, 0, 0);
-      }
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = 16 * rb + 4 * quad + i;
-        const float dec = Es[d];
-#pragma unroll
-        for (int cb = 0; cb < 4; ++cb) {
-          float* p = Sst + d * CS + 16 * cb + r16;
-          *p = dec * *p + acc[cb][i];
-        }
-      }
-    }
+  };
+  // three sets of operands: a chunk's loads are under way for two chunks
+  Operands o0, o1, o2;
+  fetch(o0, t_lo);
+  if (t_lo + CT < t_hi) fetch(o1, t_lo + CT);
+  for (int tb = t_lo; tb < t_hi; tb += 3 * CT) {
+    if (tb + 2 * CT < t_hi) fetch(o2, tb + 2 * CT);
+    chunk(o0, tb);
+    if (tb + CT >= t_hi) break;
+    if (tb + 3 * CT < t_hi) fetch(o0, tb + 3 * CT);
+    chunk(o1, tb + CT);
+    if (tb + 2 * CT >= t_hi) break;
+    if (tb + 4 * CT < t_hi) fetch(o1, tb + 4 * CT);
+    chunk(o2, tb + 2 * CT);
   }
-  __syncthreads();
-  for (int i = tid; i < DP * 64; i += 256) {
-    const int d = i / 64, c = i % 64;
-    if (d < D && col0 + c < V) S[(sbase + d) * V + col0 + c] = Sst[d * CS + c];
-  }
+#pragma unroll
+  for (int rb = 0; rb < NB; ++rb)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = 16 * rb + 4 * quad + i;
+      if (has && d < D) Sp[(size_t)d * V] = s[rb][i];
+    }
 }
 
 // One wave per (token, head): y = o / rms(o over V) * w * silu(gate)
@@ -320,13 +297,34 @@ template <typename T>
 __global__ void __launch_bounds__(256) gla_out_kernel(const float* __restrict__ obuf, const T* __restrict__ gate,
                                                       int64_t gate_stride, const T* __restrict__ w, T* __restrict__ out,
                                                       int64_t out_stride, float out_scale, int64_t n_rows, int NH, int V,
-                                                      float eps) {
+                                                      float eps, int vec) {
   const int lane = threadIdx.x & 63;
   const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= n_rows) return;
   const int64_t t = row / NH;
   const int hd = (int)(row % NH);
   const float* o = obuf + row * V;
+  if (vec) {  // rows of a multiple of 4 numbers, 8- / 16-byte aligned: four a lane and step
+    float ss = 0.f;
+    for (int i = 4 * lane; i < V; i += 256) {
+      const f32x4 x = *reinterpret_cast<const f32x4*>(o + i);
+      ss += x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+    }
+    const float r = 1.f / sqrtf(wave_sum(ss) / (float)V + eps) * out_scale;
+    typedef T t4 __attribute__((ext_vector_type(4)));
+    for (int i = 4 * lane; i < V; i += 256) {
+      const f32x4 x = *reinterpret_cast<const f32x4*>(o + i);
+      const t4 g4 = *reinterpret_cast<const t4*>(gate + t * gate_stride + hd * V + i), w4 = *reinterpret_cast<const t4*>(w + i);
+      t4 y;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float g = (float)g4[e];
+        y[e] = (T)(x[e] * r * (float)w4[e] * (g / (1.f + (sizeof(T) == 2 ? __expf(-g) : expf(-g)))));
+      }
+      *reinterpret_cast<t4*>(out + t * out_stride + hd * V + i) = y;
+    }
+    return;
+  }
   float ss = 0.f;
   for (int i = lane; i < V; i += 64) ss += o[i] * o[i];
   const float r = 1.f / sqrtf(wave_sum(ss) / (float)V + eps);
@@ -338,10 +336,16 @@ __global__ void __launch_bounds__(256) gla_out_kernel(const float* __restrict__ 
 
 }  // namespace
 
+// Floats of the chunked form's scratch.
+extern "C" int64_t areal_gla_scratch(int T, int B, int NH, int D) {
+  const size_t per = D <= 32 ? chunk_floats<32>() : (D <= 64 ? chunk_floats<64>() : chunk_floats<128>());
+  return (int64_t)(T / CT + B + 1) * NH * per;
+}
+
 // proj rows hold (at q_off / k_off / v_off) NH query heads of D, NH key heads of D, NH value heads of V. z fp32 rows of
 // NH D decay logits (z_stride apart), z_bias [NH D] in the storage type or null. S [slots, NH, D, V] fp32; obuf
-// [T, NH, V] fp32. scratch: T (3 NH D + 16 NH) floats for the chunked form (rows of 16 tokens and more, D <= 128), or
-// null: token by token.
+// [T, NH, V] fp32. scratch: areal_gla_scratch floats, 16-byte aligned, for the chunked form (rows of 16 tokens and more,
+// D <= 128), or null: token by token.
 extern "C" int areal_gla_scan(const void* proj, int64_t row_stride, int q_off, int k_off, int v_off, const float* z,
                               int64_t z_stride, const void* z_bias, float tau, float q_scale, const int* cu_q,
                               const int* first_pos, const int* state_slots, float* S, float* obuf, float* scratch, int T,
@@ -351,23 +355,13 @@ extern "C" int areal_gla_scan(const void* proj, int64_t row_stride, int q_off, i
   const dim3 grid(B, NH, (V + 63) / 64);
   const float inv_tau = 1.f / tau;
   if (max_q >= CT && D <= 128 && scratch) {
-    // scratch: q~ | k~ | exp(b_L) as [T, NH D] each, then A as [T, NH, CT]
-    const size_t N = (size_t)NH * D;
-    float *qd = scratch, *kd = qd + (size_t)T * N, *el = kd + (size_t)T * N, *ab = el + (size_t)T * N;
     const dim3 pgrid((max_q + CT - 1) / CT, B, NH);
-#define CHUNK(TT, DPV)                                                                                              \
-  do {                                                                                                              \
-    const size_t lds = sizeof(float) * ((size_t)DPV * 68 + 2 * (size_t)CT * (DPV + 4) + (size_t)CT * 68 + CT * (CT + 1) + DPV); \
-    static bool raised = false;                                                                                     \
-    if (!raised && lds > 64 * 1024) {                                                                               \
-      HIP_RET(hipFuncSetAttribute((const void*)gla_chunk_kernel<DPV>, hipFuncAttributeMaxDynamicSharedMemorySize,   \
-                                  160 * 1024));                                                                     \
-      raised = true;                                                                                                \
-    }                                                                                                               \
-    hipLaunchKernelGGL((gla_prep_kernel<TT, DPV>), pgrid, dim3(256), 0, st, (const TT*)proj, row_stride, q_off, k_off, \
-                       z, z_stride, (const TT*)z_bias, inv_tau, q_scale, cu_q, state_slots, qd, kd, el, ab, NH, D);  \
-    hipLaunchKernelGGL((gla_chunk_kernel<DPV>), grid, dim3(256), lds, st, qd, kd, el, ab, proj, row_stride, v_off,  \
-                       dt == 0 ? 1 : 0, cu_q, first_pos, state_slots, S, obuf, NH, D, V);                           \
+#define CHUNK(TT, DPV)                                                                                                 \
+  do {                                                                                                                 \
+    hipLaunchKernelGGL((gla_prep_kernel<TT, DPV>), pgrid, dim3(256), 0, st, (const TT*)proj, row_stride, q_off, k_off,  \
+                       z, z_stride, (const TT*)z_bias, inv_tau, q_scale, cu_q, state_slots, scratch, NH, D);            \
+    hipLaunchKernelGGL((gla_chunk_kernel<TT, DPV>), grid, dim3(256), 0, st, scratch, (const TT*)proj, row_stride,       \
+                       v_off, cu_q, first_pos, state_slots, S, obuf, NH, D, V);                                        \
   } while (0)
 #define PICKC(TT)                    \
   do {                               \
@@ -406,11 +400,13 @@ extern "C" int areal_gla_out(const float* obuf, const void* gate, int64_t gate_s
   if (T == 0) return 0;
   const int64_t n = (int64_t)T * NH;
   const dim3 grid((unsigned)((n + 3) / 4));
+  const int vec = V % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && (uintptr_t)obuf % 16 == 0 &&
+                  (((uintptr_t)gate | (uintptr_t)w | (uintptr_t)out) % (dt == 0 ? 8 : 16)) == 0;
   if (dt == 0)
     hipLaunchKernelGGL(gla_out_kernel<bf16_t>, grid, dim3(256), 0, st, obuf, (const bf16_t*)gate, gate_stride,
-                       (const bf16_t*)w, (bf16_t*)out, out_stride, out_scale, n, NH, V, eps);
+                       (const bf16_t*)w, (bf16_t*)out, out_stride, out_scale, n, NH, V, eps, vec);
   else
     hipLaunchKernelGGL(gla_out_kernel<float>, grid, dim3(256), 0, st, obuf, (const float*)gate, gate_stride,
-                       (const float*)w, (float*)out, out_stride, out_scale, n, NH, V, eps);
+                       (const float*)w, (float*)out, out_stride, out_scale, n, NH, V, eps, vec);
   return (int)hipGetLastError();
 }

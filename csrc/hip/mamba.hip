@@ -23,7 +23,17 @@ template <typename T> DEVINL void stf(T* p, size_t i, float v);
 template <> DEVINL void stf<bf16_t>(bf16_t* p, size_t i, float v) { p[i] = f2bf(v); }
 template <> DEVINL void stf<float>(float* p, size_t i, float v) { p[i] = v; }
 
-DEVINL float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// bf16 storage: hardware exponential and logarithm (a short series where 1 + e would lose e's digits)
+template <typename T> DEVINL float softplus(float z) {
+  if (sizeof(T) == 2) {
+    const float e = __expf(-fabsf(z));
+    return fmaxf(z, 0.f) + (e < 0.0156f ? e * (1.f - e * (0.5f - 0.33333333f * e)) : __logf(1.f + e));
+  }
+  return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+}
+template <typename T> DEVINL float silu(float z) {
+  return sizeof(T) == 2 ? z * __builtin_amdgcn_rcpf(1.f + __expf(-z)) : z / (1.f + expf(-z));
+}
 // bf16 storage: v_exp_f32 (relative error ~1e-6, far below the storage's); fp32 storage: the library's
 template <typename T> DEVINL float exp2_le0(float x) { return sizeof(T) == 2 ? fast_exp2(x) : exp2f(x); }
 constexpr float LOG2E = 1.4426950408889634f;
@@ -85,7 +95,8 @@ __global__ void __launch_bounds__(64 * RW) selective_scan_kernel(
     float cx[EC], cz[EC];
 #pragma unroll
     for (int e = 0; e < EC; ++e) {
-      const float d = softplus(fr[e] + bias);
+      // tokens past the row's end leave the state as it is: step size zero
+      const float d = tb + w + RW * e < t_hi ? softplus<T>(fr[e] + bias) : 0.f;
       sdt[w + RW * e][lane] = d;
       sdx[w + RW * e][lane] = d * fx[e];
       cx[e] = fx[e];
@@ -101,8 +112,8 @@ __global__ void __launch_bounds__(64 * RW) selective_scan_kernel(
     }
     if (tb + TC < t_hi) fetch(tb + TC);
     __syncthreads();
-#pragma unroll 4
-    for (int tt = 0; tt < nt; ++tt) {
+#pragma unroll
+    for (int tt = 0; tt < TC; ++tt) {
       const float d = sdt[tt][lane], u = sdx[tt][lane];
       float y = 0.f;
 #pragma unroll
@@ -121,7 +132,7 @@ __global__ void __launch_bounds__(64 * RW) selective_scan_kernel(
 #pragma unroll
         for (int k = 0; k < RW; ++k) y += part[k][tt][lane];
         y += dsk * cx[e];
-        stf<T>(out, (size_t)(tb + tt) * I + c, y * (cz[e] / (1.f + expf(-cz[e]))));
+        stf<T>(out, (size_t)(tb + tt) * I + c, y * silu<T>(cz[e]));
       }
     }
     __syncthreads();  // the partials and the staged operands are free
