@@ -1777,9 +1777,15 @@ class HybridDecoder(nn.Module):
         return {f"l{i}.mix.vmix" for i, blk in enumerate(self.layers)
                 if blk.kind == "attention" and blk.mix.v_mix != "mix"}
 
+    def checkpoint_unread(self) -> set:
+        """Names a checkpoint may hold although no layer reads them: what belongs to a feed-forward a layer does not have."""
+        if not self.post_add:
+            return set()
+        return {f"l{i}.{n}" for i, blk in enumerate(self.layers) if blk.mlp is None for n in ("norm2", "norm2.b", "canon2")}
+
     def assign_named_tensors(self, tensors: Dict[str, torch.Tensor], strict: bool = True):
         views = self.checkpoint_tensors()
-        unknown = [n for n in tensors if n not in views]
+        unknown = [n for n in tensors if n not in views and n not in self.checkpoint_unread()]
         if strict and unknown:
             raise KeyError(f"{len(unknown)} tensor(s) map onto no parameter of this model: {sorted(unknown)[:8]}")
         for n, t in tensors.items():

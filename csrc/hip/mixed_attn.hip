@@ -214,7 +214,7 @@ DEVINL int key_row(int r16) { return 8 * (r16 >> 2) + (r16 & 3); }
 // the four lanes of a query at the end. The next page's keys are fetched under the current one's work. SHARED: the wave's
 // heads read one key head.
 template <int DK, bool SHARED, int HPW>
-__global__ void __launch_bounds__(512) mixed_lse_kernel(
+__global__ void __launch_bounds__(512, 2) mixed_lse_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kcache, const int* __restrict__ block_tables, int max_pages,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_len, float* __restrict__ lse, int H, int G, float scale_log2) {
   constexpr int D = 32 * DK;
@@ -236,20 +236,20 @@ __global__ void __launch_bounds__(512) mixed_lse_kernel(
   const int n_pages = (pos0 + nq + PAGE - 1) / PAGE;
   const int* bt = block_tables + (size_t)b * max_pages;
   const int row_off = key_row(r16) * D + 8 * quad;
-  auto load_keys = [&](bf16x8 (&k)[2][DK], int pg, int c) {
-    const bf16_t* kp = kcache + ((size_t)bt[pg] * G + c) * PAGE * D + row_off;
+  auto load_keys = [&](bf16x8 (&k)[2][DK], int page, int c) {
+    const bf16_t* kp = kcache + ((size_t)page * G + c) * PAGE * D + row_off;
 #pragma unroll
     for (int ks = 0; ks < DK; ++ks) {
       k[0][ks] = ld8(kp + 32 * ks);
       k[1][ks] = ld8(kp + 4 * D + 32 * ks);
     }
   };
-  auto page_step = [&](bf16x8 (&k)[2][DK], int pg) {
+  auto page_step = [&](bf16x8 (&k)[2][DK], int pg, int page) {
     const int jb = pg * PAGE;
     const bool edge = jb + PAGE - 1 > pos0;  // some query of the tile does not see the whole page
 #pragma unroll
     for (int hh = 0; hh < HPW; ++hh) {
-      if (!SHARED && hh > 0) load_keys(k, pg, (h0 + hh) / rep);
+      if (!SHARED && hh > 0) load_keys(k, page, (h0 + hh) / rep);
       f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < DK; ++ks) {
@@ -277,13 +277,19 @@ __global__ void __launch_bounds__(512) mixed_lse_kernel(
     }
   };
   bf16x8 k0[2][DK], k1[2][DK];
-  load_keys(k0, 0, h0 / rep);
+  // page ids are fetched ahead of the keys they lead to
+  int id0 = bt[0], id1 = bt[min(1, n_pages - 1)], id2 = bt[min(2, n_pages - 1)];
+  load_keys(k0, id0, h0 / rep);
   for (int pg = 0; pg < n_pages; pg += 2) {
-    if (pg + 1 < n_pages) load_keys(k1, pg + 1, h0 / rep);
-    page_step(k0, pg);
+    const int id3 = bt[min(pg + 3, n_pages - 1)], id4 = bt[min(pg + 4, n_pages - 1)];
+    if (pg + 1 < n_pages) load_keys(k1, id1, h0 / rep);
+    page_step(k0, pg, id0);
     if (pg + 1 >= n_pages) break;
-    if (pg + 2 < n_pages) load_keys(k0, pg + 2, h0 / rep);
-    page_step(k1, pg + 1);
+    if (pg + 2 < n_pages) load_keys(k0, id2, h0 / rep);
+    page_step(k1, pg + 1, id1);
+    id0 = id2;
+    id1 = id3;
+    id2 = id4;
   }
 #pragma unroll
   for (int hh = 0; hh < HPW; ++hh) {
@@ -301,13 +307,14 @@ __global__ void __launch_bounds__(512) mixed_lse_kernel(
 //   values   O^T += V^T W^T per owned head, two products (hi, lo)
 // The weights' LDS buffer is double: one barrier a page. Keys of the next page are fetched ahead.
 template <int DK, int VT, bool SHARED, int NW, int HPW>
-__global__ void __launch_bounds__(64 * NW, (NW > 8 ? 4 : 2)) mixed_apply_kernel(
+__global__ void __launch_bounds__(64 * NW, (NW * HPW == 16 && HPW == 4 ? 1 : 2)) mixed_apply_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kcache, const bf16_t* __restrict__ vcache,
     const int* __restrict__ block_tables, int max_pages, const int* __restrict__ cu_q, const int* __restrict__ ctx_len,
     const bf16_t* __restrict__ mix, const float* __restrict__ lse, bf16_t* __restrict__ out, int64_t out_stride, int G,
     float scale_log2, float out_scale) {
   constexpr int D = 32 * DK, V = 16 * VT, H = HPW * NW, NP = (H + 7) / 8;  // 16-byte pieces of the hi (and lo) halves
-  constexpr bool AHEAD = SHARED && HPW * (8 * VT / 2 + 4 * DK) < 160;     // registers left for the keys of the next page
+  // registers left for the next page's keys (four waves a workgroup, one a SIMD: all of the register file)
+  constexpr bool AHEAD = SHARED && (HPW * (8 * VT / 2 + 4 * DK) < 160 || NW == 4);
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int b = blockIdx.x, tile = gridDim.y - 1 - blockIdx.y;
   const int q0 = cu_q[b], qlen = cu_q[b + 1] - q0, t0 = tile * 16;
@@ -333,23 +340,25 @@ __global__ void __launch_bounds__(64 * NW, (NW > 8 ? 4 : 2)) mixed_apply_kernel(
   const int* bt = block_tables + (size_t)b * max_pages;
   const int row_off = key_row(r16) * D + 8 * quad;
   bf16x8 k[2][DK];
-  auto load_keys = [&](int pg, int c) {
-    const bf16_t* kp = kcache + ((size_t)bt[pg] * G + c) * PAGE * D + row_off;
+  auto load_keys = [&](int id, int c) {
+    const bf16_t* kp = kcache + ((size_t)id * G + c) * PAGE * D + row_off;
 #pragma unroll
     for (int ks = 0; ks < DK; ++ks) {
       k[0][ks] = ld8(kp + 32 * ks);
       k[1][ks] = ld8(kp + 4 * D + 32 * ks);
     }
   };
-  if (AHEAD) load_keys(0, HPW * w / rep);
+  int id = bt[0], id_next = bt[min(1, n_pages - 1)];  // page ids are fetched ahead of what they lead to
+  if (AHEAD) load_keys(id, HPW * w / rep);
   for (int pg = 0; pg < n_pages; ++pg) {
     char* buf = smem + (pg & 1) * (8 * 2 * NP * 64 * 16);
-    const size_t page = (size_t)bt[pg] * G;
+    const int id_after = bt[min(pg + 2, n_pages - 1)];
+    const size_t page = (size_t)id * G;
     const int jb = pg * PAGE;
     float p[HPW][8];
 #pragma unroll
     for (int hh = 0; hh < HPW; ++hh) {
-      if (!AHEAD && (hh == 0 || !SHARED)) load_keys(pg, (HPW * w + hh) / rep);
+      if (!AHEAD && (hh == 0 || !SHARED)) load_keys(id, (HPW * w + hh) / rep);
       f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < DK; ++ks) {
@@ -373,7 +382,7 @@ __global__ void __launch_bounds__(64 * NW, (NW > 8 ? 4 : 2)) mixed_apply_kernel(
       }
     };
     if (SHARED) load_values(HPW * w / rep);
-    if (AHEAD && pg + 1 < n_pages) load_keys(pg + 1, HPW * w / rep);
+    if (AHEAD && pg + 1 < n_pages) load_keys(id_next, HPW * w / rep);
     if (jb + PAGE - 1 > pos0) {
       const int last = pos0 + r16 - jb - 8 * quad;
 #pragma unroll
@@ -427,6 +436,8 @@ __global__ void __launch_bounds__(64 * NW, (NW > 8 ? 4 : 2)) mixed_apply_kernel(
 #pragma unroll
       for (int vt = 0; vt < VT; ++vt) acc[hh][vt] = mfma16(vf[vt], wl[hh], acc[hh][vt]);
     }
+    id = id_next;
+    id_next = id_after;
   }
   if (r16 < nq) {
 #pragma unroll
@@ -667,21 +678,24 @@ extern "C" int areal_mixed_attn_prompt(const void* q, const void* kcache, const 
   if (out_stride % 4 != 0 || (uintptr_t)out % 8 != 0 || (uintptr_t)mix % 8 != 0) return -2;
   if ((max_q + 15) / 16 > 65535) return -3;
   const float s2 = scale * LOG2E;
-  const int hpw = H == 32 ? 4 : 2, nw = H / hpw;  // heads per wave of the second pass
-  const bool shared2 = (H / G) % 2 == 0, shared = (H / G) % hpw == 0;
+  // heads per wave of the second pass; at 16 heads four of one key head: a page's keys and values are loaded once
+  const int hpw = H == 32 || (H == 16 && (H / G) % 4 == 0) ? 4 : 2, nw = H / hpw;
+  const bool shared = (H / G) % hpw == 0;
   const size_t lds = (size_t)2 * 8 * 2 * ((H + 7) / 8) * 64 * 16;
-  // the first pass: two heads a wave, at most 8 waves a workgroup
-  const int lw = H / 2 < 8 ? H / 2 : 8;
-#define STATS(DKV, SH)                                                                                               \
-  hipLaunchKernelGGL((mixed_lse_kernel<DKV, SH, 2>), dim3(B, (max_q + 15) / 16, H / (2 * lw)), dim3(64 * lw), 0, st,   \
-                     (const bf16_t*)q, (const bf16_t*)kcache, block_tables, max_pages, cu_q, ctx_len, lse, H, G, s2)
-  if (D == 128) {
-    if (shared2) STATS(4, true);
-    else STATS(4, false);
-  } else {
-    if (shared2) STATS(2, true);
-    else STATS(2, false);
-  }
+  // the first pass: four heads a wave where they read one key head (a page's keys are loaded once), else two
+#define STATS_W(DKV, SH, HW)                                                                                         \
+  hipLaunchKernelGGL((mixed_lse_kernel<DKV, SH, HW>), dim3(B, (max_q + 15) / 16, (H / HW + 7) / 8),                    \
+                     dim3(64 * (H / HW < 8 ? H / HW : 8)), 0, st, (const bf16_t*)q, (const bf16_t*)kcache,            \
+                     block_tables, max_pages, cu_q, ctx_len, lse, H, G, s2)
+#define STATS(DKV)                                       \
+  do {                                                   \
+    if ((H / G) % 4 == 0) STATS_W(DKV, true, 4);         \
+    else if ((H / G) % 2 == 0) STATS_W(DKV, true, 2);    \
+    else STATS_W(DKV, false, 2);                         \
+  } while (0)
+  if (D == 128) STATS(4);
+  else STATS(2);
+#undef STATS_W
 #undef STATS
 #define APPLY(DKV, VTV, SH, NWV, HPWV)                                                                              \
   do {                                                                                                              \
@@ -698,7 +712,8 @@ extern "C" int areal_mixed_attn_prompt(const void* q, const void* kcache, const 
 #define APPLY_NW(DKV, VTV, SH)                     \
   do {                                             \
     if (nw == 2) APPLY(DKV, VTV, SH, 2, 2);        \
-    else if (nw == 4) APPLY(DKV, VTV, SH, 4, 2);   \
+    else if (nw == 4 && hpw == 2) APPLY(DKV, VTV, SH, 4, 2); \
+    else if (nw == 4) APPLY(DKV, VTV, SH, 4, 4);   \
     else if (H == 16) APPLY(DKV, VTV, SH, 8, 2);   \
     else APPLY(DKV, VTV, SH, 8, 4);                \
   } while (0)

@@ -708,6 +708,11 @@ def test_config_reader_and_checkpoint_save_then_load(tmp_path):
     m2.load_checkpoint(str(tmp_path))
     for (n1, a), (n2, b) in zip(m.checkpoint_tensors().items(), m2.checkpoint_tensors().items()):
         assert n1 == n2 and torch.equal(a, b)
+    extra = dict(m2.checkpoint_tensors(), **{"l0.norm3": torch.zeros(40)})
+    with pytest.raises(KeyError):
+        m2.assign_named_tensors(extra)
+    no_ff = [i for i, l in enumerate(cfg.layers) if l["mlp"] is None][0]  # what a missing feed-forward would own is not read
+    m2.assign_named_tensors({f"l{no_ff}.norm2": torch.zeros(40), f"l{no_ff}.canon2": torch.zeros(40, 5)})
     bad = side()
     del bad["mixer"]["right"]["decay_rank"]
     for l in (dict(attn(), type="conv"), attn(rdims=3), attn(heads=3, kv=2), bad, dict(mamba(), mlp={"kind": "moe"})):
