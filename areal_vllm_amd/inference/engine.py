@@ -160,8 +160,8 @@ class NativeInferenceEngine:
                 blk = self.model.layers[li]
                 if hasattr(blk, "paged"):  # blocks that name the mixer with a paged cache
                     if blk.paged() is not None:
-                        g, d, v = blk.paged().cache_shape()
-                        per_tok += g * (d + v)
+                        shape = blk.paged().cache_shape()  # (heads, key size, value size), or (latent, rotary part)
+                        per_tok += shape[0] * (shape[1] + shape[2]) if len(shape) == 3 else sum(shape)
                 elif blk.kind == "attention":
                     g, d, v = blk.mix.cache_shape()
                     per_tok += g * (d + v)

@@ -875,7 +875,12 @@ class HybridModelRunner(ModelRunner):
         self.parallel = bool(getattr(self.model, "parallel", False))
         self.prepost = bool(getattr(self.model, "prepost", False))
         self.post_add = bool(getattr(self.model, "post_add", False))
-        self.keeps_positions = self.sandwich or self.parallel or self.prepost or self.post_add
+        self.tanh_norm = bool(getattr(self.model, "tanh_norm", False))
+        self.keeps_positions = self.sandwich or self.parallel or self.prepost or self.post_add or self.tanh_norm
+        if self.tanh_norm:
+            from ..ops.tanh_norm import sinusoid_frequencies
+
+            self.pos_freq = sinusoid_frequencies(self.cfg.hidden_size, 10000.0, self.device)
         # one cache / state per layer RUN: a layer that runs several times keeps every pass apart
         self.layer_runs = list(getattr(self.model, "layer_runs", range(len(self.model.layers))))
         self.kv, self.state = [], []
@@ -958,6 +963,8 @@ class HybridModelRunner(ModelRunner):
             return self._run_layers_prepost(xc, st)
         if self.post_add:
             return self._run_layers_post_add(xc, st)
+        if self.tanh_norm:
+            return self._run_layers_tanh_norm(xc, st)
         x32 = xc.float() if xc.dtype != torch.float32 else xc.clone()
         alpha, eps = float(cfg.postln_alpha), float(cfg.rms_norm_eps)
         trace = getattr(self, "layer_trace", None)
@@ -1076,8 +1083,56 @@ class HybridModelRunner(ModelRunner):
                 trace.append(x.clone())
         return x
 
+    def _run_layers_tanh_norm(self, ids: torch.Tensor, st) -> torch.Tensor:
+        """Token ids -> fp32 residual stream after the last layer run. One launch closes a sublayer (recombination of the
+        experts, norm, sum) and forms the norm the next one reads. A pass over the loop's span is entered with
+        x <- W_in [x; x_0] + step: the product with x_0 is the same for every pass and formed once."""
+        from ..models.hybrid import linear32
+        from ..ops import tanh_norm as tn
+
+        model = self.model
+        blocks = [model.layers[li] for li in self.layer_runs]
+        starts = self.cfg.pass_starts
+        trace = getattr(self, "layer_trace", None)
+        x, xc = tn.embed_sinusoid(ids, st.positions, model.embed, self.pos_freq, want_copy=bool(starts))
+        W = x.shape[1]
+        c = linear32(xc, model.loop_in[:, W:]) if starts else None
+
+        def opening(ri):  # what the launch ahead of layer run ri hands on: (its norm or None, whether a copy of the stream)
+            if ri >= len(blocks):
+                return None, False
+            return (None, True) if ri in starts else (blocks[ri].norm1.args(), False)
+
+        if 0 not in starts:
+            _, _, xc = tn.norm_add(x, None, None, blocks[0].norm1.args(), self.dtype)
+        for ri, blk in enumerate(blocks):
+            hc = xc
+            if ri in starts:
+                p = linear32(xc, model.loop_in[:, :W])
+                x, _, hc = tn.enter_pass(p, c, model.loop_step[starts[ri]], x, blk.norm1.args(), self.dtype)
+            y = blk.mix.step(hc, st, self.kv[ri] if blk.paged() is not None else self.state[ri])
+            nxt, copy = opening(ri + 1)
+            if blk.mlp is not None:
+                x, h32, hc = tn.norm_add(x, y, blk.norm1b.args(), blk.norm2.args(), self.dtype, want32=blk.needs32)
+                y = blk.mlp.step(hc, h32, st)
+                x, _, xc = tn.norm_add(x, y, blk.norm2b.args(), nxt, self.dtype, want_copy=copy)
+            else:
+                x, _, xc = tn.norm_add(x, y, blk.norm1b.args(), nxt, self.dtype, want_copy=copy)
+            if trace is not None:
+                trace.append(x.clone())
+        return x
+
     def _final_logits(self, h, residual, fp32: bool = False) -> torch.Tensor:
         from ..ops.post_norm import scaled_add_norm
+
+        if self.tanh_norm:
+            from ..ops import tanh_norm as tn
+
+            want32 = fp32 or self.keep_logits
+            _, h32, hc = tn.norm_add(h.contiguous(), None, None, self.model.norm.args(), self.dtype, want32=want32)
+            z = F.linear(h32, self.model.head_weight.float()) if want32 else self._lm_head(hc)
+            cap = float(self.cfg.logit_softcap)
+            return tn.softcap_(z, cap) if cap > 0 else z
 
         if self.prepost:
             from ..ops import depth_avg as da
@@ -1171,10 +1226,10 @@ class HybridModelRunner(ModelRunner):
                            for i in range(2))
             return nsplit, ws
         latent = [blk.mix for blk in self.model.layers if blk.kind == "latent_attention"]
-        if self.prepost and self.device.type == "cuda":
+        if (self.prepost or self.tanh_norm) and self.device.type == "cuda":
             # mixers of several kinds share one workspace; each takes its own share of the step's splits
             need = [(m.decode_splits(Bp, self.max_context), m.H * (m.R if blk.kind == "latent_attention" else m.V), m.H)
-                    for blk in self.model.layers if blk.kind != "gla" for m in (blk.mix,)]
+                    for blk in self.model.layers if blk.kind not in ("gla", "channel_delta") for m in (blk.mix,)]
             nsplit = max([n for n, _, _ in need] or [1])
             if nsplit > 1:
                 ws = (torch.empty(Bp * max(n * a for n, a, _ in need), dtype=torch.float32, device=self.device),
@@ -1211,4 +1266,6 @@ class HybridModelRunner(ModelRunner):
                            nsplit=st["nsplit"], workspace=st["ws"], positions=st["positions"])
         if self.post_add:
             step.decode_gemms = self._decode_gemms(Bp)
+        elif self.tanh_norm and self.dtype == torch.bfloat16 and self.device.type == "cuda":
+            step.decode_gemms = {}  # closing products go through the split decode GEMM; its slabs are summed by the norm
         return self._final_logits(self._run_layers(h, step), None)

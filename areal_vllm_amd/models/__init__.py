@@ -5,7 +5,7 @@ from .hybrid import HybridConfig, HybridDecoder  # noqa: F401
 
 # model family (``ModelConfig.family``) -> class; every family not listed is a ``Transformer`` variant
 MODEL_CLASSES = {"kuzanex": HybridDecoder, "lufivik": HybridDecoder, "pobelorn": HybridDecoder,
-                 "zusotar": HybridDecoder, "gusolix": HybridDecoder}
+                 "zusotar": HybridDecoder, "gusolix": HybridDecoder, "keginex": HybridDecoder}
 
 
 def model_class(cfg: ModelConfig):

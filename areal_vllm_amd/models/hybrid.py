@@ -47,13 +47,24 @@ Mixers:     grouped-query attention inside chunks of positions, RMS norm over al
 ff:         gated MLP
 Embedding:  table row times a constant
 
+The Keginex design is the sixth member. An element-wise norm, tanh(alpha z) w + b, stands before and after a sublayer:
+
+Layer:      x <- x + norm1b(mixer(norm1(x)));  x <- x + norm2b(ff(norm2(x)))
+Mixers:     gated delta rule with a decay per head and key channel (queries, keys and values behind short convolutions,
+            fp32 state);  or causal attention through a shared latent without positions (query latent, one sink logit per
+            head in the softmax denominator)
+ff:         squared-ReLU MLP, or routed gated experts (softmax scores, a learned correction of the choice, group-limited,
+            weights renormalised) plus a shared expert behind a sigmoid gate of its own
+Embedding:  table row plus a sinusoidal position vector;  a span of layers may run several times: every pass is entered
+            through a projection of stream and embedding, plus a vector of the pass;  soft cap on the logits
+
 The mechanisms are separate modules with their constants as constructor arguments (``WindowAttentionMixer``,
 ``MLSTMMixer``, ``XieluMLP``, ``LatentAttentionMixer``, ``RoutedGLUExperts``, ``RotaryWindowAttentionMixer``,
 ``LightningMixer``, ``SquaredReluMLP``, ``RoutedSwiGLUExperts``, ``LogBiasWindowAttentionMixer``, ``GLAMixer``,
-``GatedMLP``, ``RowNormAttentionMixer``, ``MixedAttentionMixer``, ``MambaMixer``, ``SideBySideMixer``); what they compute is
+``GatedMLP``, ``RowNormAttentionMixer``, ``MixedAttentionMixer``, ``MambaMixer``, ``SideBySideMixer``, ``ChannelDeltaMixer``); what they compute is
 documented with their kernels (``ops/window_attention.py``, ``ops/mlstm.py``, ``ops/post_norm.py``, ``ops/latent_attention.py``,
 ``ops/sandwich.py``, ``ops/lightning.py``, ``ops/parallel_block.py``, ``ops/gla.py``, ``ops/depth_avg.py``,
-``ops/mixed_attention.py``, ``ops/mamba.py``). The modules hold parameters and know how to run ONE step on the tensors of a
+``ops/mixed_attention.py``, ``ops/mamba.py``, ``ops/delta_rule.py``, ``ops/tanh_norm.py``). The modules hold parameters and know how to run ONE step on the tensors of a
 batch plan; paged caches, state slots and the loop over layers belong to the model runner
 (``inference/model_runner.py::HybridModelRunner``).
 """
@@ -68,6 +79,7 @@ import torch.nn.functional as F
 
 from .. import ops
 from ..ops import decode_gemm, train_gemm
+from ..ops import delta_rule
 from ..ops import depth_avg as davg
 from ..ops import gla as gla_ops
 from ..ops import lightning as lightning_ops
@@ -77,7 +89,7 @@ from ..ops import mlstm as mlstm_ops
 from ..ops import parallel_block as pblock
 from ..ops import latent_attention as lattn
 from ..ops import moe as moe_ops
-from ..ops import post_norm, sandwich, window_attention as wattn
+from ..ops import post_norm, sandwich, tanh_norm, window_attention as wattn
 from ..ops.grouped_gemm import grouped_gemm_rows
 from .config import ModelConfig
 from .transformer import FlatParams
@@ -93,7 +105,8 @@ class HybridConfig(ModelConfig):
     # "post_norm": norm after every sum; "sandwich": layer norms before and after a sublayer, gated; "parallel": one
     # norm, mixer and feed-forward read it and are added together; "prepost": RMS norms before and after a sublayer,
     # the normed output times `residual_mult` added to the stream, optionally averaged over depth; "post_add": layer norm
-    # on a sublayer's output, which is added to the stream; sublayers read the stream through a short convolution
+    # on a sublayer's output, which is added to the stream; sublayers read the stream through a short convolution;
+    # "tanh_norm": an element-wise norm before and after a sublayer
     block_style: str = "post_norm"
     residual_mult: float = 1.0  # factor on every normed sublayer output ("prepost" designs)
     depth_average: bool = False  # the stream that leaves a layer is a learned average of all streams so far
@@ -101,10 +114,11 @@ class HybridConfig(ModelConfig):
     loop: Optional[Dict[str, int]] = None  # layers start .. stop - 1 run `times` times in a row
     canon_taps: int = 0  # taps of the causal convolution on a mixer's ("post_add": every sublayer's) input (0: none)
     bigram: Optional[Dict[str, int]] = None  # hashed-bigram embedding: buckets, mul_prev, mul_cur
+    logit_softcap: float = 0.0  # logits <- cap tanh(logits / cap) (0: none)
 
     @property
     def has_recurrent_state(self) -> bool:
-        return (any(l["type"] in ("mlstm", "lightning", "gla", "mamba1", "parallel") for l in self.layers)
+        return (any(l["type"] in ("mlstm", "lightning", "gla", "mamba1", "parallel", "channel_delta") for l in self.layers)
                 or self.canon_taps > 1
                 or self.bigram is not None)
 
@@ -117,6 +131,14 @@ class HybridConfig(ModelConfig):
         a, b, k = int(self.loop["start"]), int(self.loop["stop"]), int(self.loop["times"])
         return list(range(a)) + list(range(a, b)) * k + list(range(b, n))
 
+    @property
+    def pass_starts(self) -> Dict[int, int]:
+        """Place in `layer_runs` -> number of the pass over the loop's span that begins there."""
+        if not self.loop:
+            return {}
+        a, b, k = int(self.loop["start"]), int(self.loop["stop"]), int(self.loop["times"])
+        return {a + t * (b - a): t for t in range(k)}
+
     def n_params(self, with_embedding: bool = True) -> int:
         if self.block_style == "sandwich":
             return self._n_params_sandwich(with_embedding)
@@ -126,6 +148,8 @@ class HybridConfig(ModelConfig):
             return self._n_params_prepost(with_embedding)
         if self.block_style == "post_add":
             return self._n_params_post_add(with_embedding)
+        if self.block_style == "tanh_norm":
+            return self._n_params_tanh_norm(with_embedding)
         W, n = self.hidden_size, 1
         for l in self.layers:
             m = l["mixer"]
@@ -227,7 +251,42 @@ class HybridConfig(ModelConfig):
                 n += 2 * W + W * self.canon_taps + 3 * W * l["mlp"]["ff"]
         return n + (2 * self.vocab_size * W if with_embedding else 0)
 
+    def _n_params_tanh_norm(self, with_embedding: bool) -> int:
+        W = self.hidden_size
+        n = 2 * W + 1  # final norm
+        if self.loop:
+            n += 2 * W * W + int(self.loop["times"]) * W
+        for l in self.layers:
+            m = l["mixer"]
+            H, D, V = m["heads"], m["dim"], m["vdim"]
+            if l["type"] == "channel_delta":
+                G, C = m["kv_heads"], 2 * m["kv_heads"] * D + H * V
+                ra, rg = m["decay_rank"], m["gate_rank"]
+                n += W * (C + ra + rg + H) + C * m["conv"] + H + V + H * D * (ra + 1) + H * V * rg + W * H * V
+            else:
+                Q, R = m["q_rank"], m["kv_rank"]
+                n += W * (Q + R) + Q + R + Q * H * D + R * H * (D + V) + H + W * H * V
+            n += 2 * (2 * W + 1)
+            e = l.get("mlp")
+            if e:
+                n += 2 * (2 * W + 1)
+                if e["kind"] == "dense":
+                    n += 2 * W * e["ff"]
+                else:
+                    n += e["router"]["experts"] * (W + 1 + 3 * W * e["expert"]["ff"])
+                    if e.get("shared"):
+                        n += 3 * W * e["shared"]["ff"] + W
+        return n + (2 * self.vocab_size * W if with_embedding else 0)
+
     def to_hf_dict(self) -> Dict[str, Any]:
+        if self.block_style == "tanh_norm":  # delta-rule mixers carry their two ranks (a checkpoint's shapes give them too)
+            d = {"architecture": self.design, "layers": json.loads(json.dumps(self.layers)),
+                 "norm": {"eps": self.rms_norm_eps}, "vocab": self.vocab_size, "width": self.hidden_size}
+            if self.loop:
+                d["loop"] = dict(self.loop)
+            if self.logit_softcap:
+                d["logit_softcap"] = self.logit_softcap
+            return d
         if self.block_style == "post_add":  # right-hand mixers carry `decay_rank` (a checkpoint's shapes give it too)
             return {"architecture": self.design, "canon": {"taps": self.canon_taps},
                     "embedding": {"scale": self.embed_scale}, "layers": json.loads(json.dumps(self.layers)),
@@ -418,11 +477,11 @@ def zusotar_config_from_dir(path: str) -> HybridConfig:
     return zusotar_config(d, _first_sizes(path, {f"l{i}.mix.a1": i for i, l in enumerate(d["layers"]) if l["type"] == "gla"}))
 
 
-def _first_sizes(path: str, want: Dict[str, int]) -> Dict[int, int]:
+def _first_sizes(path: str, want: Dict[str, Any]) -> Dict[Any, int]:
     """`want`: tensor name -> key. {key: size of the tensor's first axis} for those that the checkpoint in `path` holds."""
     from safetensors import safe_open
 
-    out: Dict[int, int] = {}
+    out: Dict[Any, int] = {}
     for fn in sorted(os.listdir(path)) if want else []:
         if fn.endswith(".safetensors"):
             with safe_open(os.path.join(path, fn), framework="pt") as f:
@@ -485,6 +544,60 @@ def gusolix_config_from_dir(path: str) -> HybridConfig:
         d = json.load(f)
     return gusolix_config(d, _first_sizes(path, {f"l{i}.mix.right.a1": i for i, l in enumerate(d["layers"])
                                                  if l["type"] == "parallel"}))
+
+
+def keginex_config(d: Dict[str, Any], ranks: Optional[Dict[Any, int]] = None) -> HybridConfig:
+    """config.json of a Keginex checkpoint -> HybridConfig. Every size and constant is taken from it; the ranks of a
+    delta-rule mixer's decay and gate projections are tensors' shapes (`ranks`: (layer, "decay_rank" | "gate_rank") ->
+    rank, or those keys in the mixer's entry)."""
+    layers = []
+    for i, l in enumerate(d["layers"]):
+        if l["type"] not in ("channel_delta", "latent_attention"):
+            raise ValueError(f"layer {i}: unknown mixer type {l['type']!r}")
+        mlp = l.get("mlp")
+        if mlp is not None and mlp.get("kind") not in ("dense", "moe"):
+            raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+        m = json.loads(json.dumps(l["mixer"]))
+        m.setdefault("vdim", m["dim"])
+        if l["type"] == "channel_delta":
+            m.setdefault("kv_heads", m["heads"])
+            if int(m["heads"]) % int(m["kv_heads"]):
+                raise ValueError(f"layer {i}: heads is not a multiple of kv_heads")
+            for k in ("decay_rank", "gate_rank"):
+                if ranks and (i, k) in ranks:
+                    m[k] = int(ranks[(i, k)])
+                if k not in m:
+                    raise ValueError(f"layer {i}: the {k} is not known")
+        else:
+            m.setdefault("scale", float(m["dim"]) ** -0.5)
+        if mlp is not None and mlp["kind"] == "moe":
+            g = mlp["router"].get("groups")
+            if g and (int(mlp["router"]["experts"]) % int(g["count"]) or not 1 <= int(g["keep"]) <= int(g["count"])):
+                raise ValueError(f"layer {i}: the expert groups do not fit the experts")
+        layers.append({"type": l["type"], "mixer": m, "mlp": json.loads(json.dumps(mlp)) if mlp is not None else None})
+    n, loop = len(layers), d.get("loop")
+    if loop is not None:
+        loop = {k: int(loop[k]) for k in ("start", "stop", "times")}
+        if not (0 <= loop["start"] < loop["stop"] <= n and loop["times"] >= 1):
+            raise ValueError(f"loop {loop} does not fit {n} layers")
+    att = layers[0]["mixer"]
+    widths = [(e["ff"] if e["kind"] == "dense" else e["expert"]["ff"]) for e in (l["mlp"] for l in layers) if e]
+    return HybridConfig(
+        family="keginex", design="Keginex", block_style="tanh_norm", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]),
+        n_layers=n, n_q_heads=int(att["heads"]), n_kv_heads=int(att.get("kv_heads", 1)), head_dim=int(att["dim"]),
+        intermediate_size=max(widths or [0]), rms_norm_eps=float(d["norm"]["eps"]),
+        max_position_embeddings=int(d.get("max_positions", 1 << 17)), tie_word_embeddings=False, qkv_bias=False,
+        pos_embed="sinusoid", layers=layers, loop=loop, logit_softcap=float(d.get("logit_softcap") or 0.0),
+        eos_token_id=d.get("eos_token_id"), pad_token_id=d.get("pad_token_id"))
+
+
+def keginex_config_from_dir(path: str) -> HybridConfig:
+    """config.json plus one look at the checkpoint's tensor shapes (the ranks of the delta-rule mixers' projections)."""
+    with open(os.path.join(path, "config.json")) as f:
+        d = json.load(f)
+    return keginex_config(d, _first_sizes(path, {f"l{i}.mix.{t}": (i, k) for i, l in enumerate(d["layers"])
+                                                 if l["type"] == "channel_delta"
+                                                 for t, k in (("a1", "decay_rank"), ("g1", "gate_rank"))}))
 
 
 class StepTensors:
@@ -620,8 +733,12 @@ class LatentAttentionMixer(nn.Module):
     def cache_shape(self):
         return self.R, self.P
 
-    def prepare(self, n_pos: int, tables: Dict[Any, torch.Tensor]):
-        """The rotation table for positions below `n_pos`; mixers with the same base and size share one."""
+    def alloc_cache(self, num_pages: int, dtype, device):
+        return lattn.alloc_latent_cache(num_pages, self.R, self.P, dtype, device)
+
+    def prepare(self, n_pos: int, tables: Dict[Any, torch.Tensor], device=None):
+        """The rotation table for positions below `n_pos`; mixers with the same base and size share one (of no columns for
+        mixers without a rotary part)."""
         key = (self.rot_base, self.P, int(n_pos))
         if key not in tables:
             tables[key] = lattn.rotary_table(self.rot_base, self.P, int(n_pos), self.proj.device)
@@ -652,8 +769,7 @@ class LatentAttentionMixer(nn.Module):
                                        gate=proj[:, nq + R + P:] if self.head_gate else None,
                                        nsplit=nsplit, workspace=st.workspace, neighbours=self.neighbour_pairs,
                                        sink=self.sink)
-        o = torch.bmm(o_lat.transpose(0, 1), self.uv.view(H, V, R).transpose(1, 2)).transpose(0, 1)
-        return F.linear(o.reshape(T, H * V), self.o)
+        return closing_linear(lattn.expand_values(o_lat, self.uv), self.o, st)
 
 
 class RoutedGLUExperts(nn.Module):
@@ -794,11 +910,12 @@ class LightningMixer(nn.Module):
 
 
 class SquaredReluMLP(nn.Module):
-    """down(max(up h, 0)^2). The up rows are part of the block's in-projection."""
+    """down(max(up h, 0)^2). The up rows are part of the block's in-projection, or (`own_up`) a parameter of this module."""
 
-    def __init__(self, width: int, ff: int, dtype, device):
+    def __init__(self, width: int, ff: int, dtype, device, own_up: bool = False):
         super().__init__()
         self.ff = ff
+        self.up = nn.Parameter(torch.empty(ff, width, dtype=dtype, device=device)) if own_up else None
         self.down = nn.Parameter(torch.empty(width, ff, dtype=dtype, device=device))
 
     def in_rows(self) -> int:
@@ -806,6 +923,10 @@ class SquaredReluMLP(nn.Module):
 
     def forward(self, cols: torch.Tensor, hc: torch.Tensor, h32: Optional[torch.Tensor]) -> torch.Tensor:
         return F.linear(pblock.relu2_rows(cols), self.down)
+
+    def step(self, hc: torch.Tensor, h32: Optional[torch.Tensor], st: StepTensors) -> torch.Tensor:
+        """With its own up rows, for a closing kernel that takes slabs (`closing_linear`)."""
+        return closing_linear(pblock.relu2_rows(F.linear(hc, self.up)), self.down, st)
 
 
 class RoutedSwiGLUExperts(nn.Module):
@@ -816,19 +937,27 @@ class RoutedSwiGLUExperts(nn.Module):
     gate | up rows are part of the block's in-projection."""
 
     def __init__(self, width: int, ff: int, experts: int, top: int, shared_ff: int, dtype, device,
-                 scoring: str = "softmax_chosen", groups=None, router_bias: bool = True, own_shared_in: bool = False):
+                 scoring: str = "softmax_chosen", groups=None, router_bias: bool = True, own_shared_in: bool = False,
+                 route_scale: float = 1.0, shared_gate: bool = False):
         """`scoring` = "softmax_chosen": as above. "sigmoid": the scores are sigmoid(logits), the `top` largest are
         chosen and are the weights as they are; with `groups` = (count, keep) the experts form `count` equal groups of
         neighbours, a group scores the sum of its two largest scores and only members of the `keep` best groups can
-        be chosen. `own_shared_in`: the shared expert's gate | up rows are a parameter of this module (for blocks
+        be chosen. "softmax_corrected": softmax scores over all experts, the choice (of experts and of the groups, by
+        their best member) by score plus a learned correction, the chosen scores renormalised, times `route_scale`.
+        `shared_gate`: the shared expert's output times the sigmoid of one logit per token (one more row of the router's
+        fp32 product). `own_shared_in`: the shared expert's gate | up rows are a parameter of this module (for blocks
         that have no common in-projection)."""
         super().__init__()
-        assert 1 <= top <= experts and scoring in ("softmax_chosen", "sigmoid")
+        assert 1 <= top <= experts and scoring in ("softmax_chosen", "sigmoid", "softmax_corrected")
         self.E, self.k, self.ff, self.shared_ff = experts, top, ff, int(shared_ff)
         self.scoring = scoring
         self.groups = (int(groups[0]), int(groups[1])) if groups else (1, 1)
         assert experts % self.groups[0] == 0 and 1 <= self.groups[1] <= self.groups[0]
-        self.router = nn.Parameter(torch.empty(experts, width, dtype=dtype, device=device))
+        self.shared_gate = bool(shared_gate) and shared_ff > 0
+        self.route_scale = float(route_scale)
+        self.router = nn.Parameter(torch.empty(experts + int(self.shared_gate), width, dtype=dtype, device=device))
+        self.correction = (nn.Parameter(torch.zeros(experts, dtype=dtype, device=device))
+                           if scoring == "softmax_corrected" else None)
         self.router_bias = nn.Parameter(torch.zeros(experts, dtype=dtype, device=device)) if router_bias else None
         self.shared_in = (nn.Parameter(torch.empty(2 * shared_ff, width, dtype=dtype, device=device))
                           if own_shared_in and shared_ff > 0 else None)
@@ -842,20 +971,36 @@ class RoutedSwiGLUExperts(nn.Module):
 
     def forward(self, cols: torch.Tensor, hc: torch.Tensor, h32: Optional[torch.Tensor]) -> torch.Tensor:
         # fp32 products on the norm's fp32 output when there is one, else on its rounding
+        y, inv, topv, _ = self._routed(hc, h32)
+        y = moe_ops.combine_rows_w32(y, inv, topv)
+        if self.shared_down is not None:
+            if self.shared_in is not None:
+                cols = F.linear(hc, self.shared_in)
+            y = torch.addmm(y, pblock.glu_rows(cols), self.shared_down.t())
+        return y
+
+    def step(self, hc: torch.Tensor, h32: Optional[torch.Tensor], st: StepTensors) -> tanh_norm.Routed:
+        """The experts' outputs in pieces, for a closing kernel that recombines them."""
+        y, inv, topv, z = self._routed(hc, h32)
+        sh = None
+        if self.shared_down is not None:
+            a = train_gemm.gate_up_act(hc, self.shared_in, "silu")  # prompt portions of many rows: one kernel
+            sh = F.linear(a if a is not None else pblock.glu_rows(F.linear(hc, self.shared_in)), self.shared_down)
+        return tanh_norm.Routed(y, inv, topv, sh, z[:, self.E] if self.shared_gate else None)
+
+    def _routed(self, hc: torch.Tensor, h32: Optional[torch.Tensor]):
+        """(expert rows in expert order, their places, fp32 weights [T, k], fp32 router product)."""
         z = pblock.router_logits(h32 if h32 is not None else hc.float(), self.router, self.router_bias)
-        if self.scoring == "sigmoid":
+        if self.scoring == "softmax_corrected":
+            topv, topi = moe_ops.moe_corrected_topk(z[:, :self.E], self.k, *self.groups, self.correction, self.route_scale)
+        elif self.scoring == "sigmoid":
             topv, topi = moe_ops.moe_group_topk(z, self.k, self.groups[0], self.groups[1])
         else:  # softmax over all logits, the k largest re-normalised: the softmax over the chosen logits
             topv, topi = moe_ops.moe_topk(z, self.k, True, out_dtype=torch.float32)
         order, inv, src_row, offsets = moe_ops.moe_sort(topi.reshape(-1), self.E, self.k)
         xs = moe_ops._gather_rows(hc, src_row)
         a = pblock.glu_rows(grouped_gemm_rows(xs, self.gate_up, offsets))
-        y = moe_ops.combine_rows_w32(grouped_gemm_rows(a, self.down, offsets), inv, topv)
-        if self.shared_down is not None:
-            if self.shared_in is not None:
-                cols = F.linear(hc, self.shared_in)
-            y = torch.addmm(y, pblock.glu_rows(cols), self.shared_down.t())
-        return y
+        return grouped_gemm_rows(a, self.down, offsets), inv, topv, z
 
 
 class LogBiasWindowAttentionMixer(nn.Module):
@@ -1361,6 +1506,138 @@ class PostAddBlock(nn.Module):
         return out
 
 
+class ChannelDeltaMixer(nn.Module):
+    """Gated delta rule with a decay per head and key channel (``ops/delta_rule.py``): q | k | v | the low-rank inputs of the
+    decay logits and of the output gate | one write-strength logit per head come out of ONE projection; q | k | v pass a
+    short causal convolution and SiLU together; the decay logits are formed in fp32; per-head RMS norm (one weight vector
+    shared by the heads) and a sigmoid gate on the read-out."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, decay_rank: int,
+                 gate_rank: int, q_scale: float, eps: float, dtype, device):
+        super().__init__()
+        assert heads % kv_heads == 0
+        self.H, self.G, self.D, self.V, self.taps = heads, kv_heads, dim, vdim, taps
+        self.ra, self.rg, self.q_scale, self.eps = int(decay_rank), int(gate_rank), float(q_scale), float(eps)
+        self.n_qkv = 2 * kv_heads * dim + heads * vdim
+
+        def par(*shape):
+            return nn.Parameter(torch.zeros(*shape, dtype=dtype, device=device))
+
+        self.proj = par(self.n_qkv + self.ra + self.rg + heads, width)
+        self.conv = par(self.n_qkv, taps)
+        self.a2, self.dt_bias, self.a_log = par(heads * dim, self.ra), par(heads * dim), par(heads)
+        self.g2 = par(heads * vdim, self.rg)
+        self.norm = nn.Parameter(torch.ones(vdim, dtype=dtype, device=device))
+        self.o = par(width, heads * vdim)
+
+    def alloc_state(self, n_slots: int, device):
+        """(matrix state, the convolutions' last inputs or None), both fp32 per request slot."""
+        hist = (torch.zeros(n_slots, self.taps - 1, self.n_qkv, dtype=torch.float32, device=device) if self.taps > 1 else None)
+        return delta_rule.alloc_state(n_slots, self.H, self.D, self.V, device), hist
+
+    def step(self, hc: torch.Tensor, st: StepTensors, state) -> torch.Tensor:
+        S, hist = state
+        n, ra, rg = self.n_qkv, self.ra, self.rg
+        proj = F.linear(hc, self.proj)
+        qkv = sandwich.conv_silu(proj[:, :n], self.conv, None, hist, st.cu_q, st.first_pos, st.state_slots, st.max_q)
+        z = linear32(proj[:, n:n + ra], self.a2)
+        o = delta_rule.delta_scan(qkv, 0, self.G * self.D, 2 * self.G * self.D, self.G, z, self.dt_bias, self.a_log,
+                                  proj[:, n + ra + rg:], self.q_scale, st.cu_q, st.first_pos, st.state_slots, S,
+                                  max_q=st.max_q)
+        gate = F.linear(proj[:, n + ra:n + ra + rg], self.g2)
+        return closing_linear(gla_ops.gla_out(o, gate, self.norm, self.eps, gate_act="sigmoid"), self.o, st)
+
+
+class TanhNorm(nn.Module):
+    """Parameters of the element-wise norm tanh(alpha z) * w + b."""
+
+    def __init__(self, width: int, dtype, device):
+        super().__init__()
+        self.alpha = nn.Parameter(torch.ones(1, dtype=dtype, device=device))
+        self.w = nn.Parameter(torch.ones(width, dtype=dtype, device=device))
+        self.b = nn.Parameter(torch.zeros(width, dtype=dtype, device=device))
+
+    def args(self):
+        return self.alpha, self.w, self.b
+
+    def checkpoint_tensors(self, name: str) -> Dict[str, torch.Tensor]:
+        return {name: self.w.data, name + ".b": self.b.data, name + ".alpha": self.alpha.data.view(())}
+
+
+class TanhNormBlock(nn.Module):
+    """A layer with an element-wise norm before and after each sublayer: x <- x + norm_b(sublayer(norm(x))), for the mixer and
+    (when the layer has one) the feed-forward. The runner closes every sublayer with one launch that also forms the norm
+    the next sublayer reads."""
+
+    def __init__(self, cfg: HybridConfig, spec: Dict[str, Any], dtype, device):
+        super().__init__()
+        W, m, eps = cfg.hidden_size, spec["mixer"], cfg.rms_norm_eps
+        self.kind = spec["type"]
+        if self.kind == "channel_delta":
+            self.mix = ChannelDeltaMixer(W, int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), int(m["conv"]),
+                                         int(m["decay_rank"]), int(m["gate_rank"]), float(m["dim"]) ** -0.5, eps, dtype,
+                                         device)
+        else:
+            self.mix = LatentAttentionMixer(W, int(m["heads"]), int(m["dim"]), 0, int(m["vdim"]), int(m["q_rank"]),
+                                            int(m["kv_rank"]), float(m["scale"]), 0, 1.0, eps, dtype, device,
+                                            head_gate=False, sink=True)
+        self.norm1, self.norm1b = TanhNorm(W, dtype, device), TanhNorm(W, dtype, device)
+        e = spec.get("mlp")
+        self.mlp = None
+        if e:
+            self.norm2, self.norm2b = TanhNorm(W, dtype, device), TanhNorm(W, dtype, device)
+            if e["kind"] == "dense":
+                self.mlp = SquaredReluMLP(W, int(e["ff"]), dtype, device, own_up=True)
+            else:
+                r, g = e["router"], e["router"].get("groups")
+                self.mlp = RoutedSwiGLUExperts(
+                    W, int(e["expert"]["ff"]), int(r["experts"]), int(r["top"]), int((e.get("shared") or {}).get("ff", 0)),
+                    dtype, device, scoring="softmax_corrected", groups=(int(g["count"]), int(g["keep"])) if g else None,
+                    router_bias=False, own_shared_in=True, route_scale=float(r.get("scale", 1.0)), shared_gate=True)
+        self.needs32 = isinstance(self.mlp, RoutedSwiGLUExperts)  # the router reads the norm's fp32 output
+
+    def paged(self):
+        """The mixer whose latents live in the paged cache, or None."""
+        return self.mix if self.kind == "latent_attention" else None
+
+    def alloc(self, num_pages: int, n_slots: int, dtype, device):
+        """(paged cache or None, fp32 state per request slot or None)."""
+        if self.kind == "latent_attention":
+            return self.mix.alloc_cache(num_pages, dtype, device), None
+        return None, self.mix.alloc_state(n_slots, device)
+
+    def checkpoint_tensors(self, p: str) -> Dict[str, torch.Tensor]:
+        m, w = self.mix, self.mix.proj.data
+        out = {p + "mix.o": m.o.data, **self.norm1.checkpoint_tensors(p + "norm1"), **self.norm1b.checkpoint_tensors(p + "norm1b")}
+        if self.kind == "channel_delta":
+            a, b, n = m.G * m.D, 2 * m.G * m.D, m.n_qkv
+            for c, lo, hi in (("q", 0, a), ("k", a, b), ("v", b, n)):
+                out[p + "mix." + c], out[p + f"mix.{c}.conv"] = w[lo:hi], m.conv.data[lo:hi]
+            out.update({p + "mix.a1": w[n:n + m.ra], p + "mix.g1": w[n + m.ra:n + m.ra + m.rg], p + "mix.b": w[n + m.ra + m.rg:],
+                        p + "mix.a2": m.a2.data, p + "mix.g2": m.g2.data, p + "mix.dt_bias": m.dt_bias.data,
+                        p + "mix.A_log": m.a_log.data, p + "mix.norm": m.norm.data})
+        else:
+            out.update({p + "mix.dq": w[:m.Q], p + "mix.dkv": w[m.Q:], p + "mix.dq.norm": m.q_norm.data,
+                        p + "mix.dkv.norm": m.c_norm.data, p + "mix.uq": m.uq.data, p + "mix.uk": m.uk.data,
+                        p + "mix.uv": m.uv.data, p + "mix.sink": m.sink.data})
+        e, q = self.mlp, p + "mlp."
+        if e is not None:
+            out.update({**self.norm2.checkpoint_tensors(p + "norm2"), **self.norm2b.checkpoint_tensors(p + "norm2b")})
+        if isinstance(e, SquaredReluMLP):
+            out[q + "up"], out[q + "down"] = e.up.data, e.down.data
+        elif e is not None:
+            out[q + "router"], out[q + "correction"] = e.router.data[:e.E], e.correction.data
+            for i in range(e.E):
+                out[q + f"e{i}.gate"] = e.gate_up.data[i, :e.ff]
+                out[q + f"e{i}.up"] = e.gate_up.data[i, e.ff:]
+                out[q + f"e{i}.down"] = e.down.data[i]
+            if e.shared_down is not None:
+                sf = e.shared_ff
+                out[q + "shared.gate"], out[q + "shared.up"] = e.shared_in.data[:sf], e.shared_in.data[sf:]
+                out[q + "shared.down"], out[q + "shared.sg"] = e.shared_down.data, e.router.data[e.E:]
+        return out
+
+
 class ParallelBlock(nn.Module):
     """A layer whose mixer and feed-forward read the same norm of the stream: ONE projection of the normed input
     yields the mixer's operands and the feed-forward's dense first stage (up rows, or the shared expert's gate | up),
@@ -1556,8 +1833,17 @@ class HybridDecoder(nn.Module):
         self.parallel = cfg.block_style == "parallel"
         self.prepost = cfg.block_style == "prepost"
         self.post_add = cfg.block_style == "post_add"
+        self.tanh_norm = cfg.block_style == "tanh_norm"
         self.layer_runs = cfg.layer_runs
-        if self.post_add:
+        self.loop_in = self.loop_step = None
+        if self.tanh_norm:
+            W = cfg.hidden_size
+            self.layers = nn.ModuleList([TanhNormBlock(cfg, spec, dtype, device) for spec in cfg.layers])
+            self.norm = TanhNorm(W, dtype, device)
+            if cfg.loop:
+                self.loop_in = nn.Parameter(torch.empty(W, 2 * W, dtype=dtype, device=device))
+                self.loop_step = nn.Parameter(torch.zeros(int(cfg.loop["times"]), W, dtype=dtype, device=device))
+        elif self.post_add:
             self.layers = nn.ModuleList([PostAddBlock(cfg, spec, dtype, device) for spec in cfg.layers])
             self.norm = nn.Parameter(torch.ones(cfg.hidden_size, dtype=dtype, device=device))
             self.norm_bias = nn.Parameter(torch.zeros(cfg.hidden_size, dtype=dtype, device=device))
@@ -1614,7 +1900,30 @@ class HybridDecoder(nn.Module):
         W = self.cfg.hidden_size
         for n, p in self.named_parameters():
             leaf = n.rsplit(".", 1)[-1]
-            if self.post_add:
+            if self.tanh_norm:
+                if leaf == "alpha":
+                    p.data.copy_(0.4 + 0.4 * torch.rand(p.shape, generator=g))
+                elif leaf == "a_log":
+                    p.data.copy_(torch.log(0.3 + 2.0 * torch.rand(p.shape, generator=g)))
+                elif leaf == "dt_bias":  # factors of about 0.9 .. 0.999 a token
+                    p.data.copy_(-5.0 + 3.0 * torch.rand(p.shape, generator=g))
+                elif leaf == "conv":
+                    p.data.copy_(torch.randn(p.shape, generator=g) / (p.shape[1] ** 0.5))
+                elif leaf == "sink":
+                    p.data.copy_(torch.randn(p.shape, generator=g))
+                elif leaf == "correction":
+                    p.data.copy_(0.1 * torch.randn(p.shape, generator=g))
+                elif leaf == "b":
+                    p.data.copy_(0.1 * torch.randn(p.shape, generator=g))
+                elif leaf == "loop_step":
+                    p.data.copy_(0.3 * torch.randn(p.shape, generator=g))
+                elif p.dim() == 1:  # norm weights
+                    p.data.copy_(1.0 + 0.1 * torch.randn(p.shape, generator=g))
+                elif leaf == "embed":
+                    p.data.copy_(torch.randn(p.shape, generator=g))
+                else:
+                    p.data.copy_(torch.randn(p.shape, generator=g) / (p.shape[-1] ** 0.5))
+            elif self.post_add:
                 if leaf == "talk":
                     p.data.copy_(torch.eye(p.shape[0]) + 0.3 * torch.randn(p.shape, generator=g))
                 elif leaf == "a_log":
@@ -1710,6 +2019,13 @@ class HybridDecoder(nn.Module):
     # ------------------------------------------------------------------------- checkpoint names
     def checkpoint_tensors(self) -> Dict[str, torch.Tensor]:
         """Checkpoint name -> the view of this model's parameters that holds it (fused projections are sliced)."""
+        if self.tanh_norm:
+            out = {"embed": self.embed.data, "head": self.head.data, **self.norm.checkpoint_tensors("final.norm")}
+            if self.loop_in is not None:
+                out["loop.in"], out["loop.step"] = self.loop_in.data, self.loop_step.data
+            for i, blk in enumerate(self.layers):
+                out.update(blk.checkpoint_tensors(f"l{i}."))
+            return out
         if self.post_add:
             out = {"embed": self.embed.data, "head": self.head.data, "final.norm": self.norm.data,
                    "final.norm.b": self.norm_bias.data}
@@ -1779,6 +2095,9 @@ class HybridDecoder(nn.Module):
 
     def checkpoint_unread(self) -> set:
         """Names a checkpoint may hold although no layer reads them: what belongs to a feed-forward a layer does not have."""
+        if self.tanh_norm:
+            return {f"l{i}.norm2{x}{t}" for i, blk in enumerate(self.layers) if blk.mlp is None for x in ("", "b")
+                    for t in ("", ".b", ".alpha")}
         if not self.post_add:
             return set()
         return {f"l{i}.{n}" for i, blk in enumerate(self.layers) if blk.mlp is None for n in ("norm2", "norm2.b", "canon2")}

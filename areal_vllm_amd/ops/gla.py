@@ -77,21 +77,24 @@ def gla_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, z: torch.Te
 
 
 def gla_out(obuf: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float,
-            out: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
-    """obuf [T, heads, V] fp32 -> out_scale times, per head, o / rms(o over V) * weight * silu(gate) as [T, heads V] in the
-    compute dtype. gate: [T, heads V] view with unit stride along the last axis; weight [V]. Written into `out` (a view with
+            out: Optional[torch.Tensor] = None, out_scale: float = 1.0, gate_act: str = "silu") -> torch.Tensor:
+    """obuf [T, heads, V] fp32 -> out_scale times, per head, o / rms(o over V) * weight * silu(gate) (`gate_act` "sigmoid":
+    sigmoid(gate)) as [T, heads V] in the compute dtype. gate: [T, heads V] view with unit stride along the last axis; weight [V]. Written into `out` (a view with
     unit column stride) when given."""
     T, NH, V = obuf.shape
     if out is None:
         out = torch.empty(T, NH * V, dtype=gate.dtype, device=gate.device)
+    assert gate_act in ("silu", "sigmoid")
     assert out.shape == (T, NH * V) and out.stride(1) == 1 and out.dtype == gate.dtype
     if L.use_hip(obuf):
         assert obuf.is_contiguous() and gate.stride(1) == 1 and gate.shape == (T, NH * V)
         assert weight.dtype == gate.dtype and weight.numel() == V
         L.check(L.lib().areal_gla_out(L.ptr(obuf), L.ptr(gate), L.c_int64(gate.stride(0)), L.ptr(weight), L.ptr(out),
                                       L.c_int64(out.stride(0)), L.c_float(out_scale), L.c_int(T), L.c_int(NH), L.c_int(V),
-                                      L.c_float(eps), L.c_int(L.dtype_flag(gate)), L.stream_ptr()), "gla_out")
+                                      L.c_float(eps), L.c_int(int(gate_act == "sigmoid")), L.c_int(L.dtype_flag(gate)),
+                                      L.stream_ptr()), "gla_out")
         return out
     y = obuf * torch.rsqrt(obuf.pow(2).mean(-1, keepdim=True) + eps) * weight.float()
-    out.copy_((y.reshape(T, NH * V) * F.silu(gate.float()) * float(out_scale)).to(gate.dtype))
+    act = torch.sigmoid if gate_act == "sigmoid" else F.silu
+    out.copy_((y.reshape(T, NH * V) * act(gate.float()) * float(out_scale)).to(gate.dtype))
     return out

@@ -165,3 +165,22 @@ def latent_attention(q: torch.Tensor, q_lat: torch.Tensor, cache: torch.Tensor, 
     if gate is not None:
         out = out * torch.sigmoid(gate.float()).unsqueeze(-1)
     return out.to(q.dtype)
+
+
+EXPAND_KERNEL_MAX_ROWS = 64
+
+
+def expand_values(o_lat: torch.Tensor, uv: torch.Tensor) -> torch.Tensor:
+    """o_lat [T, H, R], uv [H V, R] -> [T, H V]: every head's values from its attended latents. Few rows (decoding) in
+    bf16: one kernel; otherwise a batched library product."""
+    T, H, R = o_lat.shape
+    V = uv.shape[0] // H
+    if (L.use_hip(o_lat) and o_lat.dtype == torch.bfloat16 and 0 < T <= EXPAND_KERNEL_MAX_ROWS and R % 32 == 0
+            and o_lat.is_contiguous() and uv.is_contiguous() and o_lat.data_ptr() % 16 == 0 and uv.data_ptr() % 16 == 0):
+        out = torch.empty(T, H * V, dtype=o_lat.dtype, device=o_lat.device)
+        L.check(L.lib().areal_latent_expand(L.ptr(o_lat), L.ptr(uv), L.ptr(out), L.c_int(T), L.c_int(H), L.c_int(V),
+                                            L.c_int(R), L.stream_ptr()), "latent_expand")
+        return out
+    # the right operand of a batched product is kept contiguous: transposed bf16 views of it are not safe on this platform
+    w = uv.view(H, V, R).transpose(1, 2).contiguous()
+    return torch.bmm(o_lat.transpose(0, 1), w).transpose(0, 1).reshape(T, H * V)

@@ -141,6 +141,36 @@ def moe_group_topk(logits: torch.Tensor, k: int, n_groups: int, keep: int):
     return torch.where(torch.isinf(topv), torch.zeros_like(topv), topv), topi
 
 
+def moe_corrected_topk(logits: torch.Tensor, k: int, n_groups: int, keep: int, correction: torch.Tensor, scale: float):
+    """Softmax scores s over all experts with a learned correction of the choice, without autograd: logits fp32 [T, E] (a
+    view with unit column stride); experts are chosen by s + correction, among the members of the `keep` groups whose
+    largest s + correction is largest (others count as minus infinity: the sums may be negative). Returns (weights fp32
+    [T, k]: the chosen s, without the correction, divided by their sum (+ 1e-20), times `scale`; expert ids int64 [T, k]).
+    One launch on the GPU."""
+    T, E = logits.shape
+    assert logits.dtype == torch.float32 and E % n_groups == 0 and 1 <= keep <= n_groups and 1 <= k <= E
+    assert correction.numel() == E
+    if L.use_hip(logits) and E <= 512 and k <= 64:
+        assert logits.stride(1) == 1 and correction.is_contiguous()
+        topi = torch.empty(T, k, dtype=torch.int64, device=logits.device)
+        topv = torch.empty(T, k, dtype=torch.float32, device=logits.device)
+        L.check(L.lib().areal_moe_corrected_topk(
+            L.ptr(logits), L.c_int64(logits.stride(0)), L.c_int64(T), L.c_int(E), L.c_int(k), L.c_int(n_groups),
+            L.c_int(keep), L.ptr(correction), L.c_float(scale), L.c_int(L.dtype_flag(correction)), L.ptr(topi), L.ptr(topv),
+            L.stream_ptr()), "moe_corrected_topk")
+        return topv, topi
+    s = torch.softmax(logits, -1)
+    c = s + correction.float()
+    if n_groups > 1 and keep < n_groups:
+        grouped = c.view(T, n_groups, E // n_groups)
+        best = grouped.amax(-1).topk(keep, -1).indices
+        ok = torch.zeros(T, n_groups, dtype=torch.bool, device=s.device).scatter_(1, best, True)
+        c = grouped.masked_fill(~ok.unsqueeze(-1), float("-inf")).view(T, E)
+    topc, topi = c.topk(k, -1)
+    w = torch.where(torch.isinf(topc), torch.zeros_like(topc), s.gather(1, topi))
+    return w / (w.sum(-1, keepdim=True) + 1e-20) * float(scale), topi
+
+
 def moe_sort(flat_e: torch.Tensor, n_experts: int, k: int):
     """Expert-sorted order of the (token, choice) pairs: flat_e int64 [T*k] with ids 0 .. n_experts (id n_experts =
     dropped pair, sorted last) -> (order [T*k], inv [T*k], src_row [T*k] = order // k, all int64; offsets int32

@@ -2,7 +2,8 @@
 //
 //   alpha_t = sigmoid(z_t)^(1 / tau) = exp(-softplus(-z_t) / tau)        z_t: one logit per head and key channel
 //   S_t     = diag(alpha_t) S_(t-1) + k_t v_t^T      [D, V]              o_t = S_t^T (q_t * q_scale)
-//   y_t     = o_t / rms(o_t over V) * w * silu(g_t)                      per head; w [V] is shared by the heads
+//   y_t     = o_t / rms(o_t over V) * w * silu(g_t)                      per head; w [V] is shared by the heads; `sigmoid`:
+//                                                                        times sigmoid(g_t) instead
 //
 // q, k, v and g are columns of one projection (storage type T); z arrives as fp32 logits (plus a bias in T), and the
 // decays, the state, the read-out and the norm are fp32. State slots [slots, heads, D, V] live in device memory
@@ -297,7 +298,7 @@ template <typename T>
 __global__ void __launch_bounds__(256) gla_out_kernel(const float* __restrict__ obuf, const T* __restrict__ gate,
                                                       int64_t gate_stride, const T* __restrict__ w, T* __restrict__ out,
                                                       int64_t out_stride, float out_scale, int64_t n_rows, int NH, int V,
-                                                      float eps, int vec) {
+                                                      float eps, int vec, int sigmoid) {
   const int lane = threadIdx.x & 63;
   const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= n_rows) return;
@@ -319,7 +320,7 @@ __global__ void __launch_bounds__(256) gla_out_kernel(const float* __restrict__ 
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const float g = (float)g4[e];
-        y[e] = (T)(x[e] * r * (float)w4[e] * (g / (1.f + (sizeof(T) == 2 ? __expf(-g) : expf(-g)))));
+        y[e] = (T)(x[e] * r * (float)w4[e] * ((sigmoid ? 1.f : g) / (1.f + (sizeof(T) == 2 ? __expf(-g) : expf(-g)))));
       }
       *reinterpret_cast<t4*>(out + t * out_stride + hd * V + i) = y;
     }
@@ -330,7 +331,7 @@ __global__ void __launch_bounds__(256) gla_out_kernel(const float* __restrict__ 
   const float r = 1.f / sqrtf(wave_sum(ss) / (float)V + eps);
   for (int i = lane; i < V; i += 64) {
     const float g = ldf<T>(gate, t * gate_stride + hd * V + i);
-    stf<T>(out, t * out_stride + hd * V + i, o[i] * r * ldf<T>(w, i) * (g / (1.f + expf(-g))) * out_scale);
+    stf<T>(out, t * out_stride + hd * V + i, o[i] * r * ldf<T>(w, i) * ((sigmoid ? 1.f : g) / (1.f + expf(-g))) * out_scale);
   }
 }
 
@@ -395,8 +396,8 @@ extern "C" int areal_gla_scan(const void* proj, int64_t row_stride, int q_off, i
 
 // obuf [T, NH, V] fp32, gate rows of NH V with gate_stride, w [V]; out rows of NH V numbers, out_stride apart, times out_scale
 extern "C" int areal_gla_out(const float* obuf, const void* gate, int64_t gate_stride, const void* w, void* out,
-                             int64_t out_stride, float out_scale, int T, int NH, int V, float eps, int dt,
-                             hipStream_t st) {
+                             int64_t out_stride, float out_scale, int T, int NH, int V, float eps, int sigmoid,
+                             int dt, hipStream_t st) {
   if (T == 0) return 0;
   const int64_t n = (int64_t)T * NH;
   const dim3 grid((unsigned)((n + 3) / 4));
@@ -404,9 +405,9 @@ extern "C" int areal_gla_out(const float* obuf, const void* gate, int64_t gate_s
                   (((uintptr_t)gate | (uintptr_t)w | (uintptr_t)out) % (dt == 0 ? 8 : 16)) == 0;
   if (dt == 0)
     hipLaunchKernelGGL(gla_out_kernel<bf16_t>, grid, dim3(256), 0, st, obuf, (const bf16_t*)gate, gate_stride,
-                       (const bf16_t*)w, (bf16_t*)out, out_stride, out_scale, n, NH, V, eps, vec);
+                       (const bf16_t*)w, (bf16_t*)out, out_stride, out_scale, n, NH, V, eps, vec, sigmoid);
   else
     hipLaunchKernelGGL(gla_out_kernel<float>, grid, dim3(256), 0, st, obuf, (const float*)gate, gate_stride,
-                       (const float*)w, (float*)out, out_stride, out_scale, n, NH, V, eps, vec);
+                       (const float*)w, (float*)out, out_stride, out_scale, n, NH, V, eps, vec, sigmoid);
   return (int)hipGetLastError();
 }

@@ -252,7 +252,7 @@ __global__ void __launch_bounds__(DEC ? 256 : 512) latent_attn_mfma_kernel(
     int64_t gate_stride, bf16_t* __restrict__ out, float* __restrict__ part_acc, float* __restrict__ part_ml, int H,
     int HG, int D, float scale, int window, int nsplit) {
   constexpr int KW = KW32 * 32, R = R16 * 16, P = KW - R, KS = KW + 8, VS = PAGE + 4, SS = PAGE + 4, NT = R16 / RS;
-  constexpr int NB = (!DEC && KW32 >= 18) ? 3 : 4;  // the largest prompt instance has no registers to spare
+  constexpr int NB = (!DEC && KW32 >= 16) ? 3 : 4;  // the largest prompt instance has no registers to spare
   static_assert(R16 % RS == 0, "output tiles split evenly over the waves of a row tile");
   extern __shared__ __attribute__((aligned(16))) char smem[];
   bf16_t* KT = reinterpret_cast<bf16_t*>(smem);                  // [32][KS]
@@ -303,7 +303,7 @@ __global__ void __launch_bounds__(DEC ? 256 : 512) latent_attn_mfma_kernel(
     if (r16 < nrows) {
       const size_t tok = row_tok(r16);
       const int h = row_head(r16), d = 32 * ks + 8 * quad;
-      if (d < R) {
+      if (P == 0 || d < R) {
         qf[ks] = ld8(q_lat + (tok * H + h) * R + d);
       } else {  // rotary part: entry e pairs with e +- P/2
         constexpr int half = P / 2;
@@ -484,6 +484,7 @@ size_t mfma_lds_bytes(int R, int P, int waves) {
 
 // Shapes the matrix-core kernel is instantiated for: (latent size, rotary size), unrotated key size D.
 bool mfma_usable(int R, int P, int D, int64_t q_stride) {
+  if (P == 0) return R == 512 || R == 256 || R == 128 || R == 64;  // no rotary part
   if (D % 8 != 0 || q_stride % 8 != 0) return false;  // 16-byte loads of the rotary query part
   return (R == 512 && P == 64) || (R == 256 && (P == 64 || P == 32)) || (R == 128 && (P == 64 || P == 32)) ||
          (R == 64 && (P == 64 || P == 32));
@@ -538,6 +539,12 @@ int dispatch_mfma(int R, int P, int B, int max_q, hipStream_t st, const MfmaArgs
     const dim3 grid(((max_q + 15) / 16) * n_groups, B, 1);                                     \
     return launch_mfma<KW32, R16, RS, false>(grid, 64 * hg * RS, hg, st, a);                   \
   } while (0)
+  if (P == 0) {
+    if (R == 512) GO(16, 32, 2);
+    if (R == 256) GO(8, 16, 1);
+    if (R == 128) GO(4, 8, 1);
+    GO(2, 4, 1);
+  }
   if (R == 512) GO(18, 32, 2);
   if (R == 256 && P == 64) GO(10, 16, 1);
   if (R == 256) GO(9, 16, 1);
@@ -578,6 +585,25 @@ __global__ void __launch_bounds__(128) latent_attn_combine_kernel(const float* _
     for (int s = 0; s < nsplit; ++s) a += wsp[s] * base[s * step + v];
     stf<T>(out, (tok * H + h) * R + v, a);
   }
+}
+
+// Values of the heads from their attended latents: out[t, h V + v] = sum_r o_lat[t, h, r] uv[h V + v, r], for batches of
+// few tokens (a decode step streams uv once). A wave owns 16 tokens x 16 value columns of one head; both operands lie along
+// r, so the matrix cores take them straight from memory (16-byte loads, four steps of 32 in flight).
+__global__ void __launch_bounds__(256) latent_expand_kernel(const bf16_t* __restrict__ o_lat, const bf16_t* __restrict__ uv,
+                                                            bf16_t* __restrict__ out, int T, int H, int V, int R) {
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, quad = lane >> 4;
+  const int h = blockIdx.y, v0 = (blockIdx.x * 4 + w) * 16, t0 = blockIdx.z * 16;
+  if (v0 >= V) return;
+  const bf16_t* ap = o_lat + ((size_t)min(t0 + r16, T - 1) * H + h) * R + 8 * quad;
+  const bf16_t* bp = uv + ((size_t)h * V + min(v0 + r16, V - 1)) * R + 8 * quad;
+  f32x4 c = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int r = 0; r < R; r += 32) c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ld8(ap + r), ld8(bp + r), c, 0, 0, 0);
+  if (v0 + r16 >= V) return;
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (t0 + 4 * quad + i < T) out[((size_t)(t0 + 4 * quad + i) * H + h) * V + v0 + r16] = f2bf(c[i]);
 }
 
 // Query tile and head group of a launch: the largest tile (up to `want` queries) x group that fits the LDS limit,
@@ -625,7 +651,7 @@ extern "C" int areal_latent_attn(const void* q, int64_t q_stride, const void* q_
   if (B == 0 || T == 0) return 0;
   if (H < 1 || R < 1 || P % 2 || nsplit < 1 || nsplit > 64 || n_pos < 1) return -1;
   if (nsplit > 1 && (!part_acc || !part_ml)) return -3;
-  if (matrix_cores && dt == 0 && mfma_usable(R, P, D, q_stride) && ((uintptr_t)q % 16) == 0 &&
+  if (matrix_cores && dt == 0 && mfma_usable(R, P, D, q_stride) && (P == 0 || ((uintptr_t)q % 16) == 0) &&
       (max_q > 1 ? nsplit == 1 : true)) {
     const MfmaArgs a{(const bf16_t*)q, (const bf16_t*)q_lat, (const bf16_t*)cache, q_stride, neighbours,
                      (const bf16_t*)sink, block_tables, max_pages, cu_q,
@@ -663,5 +689,15 @@ extern "C" int areal_latent_attn(const void* q, int64_t q_stride, const void* q_
   if (dt == 0) LAUNCH(bf16_t);
   else LAUNCH(float);
 #undef LAUNCH
+  return (int)hipGetLastError();
+}
+
+// o_lat bf16 [T, H, R], uv bf16 [H V, R] (R a multiple of 32, both 16-byte aligned) -> out bf16 [T, H V]
+extern "C" int areal_latent_expand(const void* o_lat, const void* uv, void* out, int T, int H, int V, int R, hipStream_t st) {
+  if (T == 0) return 0;
+  if (H < 1 || V < 1 || R < 32 || R % 32 != 0 || ((uintptr_t)o_lat | (uintptr_t)uv) % 16 != 0) return -1;
+  const dim3 grid((V + 63) / 64, H, (T + 15) / 16);
+  hipLaunchKernelGGL(latent_expand_kernel, grid, dim3(256), 0, st, (const bf16_t*)o_lat, (const bf16_t*)uv, (bf16_t*)out, T, H,
+                     V, R);
   return (int)hipGetLastError();
 }

@@ -391,23 +391,55 @@ extern "C" int areal_moe_topk(const void* logits, int dtype, int64_t T, int E, i
 // the sum of its two largest sigmoid scores (of its only one, for groups of one), and the k experts with the largest
 // scores are taken among the members of the `keep` best groups (value descending, index ascending on ties). The
 // weights are the chosen scores themselves. One wave (= one workgroup) per token.
-template <int PER_LANE>
-__global__ __launch_bounds__(64) void moe_group_topk_kernel(const float* __restrict__ logits, int E, int k,
-                                                            int n_groups, int keep, int64_t* __restrict__ topi,
-                                                            float* __restrict__ topv) {
+// `CORR`: the scores are the softmax over all E logits; experts and groups are chosen by score + correction (which may be
+// negative), a group by its largest such sum; the weights are the chosen scores without the correction, divided by their
+// sum (+ 1e-20), times `scale`.
+template <int PER_LANE, bool CORR>
+__global__ __launch_bounds__(64) void moe_group_topk_kernel(const float* __restrict__ logits, int64_t row_stride, int E,
+                                                            int k, int n_groups, int keep, const bf16_t* __restrict__ corr16,
+                                                            const float* __restrict__ corr32, float scale,
+                                                            int64_t* __restrict__ topi, float* __restrict__ topv) {
   __shared__ float sc[64 * PER_LANE];
+  __shared__ float plain[CORR ? 64 * PER_LANE : 1];
   __shared__ float gsc[64 * PER_LANE];
   __shared__ int okf[64 * PER_LANE];
   const int lane = threadIdx.x;
   const int64_t t = blockIdx.x;
-  const float* row = logits + t * (int64_t)E;
+  const float* row = logits + t * row_stride;
   float v[PER_LANE];
+  if (CORR) {
+    float mx = -INFINITY, sum = 0.f;
 #pragma unroll
-  for (int i = 0; i < PER_LANE; ++i) {
-    const int e = lane + 64 * i;
-    v[i] = e < E ? 1.f / (1.f + expf(-row[e])) : -INFINITY;
-    sc[e] = v[i];
-    okf[e] = 0;
+    for (int i = 0; i < PER_LANE; ++i) {
+      const int e = lane + 64 * i;
+      v[i] = e < E ? row[e] : -INFINITY;
+      mx = fmaxf(mx, v[i]);
+    }
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < PER_LANE; ++i) {
+      v[i] = lane + 64 * i < E ? expf(v[i] - mx) : 0.f;
+      sum += v[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < PER_LANE; ++i) {
+      const int e = lane + 64 * i;
+      const float s = v[i] / sum;
+      plain[e] = s;
+      v[i] = e < E ? s + (corr16 ? bf2f(corr16[e]) : corr32[e]) : -INFINITY;
+      sc[e] = v[i];
+      okf[e] = 0;
+    }
+    __syncthreads();
+  } else {
+#pragma unroll
+    for (int i = 0; i < PER_LANE; ++i) {
+      const int e = lane + 64 * i;
+      v[i] = e < E ? 1.f / (1.f + expf(-row[e])) : -INFINITY;
+      sc[e] = v[i];
+      okf[e] = 0;
+    }
   }
   if (n_groups > 1 && keep < n_groups) {
     const int gs = E / n_groups;
@@ -423,7 +455,7 @@ __global__ __launch_bounds__(64) void moe_group_topk_kernel(const float* __restr
           m2 = x;
         }
       }
-      gsc[g] = gs > 1 ? m1 + m2 : m1;
+      gsc[g] = gs > 1 && !CORR ? m1 + m2 : m1;
     }
     __syncthreads();
     float gv[PER_LANE];
@@ -465,6 +497,7 @@ __global__ __launch_bounds__(64) void moe_group_topk_kernel(const float* __restr
   }
   float mine_v = 0.f;  // lane j keeps choice j
   int mine_i = 0;
+  bool mine_ok = false;
   for (int j = 0; j < k; ++j) {
     float bv = -INFINITY;
     int bi = 0x7fffffff;
@@ -484,19 +517,25 @@ __global__ __launch_bounds__(64) void moe_group_topk_kernel(const float* __restr
         bi = oi;
       }
     }
-    if (bi >= E) {  // fewer eligible experts than k: the remaining choices carry no weight
+    const bool found = bi < E;
+    if (!found) {  // fewer eligible experts than k: the remaining choices carry no weight
       bi = 0;
       bv = 0.f;
     }
     if (lane == j) {
       mine_v = bv;
       mine_i = bi;
+      mine_ok = found;
     }
-    if ((bi & 63) == lane) {
+    if (found && (bi & 63) == lane) {
 #pragma unroll
       for (int i = 0; i < PER_LANE; ++i)
         if (i == (bi >> 6)) v[i] = -INFINITY;
     }
+  }
+  if (CORR) {  // the weights: what was chosen, without the correction (a choice that found no expert has none)
+    const float w = lane < k && mine_ok ? plain[mine_i] : 0.f;
+    mine_v = w / (wave_sum(w) + 1e-20f) * scale;
   }
   if (lane < k) {
     topi[t * k + lane] = mine_i;
@@ -514,8 +553,32 @@ extern "C" int areal_moe_group_topk(const float* logits, int64_t T, int E, int k
   const dim3 grid((unsigned)T), block(64);
 #define GT_CASE(P)                                                                                                 \
   if (E <= 64 * P) {                                                                                               \
-    hipLaunchKernelGGL((moe_group_topk_kernel<P>), grid, block, 0, st, logits, E, k, n_groups, keep, topi, topv);  \
+    hipLaunchKernelGGL((moe_group_topk_kernel<P, false>), grid, block, 0, st, logits, (int64_t)E, E, k, n_groups,   \
+                       keep, (const bf16_t*)nullptr, (const float*)nullptr, 1.f, topi, topv);                      \
     return (int)hipGetLastError();                                                                                 \
+  }
+  GT_CASE(1) GT_CASE(2) GT_CASE(4) GT_CASE(8)
+#undef GT_CASE
+  return -1;
+}
+
+// logits fp32 [T, E], rows row_stride apart; correction [E] in the storage type dt. Softmax scores, choice by score +
+// correction among the `keep` groups with the largest such sum; weights renormalised, times scale.
+extern "C" int areal_moe_corrected_topk(const float* logits, int64_t row_stride, int64_t T, int E, int k, int n_groups,
+                                        int keep, const void* correction, float scale, int dt, int64_t* topi, float* topv,
+                                        hipStream_t st) {
+  if (T == 0) return 0;
+  if (E < 1 || E > 64 * RT_MAX_PER_LANE || k < 1 || k > 64 || k > E || n_groups < 1 || E % n_groups != 0 || keep < 1 ||
+      keep > n_groups || !correction || row_stride < E)
+    return -1;
+  const dim3 grid((unsigned)T), block(64);
+  const bf16_t* c16 = dt == 0 ? (const bf16_t*)correction : nullptr;
+  const float* c32 = dt == 0 ? nullptr : (const float*)correction;
+#define GT_CASE(P)                                                                                                  \
+  if (E <= 64 * P) {                                                                                                \
+    hipLaunchKernelGGL((moe_group_topk_kernel<P, true>), grid, block, 0, st, logits, row_stride, E, k, n_groups,     \
+                       keep, c16, c32, scale, topi, topv);                                                          \
+    return (int)hipGetLastError();                                                                                  \
   }
   GT_CASE(1) GT_CASE(2) GT_CASE(4) GT_CASE(8)
 #undef GT_CASE
