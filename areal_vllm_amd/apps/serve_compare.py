@@ -21,6 +21,11 @@ experts, the first layer a gated MLP) is compared with the same kind of twin.
 The Gusolix design (layer norm on sublayer outputs, short convolutions ahead of every sublayer; attention inside chunks of
 positions with keys as values, attention with mixed weights beside gated linear attention, and selective scan in turn;
 gated MLP) is compared with the dense Qwen3-style twin.
+
+The Keginex design (an element-wise norm before and after every sublayer; gated delta rule with a decay per channel and
+latent attention without positions in turn; group-routed + gated shared experts, the first layer a squared-ReLU MLP; the
+middle layers run twice) is compared with the same kind of routed twin, as many layers deep as it has layer runs, and
+with a Zusotar model of its width, depth and experts.
 """
 import json
 import sys
@@ -63,6 +68,14 @@ GUSOLIX_SIZES = {
     "w1024": (1024, 6, 8, 2, 128, 512, 4, 128, 256, 16, 2048, 16, 64, 4, 4096),
     "w2048": (2048, 6, 16, 4, 128, 1024, 8, 128, 256, 16, 4096, 16, 128, 4, 8192),
     "w4096": (4096, 3, 32, 8, 128, 1024, 16, 128, 256, 32, 8192, 16, 256, 4, 14336),
+}
+# Keginex: width, layers, loop (start, stop, times), delta-rule heads / key heads / key size / value size / taps / ranks,
+# latent attention's heads / key size / value size / query and key-value latent size, experts, experts per token, groups,
+# groups kept, expert width, shared expert width
+KEGINEX_SIZES = {
+    "w1024": (1024, 4, (1, 3, 2), 8, 4, 128, 128, 4, 64, 8, 64, 64, 384, 256, 16, 2, 4, 2, 512, 512),
+    "w2048": (2048, 4, (1, 3, 2), 16, 8, 128, 128, 4, 128, 16, 128, 128, 768, 512, 32, 4, 4, 2, 768, 768),
+    "w4096": (4096, 3, (1, 2, 2), 32, 16, 128, 128, 4, 128, 32, 128, 128, 1536, 512, 64, 4, 8, 4, 1024, 1024),
 }
 VOCAB = 32768
 
@@ -147,6 +160,32 @@ def gusolix_dict(width, layers, heads, kv, dim, chunk, gheads, gdim, gvdim, gran
         ls.append({"type": kind, "mixer": json.loads(json.dumps(mixer)), "mlp": {"kind": "dense", "ff": ff}})
     return {"architecture": "Gusolix", "canon": {"taps": 4}, "embedding": {"scale": float(width) ** 0.5}, "layers": ls,
             "norm": {"eps": 1e-5}, "vocab": VOCAB, "width": width}
+
+
+def keginex_dict(width, layers, loop, heads, kv, dim, vdim, taps, rank, lheads, ldim, lvdim, q_rank, kv_rank, experts, top, groups,
+                 keep, ff, shared, unrolled=False) -> Dict[str, Any]:
+    """`unrolled`: the layer runs as layers of their own."""
+    moe = {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": shared},
+           "router": {"experts": experts, "top": top, "scale": 2.0, "groups": {"count": groups, "keep": keep}}}
+    mixers = [
+        ("channel_delta", {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": taps, "decay_rank": rank,
+                           "gate_rank": rank}),
+        ("latent_attention", {"heads": lheads, "dim": ldim, "vdim": lvdim, "q_rank": q_rank, "kv_rank": kv_rank,
+                              "scale": ldim ** -0.5}),
+    ]
+    ls = []
+    for i in range(layers):
+        kind, mixer = mixers[i % 2]
+        mlp = {"kind": "dense", "ff": 4 * width} if i == 0 else moe
+        ls.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    a, b, k = loop
+    if unrolled:
+        ls = ls[:a] + ls[a:b] * k + ls[b:]
+    d = {"architecture": "Keginex", "layers": json.loads(json.dumps(ls)), "logit_softcap": 30.0, "norm": {"eps": 1e-5},
+         "vocab": VOCAB, "width": width}
+    if not unrolled:
+        d["loop"] = {"start": a, "stop": b, "times": k}
+    return d
 
 
 def moe_twin_config(lcfg, width, layers, heads, experts, top):
@@ -272,6 +311,34 @@ def run_gusolix(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: i
     return 0
 
 
+def run_keginex(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: int, dev) -> int:
+    from ..models.config import ModelConfig
+
+    for name in sizes:
+        z = KEGINEX_SIZES[name]
+        width, heads, experts, top = z[0], z[9], z[14], z[15]
+        kcfg, flat = ModelConfig.from_hf_dict(keginex_dict(*z)), ModelConfig.from_hf_dict(keginex_dict(*z, unrolled=True))
+        tcfg = moe_twin_config(flat, width, flat.n_layers, heads, experts, top)
+        zz = list(ZUSOTAR_SIZES[name])
+        zz[1] = flat.n_layers
+        zcfg = ModelConfig.from_hf_dict(zusotar_dict(*zz))
+        row = {"design": "keginex", "size": name, "width": width, "layers": z[1], "layer_runs": flat.n_layers,
+               "delta_heads": z[3], "delta_kv_heads": z[4], "delta_dim": z[5], "delta_vdim": z[6], "taps": z[7], "rank": z[8],
+               "latent_heads": heads, "latent_dim": z[10], "q_rank": z[12], "kv_rank": z[13], "experts": experts, "top": top,
+               "groups": z[16], "groups_kept": z[17], "expert_ff": z[18], "shared_ff": z[19],
+               "twin_expert_ff": tcfg.moe_intermediate_size, "prompts": n_prompts, "prompt_len": prompt_len,
+               "new_tokens": new_tokens, "dtype": "bf16", "data": "synthetic"}
+        for label, cfg in (("keginex", kcfg), ("qwen3_moe_twin", tcfg), ("zusotar", zcfg)):
+            m = measure(cfg, n_prompts, prompt_len, new_tokens, dev)
+            row[label] = {"params_no_embedding": cfg.n_params(with_embedding=False), **{k: round(v, 1) for k, v in m.items()}}
+        row["keginex"]["params_of_all_layer_runs"] = flat.n_params(with_embedding=False)
+        for label in ("qwen3_moe_twin", "zusotar"):
+            row["prefill_ratio_" + label] = round(row["keginex"]["prefill_tok_s"] / row[label]["prefill_tok_s"], 3)
+            row["decode_ratio_" + label] = round(row["keginex"]["decode_tok_s"] / row[label]["decode_tok_s"], 3)
+        print(json.dumps(row), flush=True)
+    return 0
+
+
 def run_lufivik(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: int, dev) -> int:
     from ..models.config import ModelConfig
 
@@ -304,6 +371,8 @@ def run(sizes: List[str], n_prompts: int, prompt_len: int, new_tokens: int, devi
         return run_zusotar(sizes, n_prompts, prompt_len, new_tokens, dev)
     if design == "gusolix":
         return run_gusolix(sizes, n_prompts, prompt_len, new_tokens, dev)
+    if design == "keginex":
+        return run_keginex(sizes, n_prompts, prompt_len, new_tokens, dev)
     for name in sizes:
         width, layers, heads, kv, dim, ff, window = SIZES[name]
         kcfg = ModelConfig.from_hf_dict(kuzanex_dict(width, layers, heads, kv, dim, ff, window))

@@ -1183,7 +1183,7 @@ class HybridModelRunner(ModelRunner):
 
     # ------------------------------------------------------------------------------ decode
     def tune_decode_paths(self):
-        if self.post_add and self.device.type == "cuda":
+        if (self.post_add or self.tanh_norm) and self.device.type == "cuda":
             for b in self.buckets:
                 self._decode_gemms(b)
 
@@ -1198,8 +1198,9 @@ class HybridModelRunner(ModelRunner):
         if Bp not in self._gate_up_choice:
             by_shape: Dict[Any, List[Any]] = {}
             for blk in self.model.layers:
-                if blk.mlp is not None:
-                    by_shape.setdefault(tuple(blk.mlp.gate_up.shape), []).append(blk.mlp)
+                w = blk.mlp.gated_weight() if hasattr(blk.mlp, "gated_weight") else None
+                if w is not None:
+                    by_shape.setdefault(tuple(w.shape), []).append(blk.mlp)
             choice = {}
             for shape, mlps in by_shape.items():
                 x = torch.randn(Bp, shape[1], device=self.device, dtype=self.dtype)
@@ -1264,8 +1265,6 @@ class HybridModelRunner(ModelRunner):
         eff = torch.where(st["slots"] < 0, self._neg1, st["state_slots"])
         step = StepTensors(st["cu_rows"], st["context_lens"], 1, st["slots"], st["block_tables"], st["positions"], eff,
                            nsplit=st["nsplit"], workspace=st["ws"], positions=st["positions"])
-        if self.post_add:
+        if self.post_add or self.tanh_norm:
             step.decode_gemms = self._decode_gemms(Bp)
-        elif self.tanh_norm and self.dtype == torch.bfloat16 and self.device.type == "cuda":
-            step.decode_gemms = {}  # closing products go through the split decode GEMM; its slabs are summed by the norm
         return self._final_logits(self._run_layers(h, step), None)

@@ -754,7 +754,7 @@ class LatentAttentionMixer(nn.Module):
         if Q > 0:
             cq = lattn.latent_prep(proj, Q, R, P, self.q_norm, self.c_norm, st.positions, st.slots, cache, self.table,
                                    self.eps, self.neighbour_pairs)
-            q = F.linear(cq, self.uq).view(T, H, D + P)
+            q = decode_linear(cq, self.uq, st).view(T, H, D + P)
         else:  # the queries are the projection's leading columns, read in place
             lattn.latent_prep(proj[:, nq:], 0, R, P, None, self.c_norm, st.positions, st.slots, cache, self.table,
                               self.eps, self.neighbour_pairs)
@@ -762,8 +762,13 @@ class LatentAttentionMixer(nn.Module):
         nsplit = 1
         if st.max_q == 1 and st.nsplit > 1:  # this mixer's own share of the step's key-range splits
             nsplit = min(st.nsplit, self.decode_splits(T, self.table.shape[0] - 1))
+        if self.window <= 0 and not self.head_gate and lattn.expanded_prompts_serve(
+                T, st.cu_q.numel() - 1, st.max_q, st.block_tables.shape[1], H, D, P, V, R, hc.dtype, hc.device):
+            o = lattn.expanded_attention(q, cache, st.block_tables, st.cu_q, st.cu_k, st.max_q, self.uk, self.uv, self.scale,
+                                         self.sink)
+            return closing_linear(o.view(T, H * V), self.o, st)
         # q~_h = W_uk[h]^T q^n_h: one batched product over the heads
-        q_lat = torch.bmm(q[:, :, :D].transpose(0, 1), self.uk.view(H, D, R)).transpose(0, 1).contiguous()
+        q_lat = lattn.absorb_keys(q[:, :, :D], self.uk)
         o_lat = lattn.latent_attention(q, q_lat, cache, st.block_tables, st.cu_q, st.ctx_len, st.max_q, D, P,
                                        self.scale, self.window, self.table,
                                        gate=proj[:, nq + R + P:] if self.head_gate else None,
@@ -929,6 +934,16 @@ class SquaredReluMLP(nn.Module):
         return closing_linear(pblock.relu2_rows(F.linear(hc, self.up)), self.down, st)
 
 
+def gated_act(hc: torch.Tensor, gate_up: torch.Tensor, act: str, mode: Optional[str]) -> torch.Tensor:
+    """act(gate h) * (up h) by the kernel `mode` names (None: library product, then the activation)."""
+    if mode == "balanced":
+        return decode_gemm.dgemm_swiglu_balanced(hc, gate_up, act=act)
+    if mode == "tiled":
+        return decode_gemm.dgemm(hc, gate_up, epilogue=decode_gemm.gated_epilogue(act))
+    a = train_gemm.gate_up_act(hc, gate_up, act)  # prompt portions of many rows: one kernel
+    return a if a is not None else pblock.glu_rows(F.linear(hc, gate_up), act)
+
+
 class RoutedSwiGLUExperts(nn.Module):
     """Routed gated experts, down(silu(gate h) * (up h)), no biases: router logits W_r h + b in fp32 (on the fp32
     normed input when the caller has it), the `top` largest are chosen and weighted by the softmax over the chosen
@@ -984,9 +999,16 @@ class RoutedSwiGLUExperts(nn.Module):
         y, inv, topv, z = self._routed(hc, h32)
         sh = None
         if self.shared_down is not None:
-            a = train_gemm.gate_up_act(hc, self.shared_in, "silu")  # prompt portions of many rows: one kernel
-            sh = F.linear(a if a is not None else pblock.glu_rows(F.linear(hc, self.shared_in)), self.shared_down)
+            mode = st.decode_gemms.get(tuple(self.shared_in.shape)) if st.decode_gemms is not None else None
+            sh = decode_linear(gated_act(hc, self.shared_in, "silu", mode), self.shared_down, st)
         return tanh_norm.Routed(y, inv, topv, sh, z[:, self.E] if self.shared_gate else None)
+
+    def gated_weight(self) -> Optional[torch.Tensor]:
+        """The gate | up weight every token runs through (decode steps choose a kernel for it), or None."""
+        return self.shared_in
+
+    def gated(self, hc: torch.Tensor, mode: Optional[str]) -> torch.Tensor:
+        return gated_act(hc, self.shared_in, "silu", mode)
 
     def _routed(self, hc: torch.Tensor, h32: Optional[torch.Tensor]):
         """(expert rows in expert order, their places, fp32 weights [T, k], fp32 router product)."""
@@ -1084,6 +1106,13 @@ def closing_linear(x: torch.Tensor, weight: torch.Tensor, st: StepTensors) -> to
     serves the shape, else [T, N] in the compute dtype."""
     if st.decode_gemms is not None and decode_gemm.serves(x, weight):
         return decode_gemm.dgemm(x, weight, epilogue=decode_gemm.EPI_SLAB)
+    return F.linear(x, weight)
+
+
+def decode_linear(x: torch.Tensor, weight: torch.Tensor, st: StepTensors) -> torch.Tensor:
+    """x W^T in the compute dtype: in decode steps the decode GEMM where it serves the shape, else the library's."""
+    if st.decode_gemms is not None and decode_gemm.serves(x, weight):
+        return decode_gemm.dgemm(x, weight)
     return F.linear(x, weight)
 
 
@@ -1318,14 +1347,11 @@ class GatedMLP(nn.Module):
         mode = st.decode_gemms.get(tuple(self.gate_up.shape)) if st.decode_gemms is not None else None
         return closing_linear(self.gated(hc, mode), self.down, st)
 
+    def gated_weight(self) -> torch.Tensor:
+        return self.gate_up
+
     def gated(self, hc: torch.Tensor, mode: Optional[str]) -> torch.Tensor:
-        """act(gate h) * (up h) by the kernel `mode` names (None: library product, then the activation)."""
-        if mode == "balanced":
-            return decode_gemm.dgemm_swiglu_balanced(hc, self.gate_up, act=self.act)
-        if mode == "tiled":
-            return decode_gemm.dgemm(hc, self.gate_up, epilogue=decode_gemm.gated_epilogue(self.act))
-        a = train_gemm.gate_up_act(hc, self.gate_up, self.act)  # prompt portions of many rows: one kernel
-        return a if a is not None else pblock.glu_rows(F.linear(hc, self.gate_up), self.act)
+        return gated_act(hc, self.gate_up, self.act, mode)
 
 
 class PrePostBlock(nn.Module):

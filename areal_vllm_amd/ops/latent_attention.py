@@ -18,7 +18,9 @@ alike (a dot product does not see a permutation applied to both sides).
 
 `sink` [H]: one logit per head whose exponential counts once in the softmax denominator; it has no key and no value.
 
-GPU: ``csrc/hip/latent_attn.hip`` (one kernel for prompt portions and, with a split key range, for decoding).
+GPU: ``csrc/hip/latent_attn.hip`` (one kernel for prompt portions and, with a split key range, for decoding); long prompt
+portions of heads of 128 without a rotary part expand the context's keys and values instead (`expanded_attention`,
+``csrc/hip/flash_attn_paged.hip``).
 CPU: PyTorch formulations of the same arithmetic (fp32).
 
 Cache layout: [pages, 32, R + P], token-major.
@@ -167,6 +169,47 @@ def latent_attention(q: torch.Tensor, q_lat: torch.Tensor, cache: torch.Tensor, 
     return out.to(q.dtype)
 
 
+EXPANDED_MIN_QUERIES = 96  # queries per row from which expanding a context's keys and values is the shorter way
+EXPANDED_MAX_TOKENS = 1 << 16  # context tokens expanded at once where the portion itself is shorter than a quarter of them
+
+
+def expanded_prompts_serve(T: int, B: int, max_q: int, max_pages: int, heads: int, dim: int, rot: int, vdim: int, rank: int,
+                           dtype, device) -> bool:
+    """Whether a prefill batch goes through `expanded_attention`: bf16 heads of 128 without a rotary part on the GPU, rows
+    of many queries, contexts that are not far longer than the portions."""
+    tokens = B * max_pages * PAGE_SIZE
+    return (dim == vdim == 128 and rot == 0 and rank % 8 == 0 and dtype == torch.bfloat16
+            and torch.device(device).type == "cuda" and max_q >= EXPANDED_MIN_QUERIES and T >= EXPANDED_MIN_QUERIES * B
+            and tokens <= max(4 * T, EXPANDED_MAX_TOKENS))
+
+
+def expanded_attention(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, cu_q: torch.Tensor,
+                       cu_k: torch.Tensor, max_q: int, uk: torch.Tensor, uv: torch.Tensor, scale: float,
+                       sink: Optional[torch.Tensor]) -> torch.Tensor:
+    """Prompt portions the other way round: keys and values of the whole context are expanded from the cached latents (two
+    library products that leave keys as [token, H 128] and values as [H 128, token]) and the paged flash kernel reads them
+    where they are. Per (query, key, head) that is 2 x 128 products instead of 2 x R. q [T, H, 128] (heads contiguous), cu_k
+    int32 [B + 1] cumulative context lengths. Returns [T, H, 128]."""
+    T, H, D = q.shape
+    B, mp = block_tables.shape
+    assert L.use_hip(q) and D == 128 and q.dtype == torch.bfloat16 and q.stride(2) == 1 and q.stride(1) == D
+    assert cache.dtype == q.dtype and uk.shape == (H * D, cache.shape[2]) and uv.shape == uk.shape
+    assert cu_q.numel() == B + 1 and cu_k.numel() == B + 1 and cu_q.dtype == torch.int32 and cu_k.dtype == torch.int32
+    assert sink is None or (sink.dtype == q.dtype and sink.numel() == H and sink.is_contiguous())
+    # table entries past a row's context name no page of it: any page will do, its keys are masked
+    c = cache.index_select(0, block_tables.reshape(-1).clamp(0, cache.shape[0] - 1)).view(B * mp * PAGE_SIZE, -1)
+    n = c.shape[0]
+    k, v = torch.nn.functional.linear(c, uk), torch.nn.functional.linear(uv, c)
+    bt = torch.arange(B * mp, dtype=torch.int32, device=q.device)
+    out = torch.empty(T, H, D, dtype=q.dtype, device=q.device)
+    L.check(L.lib().areal_flash_fwd_strided(
+        L.ptr(q), L.ptr(k), L.ptr(v), L.ptr(bt), L.c_int(mp), L.ptr(out), L.ptr(cu_q), L.ptr(cu_k), L.c_int(B),
+        L.c_int(int(max_q)), L.c_int(T), L.c_int(H), L.c_int(H), L.c_int(D), L.c_int64(q.stride(0)), L.c_int64(out.stride(0)),
+        L.c_int64(PAGE_SIZE * H * D), L.c_int64(D), L.c_int64(H * D), L.c_int64(PAGE_SIZE), L.c_int64(D * n), L.c_int64(n),
+        L.c_float(scale), L.ptr(sink), L.stream_ptr()), "flash_fwd_strided")
+    return out
+
+
 EXPAND_KERNEL_MAX_ROWS = 64
 
 
@@ -183,4 +226,15 @@ def expand_values(o_lat: torch.Tensor, uv: torch.Tensor) -> torch.Tensor:
         return out
     # the right operand of a batched product is kept contiguous: transposed bf16 views of it are not safe on this platform
     w = uv.view(H, V, R).transpose(1, 2).contiguous()
-    return torch.bmm(o_lat.transpose(0, 1), w).transpose(0, 1).reshape(T, H * V)
+    out = torch.empty(T, H, V, dtype=o_lat.dtype, device=o_lat.device)
+    torch.bmm(o_lat.transpose(0, 1), w, out=out.transpose(0, 1))
+    return out.view(T, H * V)
+
+
+def absorb_keys(q: torch.Tensor, uk: torch.Tensor) -> torch.Tensor:
+    """q [T, H, D] (a view with unit column stride), uk [H D, R] -> [T, H, R]: every head's query carried into latent space
+    with its key expansion, one batched product that writes rows in place."""
+    T, H, D = q.shape
+    out = torch.empty(T, H, uk.shape[1], dtype=q.dtype, device=q.device)
+    torch.bmm(q.transpose(0, 1), uk.view(H, D, -1), out=out.transpose(0, 1))
+    return out

@@ -60,7 +60,7 @@ def embed_sinusoid(tokens: torch.Tensor, positions: torch.Tensor, embed: torch.T
     return x, (x.to(embed.dtype) if want_copy else None)
 
 
-def _launch(x, y, b: Optional[Norm], enter, nxt: Optional[Norm], want32, want_copy, dtype, out):
+def _launch(x, y, b: Optional[Norm], enter, nxt: Optional[Norm], want32, want_copy, dtype, out, store=True):
     T, W = out.shape
     f32 = dtype == torch.float32
     routed, slabs = isinstance(y, Routed), 0
@@ -91,7 +91,7 @@ def _launch(x, y, b: Optional[Norm], enter, nxt: Optional[Norm], want32, want_co
         L.ptr(r.wt) if routed else None, L.c_int(r.wt.shape[1] if routed else 0),
         L.ptr(r.y_shared) if routed else None, L.ptr(r.sg) if routed and r.y_shared is not None else None,
         L.c_int64(r.sg.stride(0) if routed and r.sg is not None else 0), *(L.ptr(t) for t in (b or (None,) * 3)), L.ptr(p),
-        L.ptr(c), L.ptr(s), *(L.ptr(t) for t in (nxt or (None,) * 3)), L.ptr(out), L.ptr(o32), L.ptr(oc), L.c_int(T),
+        L.ptr(c), L.ptr(s), *(L.ptr(t) for t in (nxt or (None,) * 3)), L.ptr(out) if store else None, L.ptr(o32), L.ptr(oc), L.c_int(T),
         L.c_int(W), L.c_int(L.dtype_flag(torch.empty(0, dtype=dtype))), L.stream_ptr()), "tanh_norm_step")
     if nxt is not None:
         return out, o32, (o32 if f32 else oc)
@@ -112,7 +112,7 @@ def norm_add(x: torch.Tensor, y, b: Optional[Norm], nxt: Optional[Norm], dtype: 
     N_nxt(x) in the compute dtype); without `nxt` the last one is x itself in the compute dtype (`want_copy`) or None."""
     assert x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous()
     if L.use_hip(x):
-        return _launch(x, y, b, None, nxt, want32, want_copy, dtype, x)
+        return _launch(x, y, b, None, nxt, want32, want_copy, dtype, x, store=y is not None)
     if y is not None:
         z = y.total() if isinstance(y, Routed) else (y.sum(0) if y.dim() == 3 else y.float())
         x = x.add_(_norm(z, b))

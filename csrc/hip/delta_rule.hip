@@ -13,7 +13,7 @@
 // `delta_scan_kernel` (decoding, short portions, large D): token by token. Columns of S do not talk to each other, so
 // eight lanes own a column (an eighth of its D numbers each, as 16-byte pieces) and a token costs two 8-lane sums, which
 // run side by side: o_t = S'^T q_t + u_t (k_t . q_t). A workgroup of four waves owns 32 columns; queries, keys and
-// factors of 8 tokens are staged ahead, one wave a token.
+// factors of up to 8 tokens are staged ahead, one wave a token.
 //
 // Prompt portions: chunks of 16 tokens. With b_t = sum_{u <= t} ln g_u (per channel, from the chunk's start):
 //
@@ -33,9 +33,17 @@ namespace {
 
 template <typename T> DEVINL float ldf(const T* p, size_t i) { return (float)p[i]; }
 
-DEVINL float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+// softplus and exp; bf16 storage: hardware exponential and logarithm (a short series where 1 + e would lose e's digits)
+template <typename T> DEVINL float softplus(float x) {
+  if (sizeof(T) == 2) {
+    const float e = __expf(-fabsf(x));
+    return fmaxf(x, 0.f) + (e < 0.0156f ? e * (1.f - e * (0.5f - 0.33333333f * e)) : __logf(1.f + e));
+  }
+  return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
+}
+// x <= 0. bf16 storage: v_exp_f32 (relative error ~1e-6, far below the storage's); fp32 storage: the library's exp
+template <typename T> DEVINL float exp_le0(float x) { return sizeof(T) == 2 ? __expf(x) : expf(x); }
 
-constexpr int TC = 8;  // tokens staged per step of the token-by-token loop
 constexpr int CT = 16;  // tokens of a chunk
 
 struct DeltaArgs {
@@ -53,120 +61,167 @@ struct DeltaArgs {
   int H, G, D, V;
 };
 
-template <typename T, int DP>
+// CG: columns a lane works on (32 apart): decoding takes two, so that twice the state is under way per wave.
+template <typename T, int DP, int TC, int CG>
 __global__ void __launch_bounds__(256) delta_scan_kernel(const DeltaArgs a) {
   constexpr int NV = DP / 32;  // 16-byte pieces of a column a lane owns: channels 32 p + 4 l8 .. + 3
+  constexpr int NQ = (DP + 63) / 64;
   __shared__ __attribute__((aligned(16))) float kqg[TC][3][DP];
   __shared__ float bet[TC], kq[TC];
   const int H = a.H, G = a.G, D = a.D, V = a.V;
   const int b = blockIdx.x, hd = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int l8 = lane & 7, col = blockIdx.z * 32 + 8 * wave + (lane >> 3), hk = hd / (H / G);
-  const bool has = col < V;
+  const int l8 = lane & 7, col = blockIdx.z * 32 * CG + 8 * wave + (lane >> 3), hk = hd / (H / G);
   const int slot = a.state_slots[b], t_lo = a.cu_q[b], t_hi = a.cu_q[b + 1];
   if (slot < 0) {
-    if (has && l8 == 0)
-      for (int t = t_lo; t < t_hi; ++t) a.obuf[((size_t)t * H + hd) * V + col] = 0.f;
+#pragma unroll
+    for (int c = 0; c < CG; ++c)
+      if (col + 32 * c < V && l8 == 0)
+        for (int t = t_lo; t < t_hi; ++t) a.obuf[((size_t)t * H + hd) * V + col + 32 * c] = 0.f;
     return;
   }
   if (t_hi <= t_lo) return;
   const T* qkv = (const T*)a.qkv;
   const bool fresh = a.first_pos[b] == 0, vec = D % 4 == 0;
-  float* Sp = a.S + (((size_t)slot * H + hd) * V + min(col, V - 1)) * D;
-  f32x4 s[NV];
+  const float decay_rate = -expf(ldf<T>((const T*)a.a_log, hd));
+  float vv[CG][TC];
+  struct Token {  // what one lane loads of one token
+    float q[NQ], k[NQ], z[NQ], b;
+  };
+  auto load = [&](Token& o, int t) {
+    const T* row = qkv + (size_t)t * a.row_stride;
 #pragma unroll
-  for (int p = 0; p < NV; ++p) {
-    const int d = 32 * p + 4 * l8;
-    s[p] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    if (!fresh && has) {
-      if (vec) {
-        if (d < D) s[p] = *reinterpret_cast<const f32x4*>(Sp + d);
-      } else {
+    for (int i = 0; i < NQ; ++i) {
+      const int d = lane + 64 * i;
+      o.q[i] = d < D ? ldf<T>(row, a.q_off + hk * D + d) : 0.f;
+      o.k[i] = d < D ? ldf<T>(row, a.k_off + hk * D + d) : 0.f;
+      o.z[i] = d < D ? a.z[(size_t)t * a.z_stride + hd * D + d] + ldf<T>((const T*)a.z_bias, hd * D + d) : 0.f;
+    }
+    o.b = ldf<T>((const T*)a.beta, (size_t)t * a.beta_stride + hd);
+  };
+  auto stage = [&](const Token& o, int tt) {
+    float qq = 0.f, kk = 0.f, qk = 0.f;
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-          if (d + e < D) s[p][e] = Sp[d + e];
+    for (int i = 0; i < NQ; ++i) {
+      qq += o.q[i] * o.q[i];
+      kk += o.k[i] * o.k[i];
+      qk += o.q[i] * o.k[i];
+    }
+    const float rq = a.q_scale / sqrtf(wave_sum(qq) + a.unit_eps), rk = 1.f / sqrtf(wave_sum(kk) + a.unit_eps);
+    const float dot = wave_sum(qk) * rq * rk;
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+      const int d = lane + 64 * i;
+      if (d < DP) {
+        kqg[tt][0][d] = o.k[i] * rk;
+        kqg[tt][1][d] = o.q[i] * rq;
+        kqg[tt][2][d] = d < D ? exp_le0<T>(decay_rate * softplus<T>(o.z[i])) : 0.f;
+      }
+    }
+    if (lane == 0) {
+      bet[tt] = 1.f / (1.f + expf(-o.b));
+      kq[tt] = dot;
+    }
+  };
+  auto load_v = [&](int tb, int nt) {
+#pragma unroll
+    for (int tt = 0; tt < TC; ++tt)
+#pragma unroll
+      for (int c = 0; c < CG; ++c)
+        vv[c][tt] = (tt < nt && col + 32 * c < V)
+                        ? ldf<T>(qkv + (size_t)(tb + tt) * a.row_stride, a.v_off + hd * V + col + 32 * c) : 0.f;
+  };
+  // the first tokens' operands are asked for ahead of the state: loads return in order, and the operands' sums and
+  // exponentials run while the state arrives
+  Token first;
+  int nt = min(TC, t_hi - t_lo);
+  if (wave < nt) load(first, t_lo + wave);
+  load_v(t_lo, nt);
+  float* const Sh = a.S + ((size_t)slot * H + hd) * V * D;
+  f32x4 s[CG][NV];
+#pragma unroll
+  for (int c = 0; c < CG; ++c) {
+    const float* Sp = Sh + (size_t)min(col + 32 * c, V - 1) * D;
+#pragma unroll
+    for (int p = 0; p < NV; ++p) {
+      const int d = 32 * p + 4 * l8;
+      s[c][p] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      if (!fresh && col + 32 * c < V) {
+        if (vec) {
+          if (d < D) s[c][p] = *reinterpret_cast<const f32x4*>(Sp + d);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (d + e < D) s[c][p][e] = Sp[d + e];
+        }
       }
     }
   }
-  const float decay_rate = -expf(ldf<T>((const T*)a.a_log, hd));
+  if (wave < nt) stage(first, wave);
   for (int tb = t_lo; tb < t_hi; tb += TC) {
-    const int nt = min(TC, t_hi - tb);
-    __syncthreads();  // the tokens before are consumed
-    for (int tt = wave; tt < nt; tt += 4) {
-      const size_t tok = (size_t)(tb + tt);
-      const T* row = qkv + tok * a.row_stride;
-      float q[(DP + 63) / 64], k[(DP + 63) / 64], qq = 0.f, kk = 0.f, qk = 0.f;
-#pragma unroll
-      for (int i = 0; i < (DP + 63) / 64; ++i) {
-        const int d = lane + 64 * i;
-        q[i] = d < D ? ldf<T>(row, a.q_off + hk * D + d) : 0.f;
-        k[i] = d < D ? ldf<T>(row, a.k_off + hk * D + d) : 0.f;
-        qq += q[i] * q[i];
-        kk += k[i] * k[i];
-        qk += q[i] * k[i];
-      }
-      const float rq = a.q_scale / sqrtf(wave_sum(qq) + a.unit_eps), rk = 1.f / sqrtf(wave_sum(kk) + a.unit_eps);
-      const float dot = wave_sum(qk) * rq * rk;
-#pragma unroll
-      for (int i = 0; i < (DP + 63) / 64; ++i) {
-        const int d = lane + 64 * i;
-        if (d < DP) {
-          kqg[tt][0][d] = k[i] * rk;
-          kqg[tt][1][d] = q[i] * rq;
-          kqg[tt][2][d] =
-              d < D ? expf(decay_rate * softplus(a.z[tok * a.z_stride + hd * D + d] + ldf<T>((const T*)a.z_bias, hd * D + d))) : 0.f;
-        }
-      }
-      if (lane == 0) {
-        bet[tt] = 1.f / (1.f + expf(-ldf<T>((const T*)a.beta, tok * a.beta_stride + hd)));
-        kq[tt] = dot;
-      }
+    nt = min(TC, t_hi - tb);
+    if (tb > t_lo) {
+      __syncthreads();  // the tokens before are consumed
+      load_v(tb, nt);
     }
-    float vv[TC];
-#pragma unroll
-    for (int tt = 0; tt < TC; ++tt)
-      vv[tt] = (tt < nt && has) ? ldf<T>(qkv + (size_t)(tb + tt) * a.row_stride, a.v_off + hd * V + col) : 0.f;
+    for (int tt = wave + (tb == t_lo ? 4 : 0); tt < nt; tt += 4) {
+      Token o;
+      load(o, tb + tt);
+      stage(o, tt);
+    }
     __syncthreads();
 #pragma unroll
     for (int tt = 0; tt < TC; ++tt) {
       if (tt < nt) {
         f32x4 k4[NV];
-        float sk = 0.f, sq = 0.f;
+        float sk[CG], sq[CG];
+#pragma unroll
+        for (int c = 0; c < CG; ++c) sk[c] = sq[c] = 0.f;
 #pragma unroll
         for (int p = 0; p < NV; ++p) {
           const int d = 32 * p + 4 * l8;
           k4[p] = *reinterpret_cast<const f32x4*>(&kqg[tt][0][d]);
           const f32x4 q4 = *reinterpret_cast<const f32x4*>(&kqg[tt][1][d]), g4 = *reinterpret_cast<const f32x4*>(&kqg[tt][2][d]);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            s[p][e] *= g4[e];
-            sk += s[p][e] * k4[p][e];
-            sq += s[p][e] * q4[e];
+          for (int c = 0; c < CG; ++c)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              s[c][p][e] *= g4[e];
+              sk[c] += s[c][p][e] * k4[p][e];
+              sq[c] += s[c][p][e] * q4[e];
+            }
+        }
+#pragma unroll
+        for (int o = 4; o > 0; o >>= 1)
+#pragma unroll
+          for (int c = 0; c < CG; ++c) {
+            sk[c] += __shfl_xor(sk[c], o, 64);
+            sq[c] += __shfl_xor(sq[c], o, 64);
           }
+#pragma unroll
+        for (int c = 0; c < CG; ++c) {
+          const float u = bet[tt] * (vv[c][tt] - sk[c]);
+#pragma unroll
+          for (int p = 0; p < NV; ++p)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) s[c][p][e] += k4[p][e] * u;
+          if (col + 32 * c < V && l8 == 0) a.obuf[((size_t)(tb + tt) * H + hd) * V + col + 32 * c] = sq[c] + u * kq[tt];
         }
-#pragma unroll
-        for (int o = 4; o > 0; o >>= 1) {
-          sk += __shfl_xor(sk, o, 64);
-          sq += __shfl_xor(sq, o, 64);
-        }
-        const float u = bet[tt] * (vv[tt] - sk);
-#pragma unroll
-        for (int p = 0; p < NV; ++p)
-#pragma unroll
-          for (int e = 0; e < 4; ++e) s[p][e] += k4[p][e] * u;
-        if (has && l8 == 0) a.obuf[((size_t)(tb + tt) * H + hd) * V + col] = sq + u * kq[tt];
       }
     }
   }
-  if (has) {
+#pragma unroll
+  for (int c = 0; c < CG; ++c) {
+    if (col + 32 * c >= V) continue;
+    float* Sp = Sh + (size_t)(col + 32 * c) * D;
 #pragma unroll
     for (int p = 0; p < NV; ++p) {
       const int d = 32 * p + 4 * l8;
       if (vec) {
-        if (d < D) *reinterpret_cast<f32x4*>(Sp + d) = s[p];
+        if (d < D) *reinterpret_cast<f32x4*>(Sp + d) = s[c][p];
       } else {
 #pragma unroll
         for (int e = 0; e < 4; ++e)
-          if (d + e < D) Sp[d + e] = s[p][e];
+          if (d + e < D) Sp[d + e] = s[c][p][e];
       }
     }
   }
@@ -176,9 +231,6 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(const DeltaArgs a) {
 // (slot, head): q~ [CT][DP], k~ [CT][DP], (k exp(b_L - b))^T [DP][CT], exp(b_L) [DP], A [CT][CT], M [CT][CT].
 DEVINL size_t chunk_slot(int t_lo, int tb, int b) { return (size_t)(t_lo / CT + b + (tb - t_lo) / CT); }
 template <int DP> constexpr size_t chunk_floats() { return 3 * CT * DP + DP + 2 * CT * CT; }
-
-// bf16 storage: v_exp_f32 (relative error ~1e-6, far below the storage's); fp32 storage: the library's exp
-template <typename T> DEVINL float exp_le0(float x) { return sizeof(T) == 2 ? __expf(x) : expf(x); }
 
 template <typename T, int DP>
 __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaArgs a) {
@@ -201,7 +253,7 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaArgs a) {
     Qr[tt * QS + d] = live ? ldf<T>(row, a.q_off + hk * D + dc) : 0.f;
     // rows past the chunk's end and padding channels do not decay
     Bs[tt * QS + d] =
-        live ? decay_rate * softplus(a.z[tok * a.z_stride + hd * D + dc] + ldf<T>((const T*)a.z_bias, hd * D + dc)) : 0.f;
+        live ? decay_rate * softplus<T>(a.z[tok * a.z_stride + hd * D + dc] + ldf<T>((const T*)a.z_bias, hd * D + dc)) : 0.f;
   }
   if (tid < CT) bet[tid] = tid < nt ? 1.f / (1.f + expf(-ldf<T>((const T*)a.beta, (size_t)(tb + tid) * a.beta_stride + hd))) : 0.f;
   __syncthreads();
@@ -433,8 +485,12 @@ extern "C" int areal_delta_scan(const void* qkv, int64_t row_stride, int q_off, 
 #undef CHUNK
     return (int)hipGetLastError();
   }
-  const dim3 grid(B, H, (V + 31) / 32);
-#define LAUNCH(TT, DPV) hipLaunchKernelGGL((delta_scan_kernel<TT, DPV>), grid, dim3(256), 0, st, a)
+  const dim3 grid(B, H, (V + 31) / 32), grid2(B, H, (V + 63) / 64);
+#define LAUNCH(TT, DPV)                                                                                   \
+  do {                                                                                                    \
+    if (max_q == 1) hipLaunchKernelGGL((delta_scan_kernel<TT, DPV, 1, 2>), grid2, dim3(256), 0, st, a);   \
+    else hipLaunchKernelGGL((delta_scan_kernel<TT, DPV, 8, 1>), grid, dim3(256), 0, st, a);               \
+  } while (0)
 #define PICK(TT)                        \
   do {                                  \
     if (D <= 32) LAUNCH(TT, 32);        \

@@ -19,7 +19,10 @@
 // p - j < window or j < keep): key tiles that no query of the workgroup can see are skipped (the tiles that hold kept
 // tokens, then the tiles from the window's start on), and the softmax weights enter O^T += V^T.P^T as the pair
 // (bf16(p), bf16(p - bf16(p))), two products, so that they carry 16 bits of mantissa instead of 8. chunk > 0 confines a
-// query to the keys of its own chunk of positions (counted from the sequence's start).
+// query to the keys of its own chunk of positions (counted from the sequence's start). `sink` (one number per query head):
+// a logit without a value that joins the softmax denominator, unscaled.
+// STR = true (with WIN): K and V are not in the cache's layout but where strides say, in tokens of 32 a page: a key's
+// channels are neighbours, and so are a page's 32 tokens of one value channel (products of a library GEMM as they come).
 //
 // Role in the reference: prefill against the radix cache inside its serving engine, and
 // flash_attn_with_kvcache at realhf/impl/model/modules/attn.py:272.
@@ -27,14 +30,18 @@
 
 // FP8: the caches hold e4m3 bytes (same layouts): a thread fetches 8 bytes per fragment and widens them to bf16 on the
 // way into LDS; everything behind the staging is the bf16 kernel.
-template <bool FP8, bool WIN = false>
+struct KVStrides {  // elements
+  int64_t k_page, k_head, k_key, v_page, v_head, v_ch;
+};
+template <bool FP8, bool WIN = false, bool STR = false>
 __global__ __launch_bounds__(256, 2) void flash_fwd_paged_kernel(
     const bf16_t* __restrict__ q, const void* __restrict__ kcache, const void* __restrict__ vcache,
     const int* __restrict__ block_tables, int max_pages, bf16_t* __restrict__ o, float* __restrict__ lse,
     const int* __restrict__ cu_q, const int* __restrict__ cu_k, int64_t q_stride, int64_t o_stride, int Hq, int Hkv,
     int nbatch, int total_q, float scale_log2, int causal, int window = 0, int keep = 0,
     const bf16_t* __restrict__ r1 = nullptr, const bf16_t* __restrict__ r2 = nullptr,
-    const bf16_t* __restrict__ gate = nullptr, int64_t gate_stride = 0, int chunk = 0) {
+    const bf16_t* __restrict__ gate = nullptr, int64_t gate_stride = 0, int chunk = 0,
+    const bf16_t* __restrict__ sink = nullptr, const KVStrides str = KVStrides{}) {
   constexpr int D = 128;
   __shared__ __attribute__((aligned(16))) char smem[2 * 64 * 256];
   char* ks = smem;             // K tile  [64 keys][256 B], 16-byte chunks swizzled (flash_tiles.hpp)
@@ -76,6 +83,10 @@ __global__ __launch_bounds__(256, 2) void flash_fwd_paged_kernel(
 #pragma unroll
     for (int j = 0; j < 16; ++j) oacc[i][j] = 0.f;
   float m = -INFINITY, l = 0.f;
+  if (WIN && sink) {  // the two halves of a query's lanes share m; their l are added up at the end
+    m = bf2f(sink[head]) * 1.4426950408889634f;
+    l = hf == 0 ? 1.f : 0.f;
+  }
   // WIN with r1 / r2: r1_h ln(1 + r2_h (i - j)) is taken off the scaled score (in log2 units: r1_h log2(1 + r2_h (i - j)))
   const bool biased = WIN && r1 != nullptr;
   const float b1 = biased ? bf2f(r1[head]) : 0.f, b2 = biased ? bf2f(r2[head]) : 0.f;
@@ -115,12 +126,14 @@ __global__ __launch_bounds__(256, 2) void flash_fwd_paged_kernel(
       int key = t * 64 + lrow + 16 * i;
       key = key < k_len ? key : k_len - 1;
       const int page = bt[key >> 5];
-      kreg[i] = ld8_cache<FP8>(kcache, (((size_t)page * Hkv + kvh) * 32 + (key & 31)) * D + lch * 8);
+      kreg[i] = ld8_cache<FP8>(kcache, (STR ? page * str.k_page + kvh * str.k_head + (key & 31) * str.k_key
+                                            : (((size_t)page * Hkv + kvh) * 32 + (key & 31)) * D) + lch * 8);
       const int id = tid + 256 * i;
       const int half = id >> 9, ch = (id >> 2) & 127, c16 = id & 3;
       int pg = t * 2 + half;
       pg = pg < last_page ? pg : last_page;
-      vreg[i] = ld8_cache<FP8>(vcache, (((size_t)bt[pg] * Hkv + kvh) * D + ch) * 32 + c16 * 8);
+      vreg[i] = ld8_cache<FP8>(vcache, (STR ? bt[pg] * str.v_page + kvh * str.v_head + ch * str.v_ch
+                                            : (((size_t)bt[pg] * Hkv + kvh) * D + ch) * 32) + c16 * 8);
     }
   };
   auto store_tile = [&](int t) {
@@ -308,5 +321,27 @@ extern "C" int areal_flash_fwd_paged_window(const void* q, const void* kcache, c
                      block_tables, max_pages, (bf16_t*)o, (float*)nullptr, cu_q, cu_k, q_stride, o_stride, Hq, Hkv, B,
                      total_q, scale_log2, 1, window, keep, (const bf16_t*)r1, (const bf16_t*)r2, (const bf16_t*)gate,
                      gate_stride, chunk);
+  return (int)hipGetLastError();
+}
+
+// Prompt portions against keys and values at given strides (multiples of 8 elements; see KVStrides), causal, with one sink
+// logit per head or null; softmax weights at 16 bits of mantissa.
+extern "C" int areal_flash_fwd_strided(const void* q, const void* k, const void* v, const int* block_tables, int max_pages,
+                                       void* o, const int* cu_q, const int* cu_k, int B, int max_q, int total_q, int Hq,
+                                       int Hkv, int D, int64_t q_stride, int64_t o_stride, int64_t k_page, int64_t k_head,
+                                       int64_t k_key, int64_t v_page, int64_t v_head, int64_t v_ch, float softmax_scale,
+                                       const void* sink, hipStream_t st) {
+  if (B == 0 || max_q == 0) return 0;
+  if (D != 128) return -1;
+  if (Hq % Hkv != 0) return -2;
+  if ((q_stride | o_stride | k_page | k_head | k_key | v_page | v_head | v_ch) % 8 != 0) return -3;
+  if (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)o) % 16 != 0) return -4;
+  const float scale_log2 = softmax_scale * 1.4426950408889634f;
+  const int n_g_pad = (Hkv * B + 7) & ~7;
+  dim3 grid((unsigned)(((max_q + 127) / 128) * (Hq / Hkv) * n_g_pad)), block(256);
+  hipLaunchKernelGGL((flash_fwd_paged_kernel<false, true, true>), grid, block, 0, st, (const bf16_t*)q, k, v, block_tables,
+                     max_pages, (bf16_t*)o, (float*)nullptr, cu_q, cu_k, q_stride, o_stride, Hq, Hkv, B, total_q,
+                     scale_log2, 1, 0, 0, (const bf16_t*)nullptr, (const bf16_t*)nullptr, (const bf16_t*)nullptr,
+                     (int64_t)0, 0, (const bf16_t*)sink, KVStrides{k_page, k_head, k_key, v_page, v_head, v_ch});
   return (int)hipGetLastError();
 }

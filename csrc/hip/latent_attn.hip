@@ -589,7 +589,7 @@ __global__ void __launch_bounds__(128) latent_attn_combine_kernel(const float* _
 
 // Values of the heads from their attended latents: out[t, h V + v] = sum_r o_lat[t, h, r] uv[h V + v, r], for batches of
 // few tokens (a decode step streams uv once). A wave owns 16 tokens x 16 value columns of one head; both operands lie along
-// r, so the matrix cores take them straight from memory (16-byte loads, four steps of 32 in flight).
+// r, so the matrix cores take them straight from memory (16-byte loads, sixteen steps of 32 in flight).
 __global__ void __launch_bounds__(256) latent_expand_kernel(const bf16_t* __restrict__ o_lat, const bf16_t* __restrict__ uv,
                                                             bf16_t* __restrict__ out, int T, int H, int V, int R) {
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, quad = lane >> 4;
@@ -598,7 +598,7 @@ __global__ void __launch_bounds__(256) latent_expand_kernel(const bf16_t* __rest
   const bf16_t* ap = o_lat + ((size_t)min(t0 + r16, T - 1) * H + h) * R + 8 * quad;
   const bf16_t* bp = uv + ((size_t)h * V + min(v0 + r16, V - 1)) * R + 8 * quad;
   f32x4 c = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll 16
   for (int r = 0; r < R; r += 32) c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ld8(ap + r), ld8(bp + r), c, 0, 0, 0);
   if (v0 + r16 >= V) return;
 #pragma unroll
