@@ -1937,8 +1937,8 @@ class HybridDecoder(nn.Module):
                     p.data.copy_(torch.randn(p.shape, generator=g) / (p.shape[1] ** 0.5))
                 elif leaf == "sink":
                     p.data.copy_(torch.randn(p.shape, generator=g))
-                elif leaf == "correction":
-                    p.data.copy_(0.1 * torch.randn(p.shape, generator=g))
+                elif leaf == "correction":  # moves close choices, leaves the experts evenly used
+                    p.data.copy_(0.3 / p.numel() * torch.randn(p.shape, generator=g))
                 elif leaf == "b":
                     p.data.copy_(0.1 * torch.randn(p.shape, generator=g))
                 elif leaf == "loop_step":

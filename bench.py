@@ -112,7 +112,8 @@ def parse_args():
                         "attention, routed + shared experts) or zusotar (depth-averaged layers of window, latent and "
                         "gated linear attention, group-routed + shared experts) beside a Qwen3-MoE-style twin, gusolix "
                         "(chunked attention, mixed-weight attention beside gated linear attention, selective scan) "
-                        "beside the Qwen3-style twin")
+                        "beside the Qwen3-style twin, keginex (per-channel delta rule, latent attention without "
+                        "positions, looped passes) beside a Qwen3-MoE-style twin and zusotar")
     a = p.parse_args()
     if a.seq_len:
         a.max_new_tokens = a.seq_len - a.prompt_len_max
